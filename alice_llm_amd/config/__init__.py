@@ -6,6 +6,7 @@ from .novotar import NovotarConfig
 from .telulorn import TelulornConfig
 from .pefitar import PefitarConfig
 from .vifirax import VifiraxConfig
+from .kabapel import KabapelConfig
 from . import presets
 
 register_architecture("Gemma2ForCausalLM", Gemma2Config, model_type="gemma2")
@@ -13,3 +14,4 @@ register_architecture("Novotar", NovotarConfig)
 register_architecture("Telulorn", TelulornConfig)
 register_architecture("Pefitar", PefitarConfig)
 register_architecture("Vifirax", VifiraxConfig)
+register_architecture("Kabapel", KabapelConfig)

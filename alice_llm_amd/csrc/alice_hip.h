@@ -4,7 +4,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 
-#define ALICE_ABI_VERSION 12
+#define ALICE_ABI_VERSION 13
 
 #define ALICE_EPI_NONE 0
 #define ALICE_EPI_GEGLU 1     // W = [gate; up] stacked; epi_param 0: y = gelu_tanh(gate x) * (up x); epi_param = limit > 0:
@@ -12,8 +12,9 @@
                               // ALICE_GATED_SILU: y = (gate x) * sigmoid(gate x) * (up x)
 #define ALICE_GATED_SILU (-1.0f)
 #define ALICE_EPI_SOFTCAP 2   // one function of each output element, its form picked by epi_param: cap > 0: y = cap * tanh(y / cap);
-                              // ALICE_UNARY_RELU2: y = max(y, 0)^2
+                              // ALICE_UNARY_RELU2: y = max(y, 0)^2; ALICE_UNARY_SILU: y * sigmoid(y)
 #define ALICE_UNARY_RELU2 (-1.0f)
+#define ALICE_UNARY_SILU (-2.0f)
 #define ALICE_EPI_ROPE 3      // internal: rotation and cache write (alice_linear_rope_cache)
 
 #define ALICE_LAYOUT_ROW 0     // row-major [N, K]
@@ -47,7 +48,7 @@ int alice_embed(const int* tokens, const void* table, int table_dtype, int table
                 int T, int H, int V, float scale, hipStream_t stream);
 
 int alice_add_norm(float* resid, const float* branch, int n_partials, long partial_stride,
-                   const void* w_post, const void* w_pre, int w_dtype, void* out, int out_dtype,
+                   const void* w_post, const void* w_pre, const void* b_pre, int w_dtype, void* out, int out_dtype,
                    const int* rows, int T, int H, float eps_post, float eps_pre, float off_post,
                    float off_pre, int full_precision, int out_layout, hipStream_t stream);
 
@@ -190,8 +191,18 @@ int alice_matrix_recurrence(const float* q, int q_w, int q_col, const float* k, 
 int alice_matrix_recurrence_columns(int n_seqs, int H, int d, int dv);
 // Rows of `width` in `parts` equal parts, each RMS-normed and multiplied by a weight (w_shared: of a part's length);
 // gate_act 1: times silu(gate) before the norm, 2: times sigmoid(gate) after it, 0: no gate.
-int alice_norm_gate(const float* x, int width, int parts, const float* gate, int gate_w, int gate_col, int gate_act,
+int alice_norm_gate(const float* x, int width, int parts, const void* gate, int gate_dtype, int gate_w, int gate_col, int gate_act,
                     const float* w, int w_shared, float eps, void* out, int out_dtype, int T, hipStream_t stream);
+// Linear attention with a constant decay a head (lightning.hip): rows [T, row_w] with q, k and v (heads side by side) at
+// q_col, k_col and v_col, through silu on the way in with `act`; powers: float32 [H, ALICE_LIGHTNING_CHUNK + 1], the
+// decays' powers 0, 1, ...; S: float32 [n_slots, H, d, dv]; out: float32 [T, H dv].  chunked 0: token by token, the state
+// in registers; 1: by chunks on the matrix cores, with states: float32 [alice_lightning_chunks(T, n_seqs), H, d, dv].
+#define ALICE_LIGHTNING_CHUNK 64
+#define ALICE_LIGHTNING_MAX_KEY_DIM 256
+long alice_lightning_chunks(int T, int n_seqs);
+int alice_lightning(const void* rows, int rows_dtype, int row_w, int q_col, int k_col, int v_col, int act, const float* powers,
+                    float* out, float* states, const int* cu_seqlens, const int* slots, float* S, int T, int n_seqs,
+                    int n_slots, int H, int d, int dv, int chunked, hipStream_t stream);
 // Router of a mixture of experts: dense weights [T, E] from logits [T, E] (+ bias): softmax over the `top` largest,
 // zero elsewhere; and y[t, e F + j] = x[t, e F + j] w[t, e].  See experts.hip.
 int alice_route_topk(const float* z, const float* bias, float* w, int T, int E, int top, hipStream_t stream);
@@ -199,7 +210,17 @@ int alice_scale_columns(const void* x, int x_dtype, const float* w, void* y, int
 // The routed feed-forward by grouped products over (token, expert) pairs in expert order (bfloat16, fragment layouts).
 long alice_expert_rows(int T, int E, int top);
 int alice_expert_products(const void* x, const float* weights, const void* gate_up, const void* down, float* y, int* ints,
-                          void* mid, float* rows, int T, int W, int F, int E, int top, float epi, hipStream_t stream);
+                          void* mid, float* rows, int T, int W, int F, int E, int top, float epi, const float* side, const float* shared,
+                          int n_shared, hipStream_t stream);
+// A router that scores all n = experts + identity outputs by a softmax: z [T, z_w] float32; choice = score + correction [n]; of
+// `groups` equal runs of neighbours the `keep` with the largest choice stay, of those the `top` largest choices serve the
+// token, weighted by score / (sum of the chosen scores + 1e-20).  w [T, experts] (zero: not chosen); side [T, 2]: the weight
+// of the identity outputs together, and with has_shared sigmoid(z[t, n]) (else 0).
+int alice_route_scored(const float* z, int z_w, const float* correction, float* w, float* side, int T, int experts, int identity,
+                       int top, int groups, int keep, int has_shared, hipStream_t stream);
+// y[t] = sum of n_base partial rows base[s][t] + side[t][0] x[t] + side[t][1] (sum of n_shared partial rows shared[s][t]).
+int alice_expert_combine(const float* base, int n_base, const void* x, int x_dtype, const float* side, const float* shared, int n_shared,
+                         float* y, int T, int W, hipStream_t stream);
 // Latent attention (latent.hip): the cache row of a token is [latent (kv_rank) | rotated key part (rot_dim)], one kv head,
 // row-major pages; the first kv_rank dimensions of a row are also its value.
 int alice_latent_prepare(const float* rows, int row_width, int q_rank, int kv_rank, int rot_dim, const float* w_q,

@@ -120,8 +120,9 @@ __device__ __forceinline__ float gated_act(float g, float u, float limit, bool f
   return gelu_tanh_f(g, full) * u;
 }
 // The function of one output element, the epilogue ALICE_EPI_SOFTCAP.  Its parameter picks the form: a positive cap
-// gives cap * tanh(v / cap); a negative one (ALICE_UNARY_RELU2) the square of max(v, 0).
+// gives cap * tanh(v / cap); ALICE_UNARY_RELU2 (-1) the square of max(v, 0); ALICE_UNARY_SILU (-2) v * sigmoid(v).
 __device__ __forceinline__ float unary_act(float v, float p, bool full) {
+  if (p < -1.5f) return v / (1.f + (full ? expf(-v) : __expf(-v)));
   if (p < 0.f) {
     const float r = fmaxf(v, 0.f);
     return r * r;

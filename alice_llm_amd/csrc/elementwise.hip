@@ -65,11 +65,13 @@ __device__ __forceinline__ size_t out_index(int layout, int r, int i, int H) {
 //   x   = resid + b, written back to resid            (only when branch is given)
 //   out = x * rsqrt(mean(x^2) + eps_pre) * (off_pre + w_pre)   (only when out is given;
 //         out = x when w_pre is absent)
+// With LN the norm in front of the next part takes the row's mean off and has a bias:
+//   out = (x - mean(x)) * rsqrt(mean((x - mean(x))^2) + eps_pre) * (off_pre + w_pre) + b_pre
 // All sums are 32-bit; FULL selects 1/sqrtf over the fast reciprocal square root.
-template <typename TW, typename TO, bool FULL>
+template <typename TW, typename TO, bool FULL, bool LN>
 __global__ void add_norm_kernel(float* __restrict__ resid, const float* __restrict__ branch,
                                 int n_partials, size_t partial_stride,
-                                const TW* __restrict__ w_post, const TW* __restrict__ w_pre,
+                                const TW* __restrict__ w_post, const TW* __restrict__ w_pre, const TW* __restrict__ b_pre,
                                 TO* __restrict__ out, const int* __restrict__ rows, int H,
                                 float eps_post, float eps_pre, float off_post, float off_pre, int out_layout) {
   __shared__ float red[17];
@@ -111,12 +113,22 @@ __global__ void add_norm_kernel(float* __restrict__ resid, const float* __restri
     for (int i = threadIdx.x; i < H; i += blockDim.x) store_f32(o, out_index(out_layout, r, i, H), x[i]);
     return;
   }
+  // Each thread re-reads the elements it wrote itself above, so no barrier is needed.
+  float mu = 0.f;
+  if (LN) {
+    float sum = 0.f;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) sum += x[i];
+    mu = block_sum(sum, red) / (float)H;
+    ss_x = 0.f;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) { const float c = x[i] - mu; ss_x += c * c; }
+  }
   ss_x = block_sum(ss_x, red);
   float mean = ss_x / (float)H;
   float inv = FULL ? 1.f / sqrtf(mean + eps_pre) : rsqrtf(mean + eps_pre);
-  // Each thread re-reads the elements it wrote itself above, so no barrier is needed.
-  for (int i = threadIdx.x; i < H; i += blockDim.x)
-    store_f32(o, out_index(out_layout, r, i, H), x[i] * inv * (off_pre + load_f32(w_pre, i)));
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float y = (LN ? x[i] - mu : x[i]) * inv * (off_pre + load_f32(w_pre, i));
+    store_f32(o, out_index(out_layout, r, i, H), LN ? y + load_f32(b_pre, i) : y);
+  }
 }
 
 // The same operation with a row held in registers (EPT elements per thread): every operand is read once
@@ -141,10 +153,10 @@ __device__ __forceinline__ void load_partials(float (&t)[EPT][CMAX], const float
     for (int p = 0; p < C; ++p) t[j][p] = row[idx[j] + (size_t)min(p0 + p, n_partials - 1) * partial_stride];
 }
 
-template <typename TW, typename TO, bool FULL, int EPT>
+template <typename TW, typename TO, bool FULL, bool LN, int EPT>
 __global__ void add_norm_regs_kernel(float* __restrict__ resid, const float* __restrict__ branch,
                                      int n_partials, size_t partial_stride,
-                                     const TW* __restrict__ w_post, const TW* __restrict__ w_pre,
+                                     const TW* __restrict__ w_post, const TW* __restrict__ w_pre, const TW* __restrict__ b_pre,
                                      TO* __restrict__ out, const int* __restrict__ rows, int H,
                                      float eps_post, float eps_pre, float off_post, float off_pre, int out_layout) {
   typedef typename raw_of<TW>::type RW;
@@ -162,13 +174,17 @@ __global__ void add_norm_regs_kernel(float* __restrict__ resid, const float* __r
   // ---- loads
   constexpr int CMAX = EPT >= 8 ? 4 : 8;        // partial sums in flight per element (registers)
   float xv[EPT], bv[EPT], t[EPT][CMAX];
-  RW wq_raw[EPT], wp_raw[EPT];
+  RW wq_raw[EPT], wp_raw[EPT], bq_raw[EPT];
   const int chunk = n_partials <= 1 ? 1 : (n_partials <= 2 ? 2 : (n_partials <= 4 ? 4 : CMAX));
 #pragma unroll
   for (int j = 0; j < EPT; ++j) xv[j] = resid[src + idx[j]];
   if (w_pre) {
 #pragma unroll
     for (int j = 0; j < EPT; ++j) wq_raw[j] = reinterpret_cast<const RW*>(w_pre)[idx[j]];
+    if (LN) {
+#pragma unroll
+      for (int j = 0; j < EPT; ++j) bq_raw[j] = reinterpret_cast<const RW*>(b_pre)[idx[j]];
+    }
   }
   if (branch) {
     if (w_post) {
@@ -218,6 +234,14 @@ __global__ void add_norm_regs_kernel(float* __restrict__ resid, const float* __r
   TO* o = out;
   float inv = 1.f;
   if (w_pre) {
+    if (LN) {
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < EPT; ++j) sum += xv[j];            // elements beyond H are zero
+      const float mu = block_sum(sum, red) / (float)H;
+#pragma unroll
+      for (int j = 0; j < EPT; ++j) xv[j] = in_row[j] ? xv[j] - mu : 0.f;
+    }
     float ss = 0.f;
 #pragma unroll
     for (int j = 0; j < EPT; ++j) ss += xv[j] * xv[j];      // elements beyond H are zero
@@ -226,8 +250,12 @@ __global__ void add_norm_regs_kernel(float* __restrict__ resid, const float* __r
     inv = FULL ? 1.f / sqrtf(mean + eps_pre) : rsqrtf(mean + eps_pre);
   }
 #pragma unroll
-  for (int j = 0; j < EPT; ++j)
-    if (in_row[j]) store_f32(o, out_index(out_layout, r, idx[j], H), w_pre ? xv[j] * inv * (off_pre + wq[j]) : xv[j]);
+  for (int j = 0; j < EPT; ++j) {
+    if (!in_row[j]) continue;
+    float y = w_pre ? xv[j] * inv * (off_pre + wq[j]) : xv[j];
+    if (LN) y += raw_to_f32(bq_raw[j]);
+    store_f32(o, out_index(out_layout, r, idx[j], H), y);
+  }
 }
 
 // The same operation for many rows (prompts): one wave per row, four rows a block, four consecutive
@@ -241,14 +269,15 @@ template <> __device__ __forceinline__ float4 load4_f32<bf16_t>(const bf16_t* p,
   return float4{bf16_bits_to_f32(v.x & 0xffffu), bf16_bits_to_f32(v.x >> 16), bf16_bits_to_f32(v.y & 0xffffu), bf16_bits_to_f32(v.y >> 16)};
 }
 
-template <typename TW, typename TO, bool FULL, int K4, int WPR>
+template <typename TW, typename TO, bool FULL, bool LN, int K4, int WPR>
 __global__ __launch_bounds__(256) void add_norm_rows_kernel(float* __restrict__ resid, const float* __restrict__ branch,
                                                             int n_partials, size_t partial_stride,
                                                             const TW* __restrict__ w_post, const TW* __restrict__ w_pre,
+                                                            const TW* __restrict__ b_pre,
                                                             TO* __restrict__ out, int T, int H,
                                                             float eps_post, float eps_pre, float off_post, float off_pre,
                                                             int out_layout) {
-  __shared__ float red[2][4];
+  __shared__ float red[LN ? 3 : 2][4];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, part = wave % WPR;
   const int r_own = blockIdx.x * (4 / WPR) + wave / WPR;
   if (WPR == 1 && r_own >= T) return;
@@ -318,6 +347,15 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(float* __restrict__ 
   if (!out) return;
   float inv = 1.f;
   if (w_pre) {
+    if (LN) {
+      float sum = 0.f;
+#pragma unroll
+      for (int k = 0; k < K4; ++k) sum += (xv[k].x + xv[k].y) + (xv[k].z + xv[k].w);
+      const float mu = row_sum(sum, LN ? 2 : 0) / (float)H;
+#pragma unroll
+      for (int k = 0; k < K4; ++k)
+        if (ok[k]) { xv[k].x -= mu; xv[k].y -= mu; xv[k].z -= mu; xv[k].w -= mu; }
+    }
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < K4; ++k) ss += xv[k].x * xv[k].x + xv[k].y * xv[k].y + xv[k].z * xv[k].z + xv[k].w * xv[k].w;
@@ -332,6 +370,10 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(float* __restrict__ 
     if (w_pre) {
       const float4 w = load4_f32<TW>(w_pre, e[k]);
       o = float4{xv[k].x * inv * (off_pre + w.x), xv[k].y * inv * (off_pre + w.y), xv[k].z * inv * (off_pre + w.z), xv[k].w * inv * (off_pre + w.w)};
+      if (LN) {
+        const float4 b = load4_f32<TW>(b_pre, e[k]);
+        o = float4{o.x + b.x, o.y + b.y, o.z + b.z, o.w + b.w};
+      }
     }
     const size_t at = out_index(out_layout, r, e[k], H);     // four consecutive elements are neighbours in both layouts
     if constexpr (sizeof(TO) == 4) {
@@ -343,12 +385,13 @@ __global__ __launch_bounds__(256) void add_norm_rows_kernel(float* __restrict__ 
 }
 
 extern "C" int alice_add_norm(float* resid, const float* branch, int n_partials, long partial_stride,
-                              const void* w_post, const void* w_pre, int w_dtype, void* out, int out_dtype,
+                              const void* w_post, const void* w_pre, const void* b_pre, int w_dtype, void* out, int out_dtype,
                               const int* rows, int T, int H, float eps_post, float eps_pre,
                               float off_post, float off_pre, int full_precision, int out_layout, hipStream_t stream) {
   ALICE_CHECK(T >= 0 && H > 0, "add_norm: bad sizes T=%d H=%d", T, H);
   ALICE_CHECK(resid != nullptr, "add_norm: the residual stream is missing");
   ALICE_CHECK(dtype_ok(w_dtype) && dtype_ok(out_dtype), "add_norm: unknown dtype");
+  ALICE_CHECK(!b_pre || (w_pre && w_dtype == DT_F32), "add_norm: a norm with a bias has 32-bit weights");
   ALICE_CHECK(!(rows && branch), "add_norm: a row gather cannot be combined with a residual add");
   ALICE_CHECK(n_partials >= 1 && n_partials <= 64, "add_norm: n_partials %d out of range", n_partials);
   ALICE_CHECK(out_layout == 0 || (out_layout == 1 && out && out_dtype == DT_BF16 && H % 32 == 0),
@@ -362,32 +405,39 @@ extern "C" int alice_add_norm(float* resid, const float* branch, int n_partials,
     ept = H <= 256 ? 1 : (H <= 512 ? 2 : (H <= 4096 ? 4 : 8));
     threads = ceil_div(ceil_div(H, ept), 64) * 64;
   }
-#define ARGS resid, branch, n_partials, (size_t)partial_stride, (const TW*)w_post, (const TW*)w_pre, (TO*)out, rows, H, \
+#define ARGS resid, branch, n_partials, (size_t)partial_stride, (const TW*)w_post, (const TW*)w_pre, (const TW*)b_pre, (TO*)out, rows, H, \
              eps_post, eps_pre, off_post, off_pre, out_layout
   // Many rows, no gather: a wave per row (two from 4,097 elements on).  From 320 rows: below, a block per row
   // fills more of the chip (measured at 2,304 and 3,584 elements: up to 256 rows the block-per-row kernel is 0.5
   // to 6 us faster, from 384 rows on the wave-per-row kernel is, by half at 2,048 rows).
-  const bool aligned = (((uintptr_t)resid | (uintptr_t)branch | (uintptr_t)out | (uintptr_t)w_post | (uintptr_t)w_pre) & 15) == 0;
+  const bool aligned = (((uintptr_t)resid | (uintptr_t)branch | (uintptr_t)out | (uintptr_t)w_post | (uintptr_t)w_pre | (uintptr_t)b_pre) & 15) == 0;
   const int k4 = (!rows && aligned && T >= 320 && H % 4 == 0 && H >= 256 && H <= 8192 && (partial_stride % 4 == 0 || !branch)) ? ceil_div(H, 256) : 0;
-#define ROWS(TW, TO, FULL, K4, WPR) add_norm_rows_kernel<TW, TO, FULL, K4, WPR><<<ceil_div(T, 4 / WPR), 256, 0, stream>>>(     \
-    resid, branch, n_partials, (size_t)partial_stride, (const TW*)w_post, (const TW*)w_pre, (TO*)out, T, H, eps_post, eps_pre, \
-    off_post, off_pre, out_layout)
-#define LAUNCH(TW, TO, FULL)                                                                         \
+#define ROWS(TW, TO, FULL, LN, K4, WPR) add_norm_rows_kernel<TW, TO, FULL, LN, K4, WPR><<<ceil_div(T, 4 / WPR), 256, 0, stream>>>( \
+    resid, branch, n_partials, (size_t)partial_stride, (const TW*)w_post, (const TW*)w_pre, (const TW*)b_pre, (TO*)out, T, H,   \
+    eps_post, eps_pre, off_post, off_pre, out_layout)
+#define LAUNCH(TW, TO, FULL, LN)                                                                     \
   do {                                                                                               \
-    if (k4 > 0 && k4 <= 4) ROWS(TW, TO, FULL, 4, 1);                                                 \
-    else if (k4 > 4 && k4 <= 9) ROWS(TW, TO, FULL, 9, 1);                                            \
-    else if (k4 > 9 && k4 <= 16) ROWS(TW, TO, FULL, 16, 1);                                          \
-    else if (k4 > 16 && k4 <= 18) ROWS(TW, TO, FULL, 9, 2);                                          \
-    else if (k4 > 18) ROWS(TW, TO, FULL, 16, 2);                                                     \
-    else if (ept == 1) add_norm_regs_kernel<TW, TO, FULL, 1><<<T, threads, 0, stream>>>(ARGS);            \
-    else if (ept == 2) add_norm_regs_kernel<TW, TO, FULL, 2><<<T, threads, 0, stream>>>(ARGS);       \
-    else if (ept == 4) add_norm_regs_kernel<TW, TO, FULL, 4><<<T, threads, 0, stream>>>(ARGS);       \
-    else if (ept == 8) add_norm_regs_kernel<TW, TO, FULL, 8><<<T, threads, 0, stream>>>(ARGS);       \
-    else add_norm_kernel<TW, TO, FULL><<<T, threads, 0, stream>>>(ARGS);                             \
+    if (k4 > 0 && k4 <= 4) ROWS(TW, TO, FULL, LN, 4, 1);                                             \
+    else if (k4 > 4 && k4 <= 9) ROWS(TW, TO, FULL, LN, 9, 1);                                        \
+    else if (k4 > 9 && k4 <= 16) ROWS(TW, TO, FULL, LN, 16, 1);                                      \
+    else if (k4 > 16 && k4 <= 18) ROWS(TW, TO, FULL, LN, 9, 2);                                      \
+    else if (k4 > 18) ROWS(TW, TO, FULL, LN, 16, 2);                                                 \
+    else if (ept == 1) add_norm_regs_kernel<TW, TO, FULL, LN, 1><<<T, threads, 0, stream>>>(ARGS);   \
+    else if (ept == 2) add_norm_regs_kernel<TW, TO, FULL, LN, 2><<<T, threads, 0, stream>>>(ARGS);   \
+    else if (ept == 4) add_norm_regs_kernel<TW, TO, FULL, LN, 4><<<T, threads, 0, stream>>>(ARGS);   \
+    else if (ept == 8) add_norm_regs_kernel<TW, TO, FULL, LN, 8><<<T, threads, 0, stream>>>(ARGS);   \
+    else add_norm_kernel<TW, TO, FULL, LN><<<T, threads, 0, stream>>>(ARGS);                         \
   } while (0)
-  DISPATCH_DTYPE(w_dtype, TW, DISPATCH_DTYPE(out_dtype, TO, {
-    if (full_precision) LAUNCH(TW, TO, true); else LAUNCH(TW, TO, false);
-  }));
+  if (b_pre) {
+    using TW = float;
+    DISPATCH_DTYPE(out_dtype, TO, {
+      if (full_precision) LAUNCH(float, TO, true, true); else LAUNCH(float, TO, false, true);
+    });
+  } else {
+    DISPATCH_DTYPE(w_dtype, TW, DISPATCH_DTYPE(out_dtype, TO, {
+      if (full_precision) LAUNCH(TW, TO, true, false); else LAUNCH(TW, TO, false, false);
+    }));
+  }
 #undef LAUNCH
 #undef ROWS
 #undef ARGS

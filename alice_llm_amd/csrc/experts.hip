@@ -4,6 +4,11 @@
 // it picks the `top` largest (of equal logits the lower index), takes the softmax over the picked logits only, and
 // writes a dense row of weights [E]: the picked experts' weights, zero elsewhere.  All in 32-bit.
 //
+// route_scored_kernel: a router whose scores are a softmax over all its outputs, the last of which may be identity experts
+// (they give the token's own input back and have no matrices).  A correction is added to the scores for the choice
+// only; the outputs form equal groups of neighbours, and only experts of the groups with the largest choice in them can
+// be chosen; the chosen experts' scores, divided by their sum, are the weights.  A wave per token, all in 32-bit.
+//
 // scale_columns_kernel: y[t, e F + j] = x[t, e F + j] * w[t, e] for rows made of E parts of F columns: the experts'
 // middle activations side by side, each multiplied by its expert's weight of that token (a zero for an expert that
 // the token does not use), so that one down projection over all parts gives the weighted sum of the experts.
@@ -54,6 +59,91 @@ __global__ __launch_bounds__(64) void route_kernel(const float* __restrict__ z, 
   }
   const float inv = sum > 0.f ? 1.f / sum : 0.f;
   for (int e = lane; e < E; e += 64) w[(size_t)t * E + e] = ws[e] * inv;
+}
+
+// The largest of the wave's (value, index) pairs, of equal values the lower index; every lane gets it.
+__device__ __forceinline__ void wave_argmax(float& best, int& at) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ob = __shfl_xor(best, o, 64);
+    const int oa = __shfl_xor(at, o, 64);
+    if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+  }
+}
+
+__global__ __launch_bounds__(64) void route_scored_kernel(const float* __restrict__ z, int z_w, const float* __restrict__ correction,
+                                                          float* __restrict__ w, float* __restrict__ side, int E, int n, int top,
+                                                          int groups, int keep, int has_shared) {
+  __shared__ float score[MAX_EXPERTS], choice[MAX_EXPERTS], wt[MAX_EXPERTS], best_of[MAX_EXPERTS];
+  const int t = blockIdx.x, lane = threadIdx.x;
+  const float* zt = z + (size_t)t * z_w;
+  float m = -INFINITY;
+  for (int e = lane; e < n; e += 64) m = fmaxf(m, zt[e]);
+  m = wave_max(m);
+  float sum = 0.f;
+  for (int e = lane; e < n; e += 64) {
+    const float x = expf(zt[e] - m);
+    score[e] = x;
+    sum += x;
+  }
+  sum = wave_sum(sum);
+  for (int e = lane; e < n; e += 64) {
+    const float x = score[e] / sum;
+    score[e] = x;
+    choice[e] = x + (correction ? correction[e] : 0.f);
+    wt[e] = 0.f;
+  }
+  __syncthreads();
+  if (keep < groups) {
+    const int gs = n / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float b = -INFINITY;
+      for (int e = g * gs; e < (g + 1) * gs; ++e) b = fmaxf(b, choice[e]);
+      best_of[g] = b;
+    }
+    __syncthreads();
+    for (int k = 0; k < keep; ++k) {                   // the kept groups are marked by +infinity
+      float b = -INFINITY;
+      int at = groups;
+      for (int g = lane; g < groups; g += 64)
+        if (best_of[g] < INFINITY && (at == groups || best_of[g] > b)) { b = best_of[g]; at = g; }
+      wave_argmax(b, at);
+      __syncthreads();
+      if (lane == 0 && at < groups) best_of[at] = INFINITY;
+      __syncthreads();
+    }
+    for (int e = lane; e < n; e += 64)
+      if (best_of[e / gs] < INFINITY) choice[e] = -INFINITY;
+    __syncthreads();
+  }
+  float total = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float b = -INFINITY;
+    int at = n;
+    for (int e = lane; e < n; e += 64)
+      if (choice[e] > b) { b = choice[e]; at = e; }
+    wave_argmax(b, at);
+    if (at >= n) break;                                // (only if the scores are not numbers)
+    total += score[at];
+    __syncthreads();
+    if (lane == 0) {
+      wt[at] = score[at];
+      choice[at] = -INFINITY;
+    }
+    __syncthreads();
+  }
+  const float inv = 1.f / (total + 1e-20f);
+  float id = 0.f;
+  for (int e = lane; e < n; e += 64) {
+    const float x = wt[e] * inv;
+    if (e < E) w[(size_t)t * E + e] = x;
+    else id += x;
+  }
+  id = wave_sum(id);
+  if (lane == 0) {
+    side[2 * (size_t)t] = id;
+    side[2 * (size_t)t + 1] = has_shared ? 1.f / (1.f + expf(-zt[n])) : 0.f;
+  }
 }
 
 template <typename TI, typename TO>
@@ -233,17 +323,32 @@ __global__ __launch_bounds__(256) void expert_down_kernel(const bf16_t* __restri
   }
 }
 
-// y[t, c] = the sum of the token's rows of `rows` [R, W]
-__global__ void expert_combine_kernel(const float* __restrict__ rows, const int* __restrict__ token_rows, float* __restrict__ y,
-                                      int W, int top) {
+// y[t, c] = the sum of the token's rows of `rows` [R, W], or of the n_base partial rows base[s][t]; with `side` also
+// side[t][0] x[t, c] (the identity experts give the input back) + side[t][1] * (the sum of the shared expert's partial rows).
+template <typename TX>
+__global__ void expert_combine_kernel(const float* __restrict__ rows, const int* __restrict__ token_rows, int top,
+                                      const float* __restrict__ base, int n_base, const TX* __restrict__ x, const float* __restrict__ side,
+                                      const float* __restrict__ shared, int n_shared, float* __restrict__ y, int T, int W) {
   const int t = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= W) return;
+  const size_t at = (size_t)t * W + c, all = (size_t)T * W;
   float s = 0.f;
-  for (int j = 0; j < top; ++j) {
-    const int r = token_rows[(size_t)t * top + j];
-    if (r >= 0) s += rows[(size_t)r * W + c];
+  if (rows) {
+    for (int j = 0; j < top; ++j) {
+      const int r = token_rows[(size_t)t * top + j];
+      if (r >= 0) s += rows[(size_t)r * W + c];
+    }
   }
-  y[(size_t)t * W + c] = s;
+  for (int i = 0; i < n_base; ++i) s += base[i * all + at];
+  if (side) {
+    s = fmaf(side[2 * (size_t)t], load_f32(x, at), s);
+    if (n_shared > 0) {
+      float u = 0.f;
+      for (int i = 0; i < n_shared; ++i) u += shared[i * all + at];
+      s = fmaf(side[2 * (size_t)t + 1], u, s);
+    }
+  }
+  y[at] = s;
 }
 
 }  // namespace
@@ -255,10 +360,13 @@ extern "C" long alice_expert_rows(int T, int E, int top) {
 
 // The routed feed-forward by grouped products, see the top of the file.  x: [T, W] bfloat16; weights: [T, E] float32 of
 // alice_route_topk; gate_up, down: fragment layouts of [2 E F, W] and [W, E F]; y: [T, W] float32.  Workspaces for
-// R = alice_expert_rows(T, E, top): ints [2 R + R / 64 + T top] (row_token, tile_expert, token_rows; the row weights
+// side, shared: null, or what alice_expert_combine adds (the identity experts' weight and the shared expert's gate a token,
+// the shared expert's partial rows).  R = alice_expert_rows(T, E, top): ints [2 R + R / 64 + T top] (row_token, tile_expert, token_rows; the row weights
 // share the ints' buffer as floats), mid [R, F] bfloat16, rows [R, W] float32.
 extern "C" int alice_expert_products(const void* x, const float* weights, const void* gate_up, const void* down, float* y, int* ints,
-                                     void* mid, float* rows, int T, int W, int F, int E, int top, float epi, hipStream_t stream) {
+                                     void* mid, float* rows, int T, int W, int F, int E, int top, float epi, const float* side,
+                                     const float* shared, int n_shared, hipStream_t stream) {
+  ALICE_CHECK(n_shared == 0 || (side && shared), "expert_products: a shared expert needs its rows and its gate");
   ALICE_CHECK(x && weights && gate_up && down && y && ints && mid && rows, "expert_products: a pointer is missing");
   ALICE_CHECK(T >= 1 && E >= 1 && E <= MAX_EXPERTS && top >= 1 && top <= E, "expert_products: 1 <= top <= experts <= %d", MAX_EXPERTS);
   ALICE_CHECK(W >= 8 && W % 8 == 0 && F >= 32 && F % 32 == 0, "expert_products: the width must be a multiple of 8 and the experts' a multiple of 32");
@@ -278,7 +386,7 @@ extern "C" int alice_expert_products(const void* x, const float* weights, const 
   expert_down_kernel<4><<<g2, 256, 0, stream>>>((const bf16_t*)mid, (const bf16_t*)down, tile_expert, rows, W, F, E);
   ALICE_LAUNCH_CHECK();
   dim3 g3(T, ceil_div(W, 256));
-  expert_combine_kernel<<<g3, 256, 0, stream>>>(rows, token_rows, y, W, top);
+  expert_combine_kernel<bf16_t><<<g3, 256, 0, stream>>>(rows, token_rows, top, nullptr, 0, (const bf16_t*)x, side, shared, n_shared, y, T, W);
   ALICE_LAUNCH_CHECK();
   return 0;
 }
@@ -288,6 +396,32 @@ extern "C" int alice_route_topk(const float* z, const float* bias, float* w, int
   ALICE_CHECK(T >= 0 && E >= 1 && E <= MAX_EXPERTS && top >= 1 && top <= E, "route_topk: 1 <= top <= experts <= %d", MAX_EXPERTS);
   if (T == 0) return 0;
   route_kernel<<<T, 64, 0, stream>>>(z, bias, w, E, top);
+  ALICE_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int alice_route_scored(const float* z, int z_w, const float* correction, float* w, float* side, int T, int experts,
+                                  int identity, int top, int groups, int keep, int has_shared, hipStream_t stream) {
+  ALICE_CHECK(z && w && side, "route_scored: a pointer is missing");
+  const int n = experts + identity;
+  ALICE_CHECK(T >= 0 && experts >= 1 && identity >= 0 && n <= MAX_EXPERTS && top >= 1 && top <= n, "route_scored: 1 <= top <= outputs <= %d", MAX_EXPERTS);
+  ALICE_CHECK(groups >= 1 && n % groups == 0 && keep >= 1 && keep <= groups && (long)keep * (n / groups) >= top,
+              "route_scored: %d groups must divide %d outputs, and the kept ones hold at least `top` of them", groups, n);
+  ALICE_CHECK(z_w >= n + (has_shared ? 1 : 0), "route_scored: rows of %d logits are too short", z_w);
+  if (T == 0) return 0;
+  route_scored_kernel<<<T, 64, 0, stream>>>(z, z_w, correction, w, side, experts, n, top, groups, keep, has_shared);
+  ALICE_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int alice_expert_combine(const float* base, int n_base, const void* x, int x_dtype, const float* side, const float* shared,
+                                    int n_shared, float* y, int T, int W, hipStream_t stream) {
+  ALICE_CHECK(base && n_base >= 1 && x && side && y && dtype_ok(x_dtype), "expert_combine: a pointer is missing or the dtype is unknown");
+  ALICE_CHECK(T >= 0 && W >= 1 && n_shared >= 0 && (n_shared == 0 || shared), "expert_combine: bad sizes");
+  if (T == 0) return 0;
+  const dim3 grid(T, ceil_div(W, 256));
+  DISPATCH_DTYPE(x_dtype, TX, (expert_combine_kernel<TX><<<grid, 256, 0, stream>>>(nullptr, nullptr, 0, base, n_base, (const TX*)x, side, shared,
+                                                                                 n_shared, y, T, W)));
   ALICE_LAUNCH_CHECK();
   return 0;
 }

@@ -5,7 +5,7 @@
 // dimensions are also the value; all heads of a token read the same rows.
 //
 // Kernels of this file:
-//   alice_latent_prepare     from the float32 rows [a | c' | kr'] of the fused down projection: a / rms(a) * wa to the
+//   alice_latent_prepare     from the float32 rows [a | c' | kr'] of the fused down projection (a may be empty): a / rms(a) * wa to the
 //                            query latent (activation dtype), c' / rms(c') * wc and kr' rotated in pairs (2i, 2i + 1)
 //                            into the token's cache row
 //   alice_heads_linear       a matrix a head: y[t, h, 0:n] = M_h x[t, h, 0:k] (M given transposed, [H, k, n]), with
@@ -30,9 +30,11 @@ __global__ __launch_bounds__(PREP_THREADS) void latent_prepare_kernel(
   const int t = blockIdx.x, tid = threadIdx.x;
   const float* row = rows + (size_t)t * row_w;
   float s = 0.f;
-  for (int i = tid; i < A; i += PREP_THREADS) s = fmaf(row[i], row[i], s);
-  const float inv_a = 1.f / sqrtf(block_sum(s, red) / (float)A + eps);
-  for (int i = tid; i < A; i += PREP_THREADS) store_f32(a_out + (size_t)t * A, i, row[i] * inv_a * wa[i]);
+  if (A > 0) {
+    for (int i = tid; i < A; i += PREP_THREADS) s = fmaf(row[i], row[i], s);
+    const float inv_a = 1.f / sqrtf(block_sum(s, red) / (float)A + eps);
+    for (int i = tid; i < A; i += PREP_THREADS) store_f32(a_out + (size_t)t * A, i, row[i] * inv_a * wa[i]);
+  }
   if (!k_pool) return;
   const int pos = positions[t];
   const int page = block_table[(size_t)seq_of_token[t] * bt_stride + pos / page_size];
@@ -184,8 +186,8 @@ extern "C" int alice_latent_prepare(const float* rows, int row_width, int q_rank
                                     int page_size, int n_pages, void* q_latent, void* k_pool, int out_dtype, int T,
                                     hipStream_t stream) {
   ALICE_CHECK(dtype_ok(out_dtype), "latent_prepare: unknown dtype %d", out_dtype);
-  ALICE_CHECK(rows && w_q && w_kv && q_latent && positions, "latent_prepare: missing arguments");
-  ALICE_CHECK(T >= 0 && q_rank >= 1 && kv_rank >= 1 && rot_dim >= 0 && rot_dim % 2 == 0,
+  ALICE_CHECK(rows && w_kv && positions && (q_rank == 0 || (w_q && q_latent)), "latent_prepare: missing arguments");
+  ALICE_CHECK(T >= 0 && q_rank >= 0 && kv_rank >= 1 && rot_dim >= 0 && rot_dim % 2 == 0,
               "latent_prepare: bad sizes q_rank=%d kv_rank=%d rot_dim=%d", q_rank, kv_rank, rot_dim);
   ALICE_CHECK(row_width >= q_rank + kv_rank + rot_dim, "latent_prepare: rows of %d elements are too short", row_width);
   ALICE_CHECK(rot_dim == 0 || (cos_t && sin_t), "latent_prepare: a rotated part needs both tables");

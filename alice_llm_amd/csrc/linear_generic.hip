@@ -193,7 +193,7 @@ int alice_linear_generic(const void* x, int x_dtype, const void* w, int w_dtype,
   ALICE_CHECK(M >= 0 && N > 0 && K > 0, "linear: bad sizes M=%d N=%d K=%d", M, N, K);
   ALICE_CHECK(epi == ALICE_EPI_NONE || epi == ALICE_EPI_GEGLU || epi == ALICE_EPI_SOFTCAP,
               "linear: unknown epilogue %d", epi);
-  ALICE_CHECK(epi != ALICE_EPI_SOFTCAP || epi_param > 0.f || epi_param == ALICE_UNARY_RELU2, "linear: softcap must be positive");
+  ALICE_CHECK(epi != ALICE_EPI_SOFTCAP || epi_param > 0.f || epi_param == ALICE_UNARY_RELU2 || epi_param == ALICE_UNARY_SILU, "linear: softcap must be positive");
   ALICE_CHECK(ceil_div(M, BM) <= 65535, "linear: M=%d has too many row tiles for one launch", M);
   if (M == 0) return 0;
   int rc = 0;

@@ -281,27 +281,27 @@ __global__ __launch_bounds__(64 * WPB) void recurrence_kernel(RecurrenceArgs a) 
 // A block per (token, part): the row's part of n elements is RMS-normed (eps inside the root) and multiplied by a
 // weight (of the part's length, shared by the parts, or of the row's length).  gate_act 1: silu of the gate row,
 // applied before the norm; 2: sigmoid of the gate row, applied after it; 0: no gate.
-template <typename TO>
-__global__ __launch_bounds__(256) void norm_gate_kernel(const float* __restrict__ x, int width, int parts, const float* __restrict__ gate,
+template <typename TO, typename TG>
+__global__ __launch_bounds__(1024) void norm_gate_kernel(const float* __restrict__ x, int width, int parts, const TG* __restrict__ gate,
                                                         int gate_w, int gate_col, int gate_act, const float* __restrict__ w,
                                                         int w_shared, float eps, TO* __restrict__ out) {
   __shared__ float red[17];
   const int t = blockIdx.x, g = blockIdx.y, n = width / parts;
   const float* xr = x + (size_t)t * width + (size_t)g * n;
-  const float* gr = gate ? gate + (size_t)t * gate_w + gate_col + (size_t)g * n : nullptr;
+  const TG* gr = gate ? gate + (size_t)t * gate_w + gate_col + (size_t)g * n : nullptr;
   float ss = 0.f;
   for (int e = threadIdx.x; e < n; e += blockDim.x) {
     float y = xr[e];
-    if (gate_act == 1) y *= silu_full(gr[e]);
+    if (gate_act == 1) y *= silu_full(load_f32(gr, e));
     ss = fmaf(y, y, ss);
   }
   ss = block_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)n + eps);
   for (int e = threadIdx.x; e < n; e += blockDim.x) {
     float y = xr[e];
-    if (gate_act == 1) y *= silu_full(gr[e]);
+    if (gate_act == 1) y *= silu_full(load_f32(gr, e));
     y = y * inv * w[w_shared ? e : g * n + e];
-    if (gate_act == 2) y *= sigmoid_full(gr[e]);
+    if (gate_act == 2) y *= sigmoid_full(load_f32(gr, e));
     store_f32(out + (size_t)t * width + (size_t)g * n, e, y);
   }
 }
@@ -402,18 +402,20 @@ extern "C" int alice_matrix_recurrence(const float* q, int q_w, int q_col, const
   return 0;
 }
 
-extern "C" int alice_norm_gate(const float* x, int width, int parts, const float* gate, int gate_w, int gate_col, int gate_act,
+extern "C" int alice_norm_gate(const float* x, int width, int parts, const void* gate, int gate_dtype, int gate_w, int gate_col, int gate_act,
                                const float* w, int w_shared, float eps, void* out, int out_dtype, int T, hipStream_t stream) {
-  ALICE_CHECK(x && w && out && dtype_ok(out_dtype), "norm_gate: a pointer is missing or the dtype is unknown");
+  ALICE_CHECK(x && w && out && dtype_ok(out_dtype) && dtype_ok(gate_dtype), "norm_gate: a pointer is missing or the dtype is unknown");
   ALICE_CHECK(T >= 0 && width >= 1 && parts >= 1 && width % parts == 0 && parts <= 65535, "norm_gate: %d parts must divide the width %d", parts, width);
   ALICE_CHECK(gate_act >= 0 && gate_act <= 2 && (gate_act == 0 || (gate && gate_col >= 0 && gate_col + width <= gate_w)),
               "norm_gate: the gate rows are missing or too short");
   ALICE_CHECK(eps > 0.f, "norm_gate: eps must be positive");
   if (T == 0) return 0;
   dim3 grid(T, parts);
-  const int threads = width / parts > 128 ? 256 : 64;
-  if (out_dtype == DT_F32) norm_gate_kernel<float><<<grid, threads, 0, stream>>>(x, width, parts, gate, gate_w, gate_col, gate_act, w, w_shared, eps, (float*)out);
-  else norm_gate_kernel<bf16_t><<<grid, threads, 0, stream>>>(x, width, parts, gate, gate_w, gate_col, gate_act, w, w_shared, eps, (bf16_t*)out);
+  const int n = width / parts, threads = n > 1024 && (long)T * parts <= 256 ? 1024 : (n > 128 ? 256 : 64);      // few rows: more lanes a row
+#define GO(TO, TG) norm_gate_kernel<TO, TG><<<grid, threads, 0, stream>>>(x, width, parts, (const TG*)gate, gate_w, gate_col, gate_act, w, w_shared, eps, (TO*)out)
+  if (gate_dtype == DT_F32) { if (out_dtype == DT_F32) GO(float, float); else GO(bf16_t, float); }
+  else { if (out_dtype == DT_F32) GO(float, bf16_t); else GO(bf16_t, bf16_t); }
+#undef GO
   ALICE_LAUNCH_CHECK();
   return 0;
 }

@@ -18,9 +18,10 @@ from ..csrc import build as _build
 EPI_NONE, EPI_GEGLU, EPI_SOFTCAP = 0, 1, 2
 LAYOUT_ROW, LAYOUT_FRAG16 = 0, 1
 LINEAR_AUTO, LINEAR_GENERIC, LINEAR_SKINNY, LINEAR_MFMA, LINEAR_TILED_W16, LINEAR_TILED_W32 = 0, 1, 2, 3, 4, 5
-ABI_VERSION = 12
+ABI_VERSION = 13
 GATED_SILU = -1.0        # epi_param of EPI_GEGLU that picks silu(gate) * up
 UNARY_RELU2 = -1.0       # epi_param of EPI_SOFTCAP that picks the square of max(y, 0) instead of the capped form
+UNARY_SILU = -2.0        # likewise y * sigmoid(y)
 
 _lib = None
 _lib_path = None
@@ -39,7 +40,7 @@ def _declare(lib) -> None:
     lib.alice_device_arch.argtypes = [c.c_char_p, I]
     sigs = {
         "alice_embed": [P, P, I, I, P, I, I, I, F, P],
-        "alice_add_norm": [P, P, I, L, P, P, I, P, I, P, I, I, F, F, F, F, I, I, P],
+        "alice_add_norm": [P, P, I, L, P, P, P, I, P, I, P, I, I, F, F, F, F, I, I, P],
         "alice_softcap": [P, L, F, I, P],
         "alice_add_branches": [P, I, P, P, P, P, I, P, P, P, I, I, I, I, P],
         "alice_linear": [P, I, P, I, I, P, I, I, I, I, I, F, I, I, I, I, I, P],
@@ -71,10 +72,13 @@ def _declare(lib) -> None:
         "alice_delta_prepare": [P, I, I, I, I, F, F, P, P, P, P, I, I, P, I, I, P],
         "alice_matrix_recurrence": [P, I, I, P, I, I, P, I, I, P, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "alice_matrix_recurrence_columns": [I, I, I, I],
-        "alice_norm_gate": [P, I, I, P, I, I, I, P, I, F, P, I, I, P],
+        "alice_norm_gate": [P, I, I, P, I, I, I, I, P, I, F, P, I, I, P],
         "alice_route_topk": [P, P, P, I, I, I, P],
         "alice_scale_columns": [P, I, P, P, I, I, I, I, P],
-        "alice_expert_products": [P, P, P, P, P, P, P, P, I, I, I, I, I, F, P],
+        "alice_expert_products": [P, P, P, P, P, P, P, P, I, I, I, I, I, F, P, P, I, P],
+        "alice_route_scored": [P, I, P, P, P, I, I, I, I, I, I, I, P],
+        "alice_expert_combine": [P, I, P, I, P, P, I, P, I, I, P],
+        "alice_lightning": [P, I, I, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
         "alice_add_rows": [P, P, P, I, I, P],
         "alice_latent_prepare": [P, I, I, I, I, P, P, F, P, P, P, P, P, I, I, I, P, P, I, I, P],
         "alice_heads_linear": [P, I, L, I, P, I, P, I, L, I, I, I, I, I, I, P, P, P, P],
@@ -102,6 +106,8 @@ def _declare(lib) -> None:
     lib.alice_attention_split_workspace.restype = L
     lib.alice_mlstm_chunks_workspace.argtypes = [I, I, I, I, I, I]
     lib.alice_mlstm_chunks_workspace.restype = L
+    lib.alice_lightning_chunks.argtypes = [I, I]
+    lib.alice_lightning_chunks.restype = L
     lib.alice_expert_rows.argtypes = [I, I, I]
     lib.alice_expert_rows.restype = L
 
@@ -231,8 +237,9 @@ def add_norm(resid: torch.Tensor, branch: Optional[torch.Tensor], w_post: Option
              w_pre: Optional[torch.Tensor], out: Optional[torch.Tensor], *, eps_post: float = 0.0,
              eps_pre: float = 0.0, off_post: float = 0.0, off_pre: float = 0.0,
              rows: Optional[torch.Tensor] = None, n_partials: int = 1, full_precision: bool,
-             out_layout: int = LAYOUT_ROW) -> None:
-    """resid += norm_post(sum of branch partials); out = norm_pre(resid).  Each piece is optional.
+             out_layout: int = LAYOUT_ROW, b_pre: Optional[torch.Tensor] = None) -> None:
+    """resid += norm_post(sum of branch partials); out = norm_pre(resid).  Each piece is optional.  With b_pre (and a
+    float32 w_pre) norm_pre takes the row's mean off and adds this bias; without it is an RMS norm.
     out_layout FRAG16: `out` is a flat bfloat16 buffer of ceil16(T) * H elements in fragment order."""
     if resid.dim() != 2:
         raise HipLibraryError("resid must be [T, H]")
@@ -255,6 +262,10 @@ def add_norm(resid: torch.Tensor, branch: Optional[torch.Tensor], w_post: Option
             w_dtype = w.dtype
     if w_post is not None and branch is None:
         raise HipLibraryError("w_post without a branch")
+    if b_pre is not None:
+        if w_pre is None or w_dtype != torch.float32:
+            raise HipLibraryError("a norm with a bias needs float32 weights")
+        _dev(b_pre, "b_pre", torch.float32, (H,))
     if out is not None and out_layout == LAYOUT_FRAG16:
         _dev(out, "out", torch.bfloat16, (frag_rows(T) * H,))
     elif out is not None:
@@ -264,7 +275,7 @@ def add_norm(resid: torch.Tensor, branch: Optional[torch.Tensor], w_post: Option
     if rows is not None:
         _dev(rows, "rows", torch.int32)
     _call("alice_add_norm", resid.data_ptr(), _opt(branch, "branch"), n_partials, stride,
-          _opt(w_post, "w_post"), _opt(w_pre, "w_pre"), dtype_code(w_dtype or torch.float32),
+          _opt(w_post, "w_post"), _opt(w_pre, "w_pre"), _opt(b_pre, "b_pre"), dtype_code(w_dtype or torch.float32),
           _opt(out, "out"), dtype_code(out.dtype if out is not None else torch.float32),
           _opt(rows, "rows"), T, H, float(eps_post), float(eps_pre), float(off_post), float(off_pre),
           int(full_precision), int(out_layout), _stream())
@@ -805,34 +816,39 @@ def _rot_tables(cos, sin, rot_dim: int, max_position: int):
     return _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32)
 
 
-def latent_prepare(rows: torch.Tensor, w_q: torch.Tensor, w_kv: torch.Tensor, q_latent: torch.Tensor,
+def latent_prepare(rows: torch.Tensor, w_q: Optional[torch.Tensor], w_kv: torch.Tensor, q_latent: Optional[torch.Tensor],
                    k_pool: Optional[torch.Tensor], positions: torch.Tensor, seq_of_token: Optional[torch.Tensor],
                    block_table: Optional[torch.Tensor], *, q_rank: int, kv_rank: int, rot_dim: int, eps: float,
                    cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], max_position: int) -> None:
     """From the float32 rows [a (q_rank) | c (kv_rank) | kr (rot_dim)] of a fused down projection: the RMS-normed a
     (weight w_q) to q_latent [T, q_rank]; the RMS-normed c (weight w_kv) and kr rotated in pairs (2i, 2i + 1) into the
-    token's row of the cache, [pages, 1, page, kv_rank + rot_dim] (None: nothing is cached)."""
+    token's row of the cache, [pages, 1, page, kv_rank + rot_dim] (None: nothing is cached).  q_rank 0: no query latent
+    (w_q and q_latent are None)."""
     T = rows.shape[0]
     if rows.dim() != 2 or rows.shape[1] < q_rank + kv_rank + rot_dim:
         raise HipLibraryError(f"rows must be [T, >= {q_rank + kv_rank + rot_dim}], found {tuple(rows.shape)}")
     _dev(rows, "rows", torch.float32)
-    _dev(w_q, "w_q", torch.float32, (q_rank,))
+    if q_rank:
+        _dev(w_q, "w_q", torch.float32, (q_rank,))
+        _dev(q_latent, "q_latent", None, (T, q_rank))
+    elif k_pool is None:
+        return
     _dev(w_kv, "w_kv", torch.float32, (kv_rank,))
-    _dev(q_latent, "q_latent", None, (T, q_rank))
+    dt = q_latent.dtype if q_rank else k_pool.dtype
     _dev(positions, "positions", torch.int32, (T,))
     c, s_ = _rot_tables(cos, sin, rot_dim, max_position)
     page_size = n_pages = bt_stride = 0
     if k_pool is not None:
-        _latent_pool(k_pool, kv_rank, rot_dim, q_latent.dtype)
+        _latent_pool(k_pool, kv_rank, rot_dim, dt)
         n_pages, _, page_size, _ = k_pool.shape
         _dev(seq_of_token, "seq_of_token", torch.int32, (T,))
         _dev(block_table, "block_table", torch.int32)
         if block_table.dim() != 2 or max_position // page_size >= block_table.shape[1]:
             raise HipLibraryError(f"position {max_position} is beyond the block table")
         bt_stride = block_table.shape[1]
-    _call("alice_latent_prepare", rows.data_ptr(), rows.shape[1], q_rank, kv_rank, rot_dim, w_q.data_ptr(), w_kv.data_ptr(),
+    _call("alice_latent_prepare", rows.data_ptr(), rows.shape[1], q_rank, kv_rank, rot_dim, _opt(w_q, "w_q") if q_rank else None, w_kv.data_ptr(),
           float(eps), c, s_, positions.data_ptr(), _opt(seq_of_token, "seq_of_token"), _opt(block_table, "block_table"),
-          bt_stride, page_size, n_pages, q_latent.data_ptr(), _opt(k_pool, "k_pool"), dtype_code(q_latent.dtype), T, _stream())
+          bt_stride, page_size, n_pages, q_latent.data_ptr() if q_rank else None, _opt(k_pool, "k_pool"), dtype_code(dt), T, _stream())
 
 
 def heads_linear(x: torch.Tensor, wt: torch.Tensor, y: torch.Tensor, *, heads: int, n: int, k: int, rot_dim: int = 0,
@@ -1097,12 +1113,45 @@ def norm_gate(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, *, parts
     _dev(weight, "weight", torch.float32, (width // parts if weight_shared else width,))
     act = {None: 0, "silu": 1, "sigmoid": 2}[gate_act]
     if act:
-        _dev(gate, "gate", torch.float32)
+        _dev(gate, "gate")
         if gate.dim() != 2 or gate.shape[0] != T or gate_col + width > gate.shape[1]:
             raise HipLibraryError("the gate rows are too short")
-    _call("alice_norm_gate", x.data_ptr(), width, int(parts), _opt(gate, "gate") if act else None, gate.shape[1] if act else 0,
+    _call("alice_norm_gate", x.data_ptr(), width, int(parts), _opt(gate, "gate") if act else None,
+          dtype_code(gate.dtype) if act else 0, gate.shape[1] if act else 0,
           int(gate_col), act, weight.data_ptr(), int(bool(weight_shared)), float(eps), out.data_ptr(),
           dtype_code(out.dtype), T, _stream())
+
+
+LIGHTNING_CHUNK = 64            # tokens a chunk of the lightning kernels (ALICE_LIGHTNING_CHUNK)
+LIGHTNING_MAX_KEY_DIM = 256     # the largest key size they take
+LIGHTNING_CHUNKS_FROM = 16      # steps whose longest piece has at least this many tokens go by chunks
+
+
+def lightning(rows: torch.Tensor, columns, powers: torch.Tensor, out: torch.Tensor, ctx, S: torch.Tensor, *, heads: int,
+              head_dim: int, value_head_dim: int, silu: bool, chunked: Optional[bool] = None) -> None:
+    """Linear attention with a constant decay a head over a step (`ctx` gives cu_seqlens, slots, n_seqs, max_new): per head
+    S = g S + k v^T, o = S^T q.  rows [T, width] with q, k and v at `columns`, through silu on the way in if `silu`;
+    powers float32 [heads, LIGHTNING_CHUNK + 1]: the decays' powers; S float32 [slots, heads, d, dv]; out float32
+    [T, heads * dv].  chunked: None chooses by the step's longest piece; True, False fix the way."""
+    H, d, dv = heads, head_dim, value_head_dim
+    T = rows.shape[0]
+    _dev(rows, "rows")
+    _dev(powers, "powers", torch.float32, (H, LIGHTNING_CHUNK + 1))
+    _dev(out, "out", torch.float32, (T, H * dv))
+    if S.dim() != 4 or tuple(S.shape[1:]) != (H, d, dv):
+        raise HipLibraryError(f"S must be [slots, {H}, {d}, {dv}], found {tuple(S.shape)}")
+    _dev(S, "S", torch.float32)
+    _step_arrays(ctx)
+    q, k, v = columns
+    if chunked is None:
+        chunked = ctx.max_new >= LIGHTNING_CHUNKS_FROM
+    states = None
+    if chunked:
+        n = library().alice_lightning_chunks(T, ctx.n_seqs)
+        states = torch.empty((n * H * d * dv,), dtype=torch.float32, device=rows.device)
+    _call("alice_lightning", rows.data_ptr(), dtype_code(rows.dtype), rows.shape[1], int(q), int(k), int(v), int(bool(silu)),
+          powers.data_ptr(), out.data_ptr(), _opt(states, "states"), ctx.cu_seqlens.data_ptr(), ctx.slots.data_ptr(), S.data_ptr(),
+          T, ctx.n_seqs, S.shape[0], H, d, dv, int(chunked), _stream())
 
 
 def route_topk(logits: torch.Tensor, bias: Optional[torch.Tensor], weights: torch.Tensor, top: int) -> None:
@@ -1112,6 +1161,42 @@ def route_topk(logits: torch.Tensor, bias: Optional[torch.Tensor], weights: torc
     _opt(bias, "bias", torch.float32, (E,))
     _dev(weights, "weights", torch.float32, (T, E))
     _call("alice_route_topk", logits.data_ptr(), _opt(bias, "bias"), weights.data_ptr(), T, E, int(top), _stream())
+
+
+def route_scored(logits: torch.Tensor, correction: Optional[torch.Tensor], weights: torch.Tensor, side: torch.Tensor, *,
+                 identity: int, top: int, groups: int = 1, keep: int = 1, has_shared: bool = False) -> None:
+    """A router whose scores are a softmax over all n = experts + identity columns of logits (float32 [T, >= n]).  The
+    choice is score + correction (float32 [n]); of `groups` equal runs of neighbours the `keep` with the largest choice
+    stay, and of those the `top` largest choices serve the token, weighted by their scores divided by the scores' sum.
+    weights (float32 [T, experts]): zero where not chosen; side (float32 [T, 2]): the identity outputs' weight together,
+    and with has_shared sigmoid(logits[:, n])."""
+    T, E = weights.shape
+    n = E + int(identity)
+    _dev(logits, "logits", torch.float32)
+    if logits.dim() != 2 or logits.shape[0] != T or logits.shape[1] < n + int(bool(has_shared)):
+        raise HipLibraryError(f"logits must be [{T}, >= {n + int(bool(has_shared))}], found {tuple(logits.shape)}")
+    _dev(weights, "weights", torch.float32)
+    _dev(side, "side", torch.float32, (T, 2))
+    _call("alice_route_scored", logits.data_ptr(), logits.shape[1], _opt(correction, "correction", torch.float32, (n,)),
+          weights.data_ptr(), side.data_ptr(), T, E, int(identity), int(top), int(groups), int(keep), int(bool(has_shared)), _stream())
+
+
+def _partial_rows(t: Optional[torch.Tensor], name: str, T: int, W: int) -> int:
+    """How many partial results `t` holds: float32 [T, W] or [S, T, W] (None: none)."""
+    if t is None:
+        return 0
+    _dev(t, name, torch.float32, (T, W) if t.dim() == 2 else (t.shape[0], T, W))
+    return 1 if t.dim() == 2 else t.shape[0]
+
+
+def expert_combine(base: torch.Tensor, x: torch.Tensor, side: torch.Tensor, shared: Optional[torch.Tensor], y: torch.Tensor) -> None:
+    """y[t] = base[t] + side[t, 0] x[t] + side[t, 1] shared[t]; base and shared float32 [T, W] or partial sums [S, T, W]."""
+    T, W = x.shape
+    _dev(x, "x", None)
+    _dev(side, "side", torch.float32, (T, 2))
+    _dev(y, "y", torch.float32, (T, W))
+    _call("alice_expert_combine", base.data_ptr(), _partial_rows(base, "base", T, W), x.data_ptr(), dtype_code(x.dtype), side.data_ptr(),
+          _opt(shared, "shared"), _partial_rows(shared, "shared", T, W), y.data_ptr(), T, W, _stream())
 
 
 def scale_columns(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor) -> None:
@@ -1132,11 +1217,13 @@ def expert_products_supported(dtype: torch.dtype, width: int, expert_width: int)
 
 
 def expert_products(x: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, y: torch.Tensor, *,
-                    expert_width: int, top: int, epi_param: float) -> None:
+                    expert_width: int, top: int, epi_param: float, side: Optional[torch.Tensor] = None,
+                    shared: Optional[torch.Tensor] = None) -> None:
     """The routed feed-forward by grouped products: y[t] = sum over the experts e that token t uses (weights[t, e] > 0) of
     weights[t, e] * down_e(act(gate_e x[t]) * (up_e x[t])).  x: bfloat16 [T, W]; weights: float32 [T, E]; gate_up, down: the
     fragment layouts of [all gates; all ups] ([2 E F, W]) and of the down matrices side by side ([W, E F]); y: float32
-    [T, W].  The (token, expert) pairs are put in expert order on the device; only the chosen experts are read."""
+    [T, W].  The (token, expert) pairs are put in expert order on the device; only the chosen experts are read.  With
+    side (float32 [T, 2]): plus side[t, 0] x[t] + side[t, 1] shared[t], shared float32 [T, W] or partial sums."""
     T, W = x.shape
     E, F = weights.shape[1], int(expert_width)
     if not expert_products_supported(x.dtype, W, F):
@@ -1151,7 +1238,8 @@ def expert_products(x: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tenso
     mid = torch.empty((R, F), dtype=torch.bfloat16, device=x.device)
     rows = torch.empty((R, W), dtype=torch.float32, device=x.device)
     _call("alice_expert_products", x.data_ptr(), weights.data_ptr(), gate_up.data_ptr(), down.data_ptr(), y.data_ptr(),
-          ints.data_ptr(), mid.data_ptr(), rows.data_ptr(), T, W, F, E, int(top), float(epi_param), _stream())
+          ints.data_ptr(), mid.data_ptr(), rows.data_ptr(), T, W, F, E, int(top), float(epi_param),
+          _opt(side, "side", torch.float32, (T, 2)), _opt(shared, "shared"), _partial_rows(shared, "shared", T, W), _stream())
 
 
 def fragment_layout_supported(rows: int, k_in: int, epilogue: int) -> bool:

@@ -10,18 +10,32 @@ expert), and one down projection over all of them is the weighted sum.  Steps of
 expert) pairs are put in expert order on the device and each pair meets its own expert's matrices only (grouped
 products over the same stacked matrices).  Every kernel's launch depends on sizes only, never on which experts the
 tokens chose.
+
+Variants, by constructor arguments:
+  `scoring="all"`   the scores are a softmax over all router outputs; a stored correction (tensor "correction", one number an
+                    output) is added for the choice only; the weights are the chosen scores divided by their sum (+ 1e-20).
+                    The outputs may form `groups` = (count, keep): equal runs of neighbours of which only the `keep` with the
+                    largest choice in them can serve the token.  No router bias.
+  `identity=Z`      the last Z router outputs (behind the experts) are experts without matrices that give the token's own
+                    input back (with scoring "all").
+  `shared`          a further feed-forward of the same gated form, with sizes and constants of its own ("shared.gate" and so
+                    on), that serves every token, times sigmoid(s . h) ("shared.sg"; with scoring "all").
+  `activation="swish_limited"` with `limit`: the experts' bounded gated form.
+The shared expert's gate is one more row of the router's matrix, and its output and the identity experts' are added in
+the kernel that adds up a token's experts.
 """
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict, Mapping, Optional, Tuple
 
 import torch
 
 from ..hip import ops
 from .base import FEED_FORWARDS, ParamSpec, Part, Precision
+from .feedforward import GatedMLP
 from .linear import Linear
 
-_GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU}
+_GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
 GROUPED_FROM_TOKENS = 128      # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles);
                                # below, one pass over all experts' matrices is as fast or faster (measured at 16 experts, 2 a token)
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
@@ -32,18 +46,34 @@ class ExpertMLP(Part):
     graph_safe = True
 
     def __init__(self, precision: Precision, *, hidden_size: int, intermediate_size: int, experts: int, top: int,
-                 activation: str = "silu", router_bias: bool = True):
+                 activation: str = "silu", limit: Optional[float] = None, router_bias: bool = True, scoring: str = "chosen",
+                 identity: int = 0, groups: Optional[Tuple[int, int]] = None, shared: Optional[Mapping] = None):
         if activation not in _GATED:
             raise ValueError(f"expert_mlp has no kernel for activation '{activation}'; available: {sorted(_GATED)}")
-        if not 1 <= top <= experts <= ops.ROUTER_MAX_EXPERTS:
-            raise ValueError(f"expert_mlp: 1 <= top <= experts <= {ops.ROUTER_MAX_EXPERTS}, found top {top} of {experts}")
+        if (activation == "swish_limited") != (limit is not None) or (limit is not None and not limit > 0):
+            raise ValueError("expert_mlp: 'swish_limited' takes a positive limit, and only it does")
+        if scoring not in ("chosen", "all"):
+            raise ValueError(f"expert_mlp: scoring '{scoring}' is not known; available: 'chosen', 'all'")
+        if scoring == "chosen" and (identity or groups or shared):
+            raise ValueError("expert_mlp: identity experts, groups and a shared expert come with scoring 'all'")
+        outputs = int(experts) + int(identity)
+        if experts < 1 or identity < 0 or not 1 <= top <= outputs <= ops.ROUTER_MAX_EXPERTS:
+            raise ValueError(f"expert_mlp: 1 <= top <= experts <= {ops.ROUTER_MAX_EXPERTS}, found top {top} of {outputs}")
+        count, keep = groups or (1, 1)
+        if count < 1 or outputs % count or not 1 <= keep <= count or keep * (outputs // count) < top:
+            raise ValueError(f"expert_mlp: {count} groups must divide {outputs} outputs, and the {keep} kept ones hold at least {top}")
         self.precision = precision
         self.H, self.F, self.E, self.top = hidden_size, int(intermediate_size), int(experts), int(top)
-        self.router_bias = bool(router_bias)
-        self.router = Linear(hidden_size, self.E, precision)
-        self.gate_up = Linear(hidden_size, self.E * self.F, precision, epilogue=ops.EPI_GEGLU, epi_param=_GATED[activation])
+        self.identity, self.groups, self.scored = int(identity), (int(count), int(keep)), scoring == "all"
+        self.outputs = outputs
+        self.router_bias = bool(router_bias) and not self.scored
+        self.shared = None if shared is None else GatedMLP(precision, hidden_size=hidden_size, tensor_names={
+            "gate": "gate", "up": "up", "down": "down"}, **shared)
+        self.router = Linear(hidden_size, outputs + (self.shared is not None), precision)      # the last row: the shared expert's gate
+        self.gate_up = Linear(hidden_size, self.E * self.F, precision, epilogue=ops.EPI_GEGLU,
+                              epi_param=float(limit) if limit is not None else _GATED[activation])
         self.down = Linear(self.E * self.F, hidden_size, precision)
-        self.bias: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None           # added to the logits; with scoring "all" to the scores, for the choice
         self._parts: Dict[str, torch.Tensor] = {}
 
     def param_specs(self) -> Dict[str, ParamSpec]:
@@ -52,22 +82,35 @@ class ExpertMLP(Part):
             specs[f"e{e}.gate"] = ParamSpec((self.F, self.H))
             specs[f"e{e}.up"] = ParamSpec((self.F, self.H))
             specs[f"e{e}.down"] = ParamSpec((self.H, self.F))
-        specs["router"] = ParamSpec((self.E, self.H), init_std=0.1)
+        specs["router"] = ParamSpec((self.outputs, self.H), init_std=0.1)
         if self.router_bias:
-            specs["router.b"] = ParamSpec((self.E,), init_std=0.1)
+            specs["router.b"] = ParamSpec((self.outputs,), init_std=0.1)
+        if self.scored:
+            specs["correction"] = ParamSpec((self.outputs,), init_std=0.1)
+        if self.shared is not None:
+            specs.update({f"shared.{n}": spec for n, spec in self.shared.param_specs().items()})
+            specs["shared.sg"] = ParamSpec((1, self.H), init_std=0.1)
         return specs
 
     def assign(self, name: str, tensor: torch.Tensor) -> None:
-        if name == "router":
-            self.router.load(tensor)
-        elif name == "router.b" and self.router_bias:
+        if (name == "router.b" and self.router_bias) or (name == "correction" and self.scored):
             self.bias = tensor.float().contiguous()
+        elif self.shared is not None and name.startswith("shared.") and name != "shared.sg":
+            self.shared.assign(name[len("shared."):], tensor)
         elif name in self.param_specs():
             self._parts[name] = tensor
         else:
             raise KeyError(name)
 
     def finalize(self) -> None:
+        router = self.precision.matrix(self._parts.pop("router"))
+        if self.shared is not None:
+            self.shared.finalize()
+            sg = self.precision.matrix(self._parts.pop("shared.sg"))
+            if sg.dtype != router.dtype:
+                router, sg = router.float(), sg.float()
+            router = torch.cat([router, sg], dim=0)
+        self.router.load(router)
         take = lambda what: [self.precision.matrix(self._parts.pop(f"e{e}.{what}")) for e in range(self.E)]
         gate, up, down = take("gate"), take("up"), take("down")
         if len({m.dtype for m in gate + up}) > 1:
@@ -78,7 +121,7 @@ class ExpertMLP(Part):
         self.down.load(torch.cat(down, dim=1).contiguous())  # [W, E F]: the experts' columns side by side
 
     def weight_bytes(self) -> int:
-        return self.router.nbytes() + self.gate_up.nbytes() + self.down.nbytes()
+        return self.router.nbytes() + self.gate_up.nbytes() + self.down.nbytes() + (self.shared.weight_bytes() if self.shared else 0)
 
     @property
     def accepts_fragment_activations(self) -> bool:
@@ -88,21 +131,35 @@ class ExpertMLP(Part):
         T, dev = x.shape[0], self.down.weight.device
         logits = self.router(x, torch.float32)
         weights = torch.empty((T, self.E), dtype=torch.float32, device=dev)
-        ops.route_topk(logits, self.bias, weights, self.top)
+        side = shared = None
+        if self.scored:
+            side = torch.empty((T, 2), dtype=torch.float32, device=dev)
+            ops.route_scored(logits, self.bias, weights, side, identity=self.identity, top=self.top, groups=self.groups[0],
+                             keep=self.groups[1], has_shared=self.shared is not None)
+            if self.shared is not None:
+                shared = self.shared.forward(x, ctx)
+        else:
+            ops.route_topk(logits, self.bias, weights, self.top)
+        side_used = side if self.identity or shared is not None else None
         if (T >= GROUPED_FROM_TOKENS and self.gate_up.layout == ops.LAYOUT_FRAG16 and self.down.layout == ops.LAYOUT_FRAG16
                 and ops.expert_products_supported(x.dtype, self.H, self.F)):
             # enough tokens that the experts' products pay: each (token, expert) pair meets its own expert only
             out = torch.empty((T, self.H), dtype=torch.float32, device=dev)
             ops.expert_products(x, weights, self.gate_up.weight, self.down.weight, out, expert_width=self.F, top=self.top,
-                                epi_param=self.gate_up.epi_param)
+                                epi_param=self.gate_up.epi_param, side=side_used, shared=shared)
             return out
         rows = max(1, MIDDLE_ELEMENTS // (self.E * self.F))
         if T <= rows:
-            return self._experts(x, weights, True)
-        out = torch.empty((T, self.H), dtype=torch.float32, device=dev)      # a long step: the tokens in runs, so that the middle stays small
-        for a in range(0, T, rows):
-            out[a:a + rows] = self._experts(x[a:a + rows], weights[a:a + rows], False)
-        return out
+            out = self._experts(x, weights, True)
+        else:
+            out = torch.empty((T, self.H), dtype=torch.float32, device=dev)  # a long step: the tokens in runs, so that the middle stays small
+            for a in range(0, T, rows):
+                out[a:a + rows] = self._experts(x[a:a + rows], weights[a:a + rows], False)
+        if side_used is None:
+            return out
+        y = torch.empty((T, self.H), dtype=torch.float32, device=dev)
+        ops.expert_combine(out, x, side, shared, y)
+        return y
 
     def _experts(self, x, weights, allow_partials: bool) -> torch.Tensor:
         mid = self.gate_up(x, torch.float32)                 # every expert's middle activations, not yet rounded

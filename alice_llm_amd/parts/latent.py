@@ -18,6 +18,12 @@ page.  The per-head maps move to the query's side, where they cost one small pro
 so the attention itself runs with one shared key row of R + r dimensions whose first R are also the value.  Norms,
 rotation, scores and softmax are 32-bit; products round as the run's other matrices do.  Ranks, head sizes, scale,
 window and eps are constructor arguments; `position` names a "rope_pairs" table over the r rotated dimensions.
+
+Variants: without a `q_rank` there is no query latent, q = Q h straight from the mixer's input.  With `own_rows` false
+the mixer has no Dkv: it reads rows that an earlier run of the schedule cached (the plan's `cache_from`) through its own
+Uk and Uv.  The kernels turn neighbouring pairs (2i, 2i + 1); where the position encoding pairs halves (i, i + r/2) the
+rows of the matrices that make rotated parts are put in that order at load, the same for queries and keys: a score is a
+sum over the rotated dimensions and does not depend on their order, and layers that share rows share the encoding.
 """
 from __future__ import annotations
 
@@ -29,7 +35,7 @@ from ..hip import ops
 from .base import MIXERS, CacheNeed, KVNeed, ParamSpec, Part, Precision
 from .linear import Linear
 
-_DEFAULT_NAMES = {"dq": "q_a_proj.weight", "dq_norm": "q_a_norm.weight", "uq": "q_b_proj.weight",
+_DEFAULT_NAMES = {"q": "q_proj.weight", "dq": "q_a_proj.weight", "dq_norm": "q_a_norm.weight", "uq": "q_b_proj.weight",
                   "dkv": "kv_a_proj.weight", "dkv_norm": "kv_a_norm.weight", "uk": "k_b_proj.weight",
                   "uv": "v_b_proj.weight", "o": "o_proj.weight"}
 
@@ -39,8 +45,8 @@ class LatentAttention(Part):
     graph_safe = True
 
     def __init__(self, precision: Precision, positions: dict, *, hidden_size: int, num_heads: int, head_dim: int,
-                 rot_dim: int, value_head_dim: int, q_rank: int, kv_rank: int, scale: float, norm_eps: float,
-                 window: Optional[int] = None, position: Optional[str] = None,
+                 rot_dim: int, value_head_dim: int, kv_rank: int, scale: float, norm_eps: float, q_rank: Optional[int] = None,
+                 window: Optional[int] = None, position: Optional[str] = None, own_rows: bool = True,
                  tensor_names: Optional[Dict[str, str]] = None):
         if rot_dim % 2 or rot_dim < 0:
             raise ValueError(f"latent_attention: the rotated part ({rot_dim}) must be even")
@@ -51,15 +57,17 @@ class LatentAttention(Part):
                              f"the latent attention kernels")
         self.precision = precision
         self.H, self.nH, self.d, self.r, self.dv = hidden_size, num_heads, head_dim, rot_dim, value_head_dim
-        self.A, self.R = q_rank, kv_rank
+        self.A, self.R, self.own_rows = int(q_rank or 0), kv_rank, bool(own_rows)
+        if self.A and not self.own_rows:
+            raise ValueError("latent_attention: a layer that reads another's rows takes its queries straight from its input")
         self.scale, self.eps, self.window = float(scale), float(norm_eps), window
         self.position = positions[position] if position is not None else None
         if self.position is not None and getattr(self.position, "rotary_dim", None) != rot_dim:
             raise ValueError("latent_attention: the position encoding must turn the whole rotated part")
         self.names = dict(_DEFAULT_NAMES, **(tensor_names or {}))
         # one product for both down projections: rows [a' (A) | c' (R) | kr' (r)], the sums kept in 32-bit for the norms
-        self.down = Linear(hidden_size, q_rank + kv_rank + rot_dim, precision)
-        self.uq = Linear(q_rank, num_heads * (head_dim + rot_dim), precision)
+        self.down = Linear(hidden_size, self.A + kv_rank + rot_dim, precision) if self.own_rows else None
+        self.uq = Linear(self.A or hidden_size, num_heads * (head_dim + rot_dim), precision)
         self.o = Linear(num_heads * value_head_dim, hidden_size, precision)
         self.w_q_norm: Optional[torch.Tensor] = None
         self.w_kv_norm: Optional[torch.Tensor] = None
@@ -70,11 +78,27 @@ class LatentAttention(Part):
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         n, H = self.names, self.nH
-        return {n["dq"]: ParamSpec((self.A, self.H)), n["dq_norm"]: ParamSpec((self.A,), init_std=0.1),
-                n["uq"]: ParamSpec((H * (self.d + self.r), self.A)),
-                n["dkv"]: ParamSpec((self.R + self.r, self.H)), n["dkv_norm"]: ParamSpec((self.R,), init_std=0.1),
-                n["uk"]: ParamSpec((H * self.d, self.R)), n["uv"]: ParamSpec((H * self.dv, self.R)),
-                n["o"]: ParamSpec((self.H, H * self.dv))}
+        if self.A:
+            specs = {n["dq"]: ParamSpec((self.A, self.H)), n["dq_norm"]: ParamSpec((self.A,), init_std=0.1),
+                     n["uq"]: ParamSpec((H * (self.d + self.r), self.A))}
+        else:
+            specs = {n["q"]: ParamSpec((H * (self.d + self.r), self.H))}
+        if self.own_rows:
+            specs.update({n["dkv"]: ParamSpec((self.R + self.r, self.H)), n["dkv_norm"]: ParamSpec((self.R,), init_std=0.1)})
+        specs.update({n["uk"]: ParamSpec((H * self.d, self.R)), n["uv"]: ParamSpec((H * self.dv, self.R)),
+                      n["o"]: ParamSpec((self.H, H * self.dv))})
+        return specs
+
+    def _pair_order(self, w: torch.Tensor, heads: int, plain: int) -> torch.Tensor:
+        """The rows of `heads` heads of [plain | r rotated] with every rotated part in the order 0, r/2, 1, r/2 + 1, ...
+        where the position encoding pairs halves; as they are where it pairs neighbours."""
+        if not self.r or getattr(self.position, "interleaved", True):
+            return w
+        half = self.r // 2
+        order = torch.arange(self.r).view(2, half).t().reshape(-1)
+        rows = torch.arange(heads * (plain + self.r)).view(heads, plain + self.r)
+        rows[:, plain:] = rows[:, plain:][:, order]
+        return w[rows.reshape(-1).to(w.device)].contiguous()
 
     def cache_need(self) -> CacheNeed:
         # one row a token, [c | kr]; its first R numbers are the value too, so the pages hold no values of their own
@@ -84,23 +108,27 @@ class LatentAttention(Part):
         n = self.names
         if name == n["o"]:
             self.o.load(tensor)
-        elif name == n["uq"]:
-            self.uq.load(tensor)
-        elif name == n["dq_norm"]:
+        elif name == (n["uq"] if self.A else n["q"]):
+            self.uq.load(self._pair_order(tensor, self.nH, self.d))
+        elif name == n["dq_norm"] and self.A:
             self.w_q_norm = tensor.float().contiguous()
-        elif name == n["dkv_norm"]:
+        elif name == n["dkv_norm"] and self.own_rows:
             self.w_kv_norm = tensor.float().contiguous()
-        elif name in (n["dq"], n["dkv"], n["uk"], n["uv"]):
+        elif name in (n["uk"], n["uv"]) or (name == n["dq"] and self.A) or (name == n["dkv"] and self.own_rows):
             self._parts[name] = tensor
         else:
             raise KeyError(name)
 
     def finalize(self) -> None:
         n, p = self.names, self.precision
-        dq, dkv = p.matrix(self._parts.pop(n["dq"])), p.matrix(self._parts.pop(n["dkv"]))
-        if dq.dtype != dkv.dtype:
-            dq, dkv = dq.float(), dkv.float()
-        self.down.load(torch.cat([dq, dkv], dim=0))
+        if self.own_rows:
+            dkv = p.matrix(self._pair_order(self._parts.pop(n["dkv"]), 1, self.R))
+            if self.A:
+                dq = p.matrix(self._parts.pop(n["dq"]))
+                if dq.dtype != dkv.dtype:
+                    dq, dkv = dq.float(), dkv.float()
+                dkv = torch.cat([dq, dkv], dim=0)
+            self.down.load(dkv)
         uk, uv = p.matrix(self._parts.pop(n["uk"])), p.matrix(self._parts.pop(n["uv"]))
         if p.full:
             uk, uv = uk.float(), uv.float()
@@ -117,7 +145,7 @@ class LatentAttention(Part):
 
     def weight_bytes(self) -> int:
         small = sum(t.numel() * t.element_size() for t in (self.uk_t, self.uv_t))
-        return self.down.nbytes() + self.uq.nbytes() + self.o.nbytes() + small
+        return (self.down.nbytes() if self.own_rows else 0) + self.uq.nbytes() + self.o.nbytes() + small
 
     def forward(self, x, ctx, cache) -> torch.Tensor:
         """x: [T, H] in the activation dtype; returns the branch in float32 ([T, H] or partial sums)."""
@@ -125,14 +153,15 @@ class LatentAttention(Part):
         nH, d, r, R, dv = self.nH, self.d, self.r, self.R, self.dv
         pos = self.position
         cos, sin = (pos.cos, pos.sin) if pos is not None else (None, None)
-        rows = self.down(x, torch.float32)
-        a = torch.empty((T, self.A), dtype=act, device=dev)
-        write = cache is not None and cache.writable
-        ops.latent_prepare(rows, self.w_q_norm, self.w_kv_norm, a, cache.k if write else None, ctx.positions,
-                           ctx.seq_of_token if write else None, cache.block_table if write else None,
-                           q_rank=self.A, kv_rank=R, rot_dim=r, eps=self.eps, cos=cos, sin=sin,
-                           max_position=ctx.max_position)
-        q = self.uq(a, act)                                        # [T, H * (d + r)]
+        a = torch.empty((T, self.A), dtype=act, device=dev) if self.A else None
+        if self.own_rows:
+            rows = self.down(x, torch.float32)
+            write = cache is not None and cache.writable
+            ops.latent_prepare(rows, self.w_q_norm, self.w_kv_norm, a, cache.k if write else None, ctx.positions,
+                               ctx.seq_of_token if write else None, cache.block_table if write else None,
+                               q_rank=self.A, kv_rank=R, rot_dim=r, eps=self.eps, cos=cos, sin=sin,
+                               max_position=ctx.max_position)
+        q = self.uq(a if self.A else x, act)                       # [T, H * (d + r)]
         qk = torch.empty((T, nH * (R + r)), dtype=act, device=dev)
         (ops.heads_linear_mfma if self.uk_mfma else ops.heads_linear)(
             q, self.uk_t, qk, heads=nH, n=R, k=d, rot_dim=r, cos=cos, sin=sin, positions=ctx.positions,

@@ -60,6 +60,22 @@ class Linear:
         return (self.layout == ops.LAYOUT_FRAG16 and rows >= 1 and self.n % 32 == 0
                 and self.epilogue != ops.EPI_SOFTCAP and self.precision.act == torch.bfloat16)
 
+    def rows(self, start: int, stop: int, *, epilogue: int = ops.EPI_NONE, epi_param: float = 0.0) -> Optional["Linear"]:
+        """A projection by the weight's rows start .. stop alone, with an epilogue of its own, on the same memory; None
+        where the layout keeps rows in tiles that these limits cut."""
+        if self.epilogue == ops.EPI_GEGLU or not 0 <= start < stop <= self.n:
+            raise ValueError(f"rows {start}..{stop} of a projection of {self.n} outputs")
+        part = Linear(self.k, stop - start, self.precision, epilogue=epilogue, epi_param=epi_param)
+        part.layout = self.layout
+        if self.layout == ops.LAYOUT_ROW:
+            part.weight = self.weight[start:stop]
+            return part
+        if start % 16 or (stop % 16 and stop != self.n):
+            return None
+        per_tile = -(-self.k // 32) * 512                   # elements of 16 rows
+        part.weight = self.weight[start // 16 * per_tile:-(-stop // 16) * per_tile]
+        return part
+
     def __call__(self, x, out_dtype: torch.dtype, *, allow_partials: bool = False,
                  variant: int = ops.LINEAR_AUTO, out_fragments: bool = False):
         """x: [M, k] tensor or FragmentActs.  Returns [M, n], or [S, M, n] float32 partial sums when the

@@ -1,4 +1,5 @@
-"""Norms.  RMSNorm: y = x / sqrt(mean(x^2) + eps) * (weight_offset + w), all in 32-bit.
+"""Norms.  RMSNorm: y = x / sqrt(mean(x^2) + eps) * (weight_offset + w), all in 32-bit.  LayerNorm:
+y = (x - m) / sqrt(mean((x - m)^2) + eps) * w + b with m = mean(x), likewise.
 
 The reference multiplies by the stored weight (llama3.rs:5244-5256), its files holding 1 + w; a
 safetensors file holds w, so Gemma 2 passes weight_offset = 1.  The offset, eps and the width are
@@ -59,4 +60,42 @@ class RMSNorm(Part):
         out = torch.empty((n, self.dim), dtype=out_dtype, device=x.device)
         ops.add_norm(x, None, None, self.weight, out, eps_pre=self.eps, off_pre=self.weight_offset,
                      rows=rows, full_precision=self.precision.full)
+        return out
+
+
+@NORMS.register("layernorm")
+class LayerNorm(Part):
+    """y = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w + b.  Weight and bias (`tensor_name` and `bias_name`)
+    are kept in 32-bit.  As the norm in front of a part it rides on the fused residual-add kernel (`fused_pre`); behind
+    a part it runs through `forward`."""
+    graph_safe = True
+
+    def __init__(self, precision: Precision, *, dim: int, eps: float, tensor_name: str = "weight", bias_name: str = "bias"):
+        self.precision = precision
+        self.dim, self.eps = dim, float(eps)
+        self.tensor_name, self.bias_name = tensor_name, bias_name
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return {self.tensor_name: ParamSpec((self.dim,), init_std=0.1), self.bias_name: ParamSpec((self.dim,), init_std=0.1)}
+
+    def assign(self, name: str, tensor: torch.Tensor) -> None:
+        if name == self.tensor_name:
+            self.weight = tensor.float().contiguous()
+        elif name == self.bias_name:
+            self.bias = tensor.float().contiguous()
+        else:
+            raise KeyError(name)
+
+    def fused_pre(self) -> Tuple[torch.Tensor, float, float, torch.Tensor]:
+        """(weight, eps, offset, bias) for the fused residual-add kernel, as the norm of the stream's new rows."""
+        return self.weight, self.eps, 0.0, self.bias
+
+    def forward(self, x: torch.Tensor, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """x: float32 [T, dim]; with `rows` only these rows are normed (in their order)."""
+        n = x.shape[0] if rows is None else rows.numel()
+        out = torch.empty((n, self.dim), dtype=out_dtype, device=x.device)
+        ops.add_norm(x, None, None, self.weight, out, eps_pre=self.eps, b_pre=self.bias, rows=rows,
+                     full_precision=self.precision.full)
         return out

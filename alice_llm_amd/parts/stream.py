@@ -19,6 +19,16 @@ from .base import FragmentActs, Precision
 ADD_BRANCHES_FROM_ROWS = 256
 
 
+def _fused_pre(norm):
+    """(weight, eps, offset, bias or None) of a norm that the fused add-and-norm kernel can apply to the new rows, else None."""
+    if norm is None:
+        return None
+    if hasattr(norm, "fused_pre"):
+        return norm.fused_pre()
+    f = norm.fused() if hasattr(norm, "fused") else None
+    return None if f is None else (*f, None)
+
+
 class ResidualStream:
     def __init__(self, x: torch.Tensor, precision: Precision):
         assert x.dtype == torch.float32 and x.dim() == 2
@@ -96,7 +106,7 @@ class ResidualStream:
                 self._flush_many(out)
                 return out
             self._flush_many()
-        pre = norm.fused() if norm is not None and hasattr(norm, "fused") else None
+        pre = _fused_pre(norm)
         if fragments and pre is not None and out_dtype == torch.bfloat16 and FragmentActs.possible(self.precision, T, H):
             post = self._post
             pf = post.fused() if post is not None and hasattr(post, "fused") else None
@@ -106,7 +116,7 @@ class ResidualStream:
             w_post, eps_post, off_post = pf if (pf is not None and b is not None) else (None, 0.0, 0.0)
             out = FragmentActs.empty(T, H, self.x.device)
             ops.add_norm(self.x, b, w_post, pre[0], out.data, eps_post=eps_post, eps_pre=pre[1], off_post=off_post,
-                         off_pre=pre[2], n_partials=n, full_precision=self.precision.full, out_layout=ops.LAYOUT_FRAG16)
+                         off_pre=pre[2], b_pre=pre[3], n_partials=n, full_precision=self.precision.full, out_layout=ops.LAYOUT_FRAG16)
             self._branch = None
             self._post = None
             return out
@@ -118,9 +128,9 @@ class ResidualStream:
                 n, b = self._partials()
                 out = torch.empty((T, H), dtype=out_dtype, device=self.x.device)
                 w_post, eps_post, off_post = pf if pf is not None else (None, 0.0, 0.0)
-                w_pre, eps_pre, off_pre = pre if pre is not None else (None, 0.0, 0.0)
+                w_pre, eps_pre, off_pre, b_pre = pre if pre is not None else (None, 0.0, 0.0, None)
                 ops.add_norm(self.x, b, w_post, w_pre, out, eps_post=eps_post, eps_pre=eps_pre,
-                             off_post=off_post, off_pre=off_pre, n_partials=n,
+                             off_post=off_post, off_pre=off_pre, b_pre=b_pre, n_partials=n,
                              full_precision=self.precision.full)
                 self._branch = None
                 self._post = None
@@ -134,11 +144,11 @@ class ResidualStream:
         """norm(x[rows]) after all pending adds: what the output head reads."""
         self.flush()
         out_dtype = out_dtype or self.precision.act
-        pre = norm.fused() if norm is not None and hasattr(norm, "fused") else None
+        pre = _fused_pre(norm)
         if fragments and pre is not None and out_dtype == torch.bfloat16 and \
                 FragmentActs.possible(self.precision, rows.numel(), self.x.shape[1]):
             out = FragmentActs.empty(rows.numel(), self.x.shape[1], self.x.device)
-            ops.add_norm(self.x, None, None, pre[0], out.data, eps_pre=pre[1], off_pre=pre[2], rows=rows,
+            ops.add_norm(self.x, None, None, pre[0], out.data, eps_pre=pre[1], off_pre=pre[2], b_pre=pre[3], rows=rows,
                          full_precision=self.precision.full, out_layout=ops.LAYOUT_FRAG16)
             return out
         if norm is None:
