@@ -218,6 +218,11 @@ int alice_expert_products(const void* x, const float* weights, const void* gate_
 // of the identity outputs together, and with has_shared sigmoid(z[t, n]) (else 0).
 int alice_route_scored(const float* z, int z_w, const float* correction, float* w, float* side, int T, int experts, int identity,
                        int top, int groups, int keep, int has_shared, hipStream_t stream);
+// The routed feed-forward for at most 64 tokens: only the chosen experts' matrices are read, the shared expert is one more.
+int alice_expert_few_splits(int W);
+int alice_expert_few(const void* x, const float* w, const float* side, const void* gate_up, const void* down, const void* shared_gate_up,
+                     const void* shared_down, void* mid, float* out, int T, int W, int F, int E, int shared_width, float epi,
+                     float shared_epi, hipStream_t stream);
 // y[t] = sum of n_base partial rows base[s][t] + side[t][0] x[t] + side[t][1] (sum of n_shared partial rows shared[s][t]).
 int alice_expert_combine(const float* base, int n_base, const void* x, int x_dtype, const float* side, const float* shared, int n_shared,
                          float* y, int T, int W, hipStream_t stream);

@@ -88,6 +88,11 @@ __device__ __forceinline__ float block_max(float v, float* red) {
   return red[16];
 }
 
+// A barrier between phases that exchange data through LDS only: it waits for the wave's LDS accesses, not for its
+// loads and stores of global memory (rows fetched ahead, results on their way out), which __syncthreads() would also
+// wait for at every phase.
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // tanh at full precision for the 32-bit path, a fast form for the bfloat16 path.
 __device__ __forceinline__ float tanh_full(float x) { return tanhf(x); }
 __device__ __forceinline__ float tanh_fast(float x) {

@@ -21,6 +21,13 @@
 // tokens' rows, and writes act(gate) * up * routing weight, rounded once.  expert_down_kernel is the same walk over
 // the expert's slice of the inner dimension of the side-by-side down matrices; expert_combine_kernel adds a token's
 // rows.  Only the experts that tokens chose are read, and each row meets only its own expert.
+//
+// Steps of few tokens read every chosen expert's matrices once and do little else (expert_few_*): a block of the first
+// kernel takes one expert and 16 of its middle columns, and ends at once if no token of the step chose it; its four waves
+// share the inner dimension and meet in LDS.  A block of the second takes 16 outputs and every splits-th of the chosen
+// experts, with the tokens as the columns of all its products (zeros where a token did not choose the expert), and leaves
+// partial sums for the residual add.  The shared expert is one more expert with sizes of its own, chosen by every token,
+// and the identity experts' share is added by the first split.  Which experts are chosen is read on the device.
 #include "linear_mfma.h"
 
 namespace {
@@ -323,32 +330,220 @@ __global__ __launch_bounds__(256) void expert_down_kernel(const bf16_t* __restri
   }
 }
 
+// ------------------------------------------------------------------------------------------ few tokens
+
+struct FewArgs {
+  const bf16_t* x;                     // [T, W]
+  const float* w;                      // [T, E], zero: not chosen
+  const float* side;                   // [T, 2] or null: (identity weight, the shared expert's gate)
+  const bf16_t* gate_up;               // fragment layout of [2 E F, W]
+  const bf16_t* down;                  // fragment layout of [W, E F]
+  const bf16_t* shared_gate_up;        // fragment layout of [2 Fs, W], or null
+  const bf16_t* shared_down;           // fragment layout of [W, Fs]
+  bf16_t* mid;                         // [T, E F + Fs]
+  float* out;                          // [splits, T, W]
+  int T, W, F, E, Fs, splits;
+  float epi, shared_epi;
+};
+
+// The weight with which token t uses expert e (e == E: the shared one).
+__device__ __forceinline__ float few_weight(const FewArgs& a, int t, int e) {
+  if (t >= a.T) return 0.f;
+  return e < a.E ? a.w[(size_t)t * a.E + e] : a.side[2 * (size_t)t + 1];
+}
+
+template <int RS>
+__global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
+  __shared__ f32x4 part[4][RS][2][64];
+  const int e = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+  const bool shared = e == a.E;
+  const int F = shared ? a.Fs : a.F, f0 = blockIdx.x * 16;
+  if (f0 >= F) return;
+  const float wt = few_weight(a, lane, e);                // lane = token (at most 64)
+  const unsigned long long used = __ballot(wt != 0.f);
+  if (used == 0ull) return;
+  const int KT = (a.W + 31) / 32;
+  const bf16_t* base = shared ? a.shared_gate_up : a.gate_up;
+  const int first = shared ? f0 : e * F + f0, half = shared ? F : a.E * F;
+  const bf16_t* wg = base + (size_t)(first / 16) * KT * 512 + lane * 8;
+  const bf16_t* wu = base + (size_t)((half + first) / 16) * KT * 512 + lane * 8;
+  const bf16_t* xr[RS];
+  bool on[RS];
+#pragma unroll
+  for (int s = 0; s < RS; ++s) {
+    on[s] = ((used >> (16 * s)) & 0xffffull) != 0ull;
+    xr[s] = a.x + (size_t)min(s * 16 + c, a.T - 1) * a.W;
+  }
+  f32x4 ag[RS], au[RS];
+#pragma unroll
+  for (int s = 0; s < RS; ++s) ag[s] = au[s] = f32x4{0.f, 0.f, 0.f, 0.f};
+  auto step = [&](int kt, u32x4 vg, u32x4 vu) {
+    const int k = min(kt * 32 + g * 8, a.W - 8);          // a row's last, partial k-tile: the weights are zero there
+#pragma unroll
+    for (int s = 0; s < RS; ++s) {
+      if (!on[s]) continue;
+      const u32x4 b = *reinterpret_cast<const u32x4*>(xr[s] + k);
+      ag[s] = mfma16(vg, b, ag[s]);
+      au[s] = mfma16(vu, b, au[s]);
+    }
+  };
+  constexpr int U = 8;                                    // weight tiles in flight: 2 U loads of 1 KB a wave
+  int kt = wave;
+  for (; kt + 4 * (U - 1) < KT; kt += 4 * U) {
+    u32x4 vg[U], vu[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      vg[u] = *reinterpret_cast<const u32x4*>(wg + (size_t)(kt + 4 * u) * 512);
+      vu[u] = *reinterpret_cast<const u32x4*>(wu + (size_t)(kt + 4 * u) * 512);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) step(kt + 4 * u, vg[u], vu[u]);
+  }
+  for (; kt < KT; kt += 4)
+    step(kt, *reinterpret_cast<const u32x4*>(wg + (size_t)kt * 512), *reinterpret_cast<const u32x4*>(wu + (size_t)kt * 512));
+#pragma unroll
+  for (int s = 0; s < RS; ++s) {
+    part[wave][s][0][lane] = ag[s];
+    part[wave][s][1][lane] = au[s];
+  }
+  __syncthreads();
+  for (int s = wave; s < RS; s += 4) {
+    const int t = s * 16 + c;
+    const float wr = __shfl(wt, t, 64);
+    f32x4 gs = part[0][s][0][lane], us = part[0][s][1][lane];
+#pragma unroll
+    for (int n = 1; n < 4; ++n) {
+      gs += part[n][s][0][lane];
+      us += part[n][s][1][lane];
+    }
+    f32x4 o;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = gated_act(gs[i], us[i], shared ? a.shared_epi : a.epi, false) * wr;
+    if (t < a.T && wr != 0.f) store4(a.mid, (size_t)t * (a.E * a.F + a.Fs), e * a.F + f0 + g * 4, e * a.F + F, o);
+  }
+}
+
+template <int RS>
+__global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
+  __shared__ unsigned short list[MAX_EXPERTS + 1];
+  __shared__ int n_list;
+  __shared__ f32x4 part[4][RS][64];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, c = lane & 15;
+  const int n0 = blockIdx.x * 16, z = blockIdx.y, n_exp = a.E + (a.Fs > 0 ? 1 : 0), row = a.E * a.F + a.Fs;
+  if (wave == 0) {                                        // the chosen experts in their order
+    int n = 0;
+    for (int e0 = 0; e0 < n_exp; e0 += 64) {
+      const int e = e0 + lane;
+      bool any = false;
+      if (e < n_exp)
+        for (int t = 0; t < a.T; ++t) any = any || few_weight(a, t, e) != 0.f;
+      const unsigned long long m = __ballot(any);
+      if (any) list[n + __popcll(m & ((1ull << lane) - 1ull))] = (unsigned short)e;
+      n += __popcll(m);
+    }
+    if (lane == 0) n_list = n;
+  }
+  __syncthreads();
+  const int KT = (a.E * a.F + 31) / 32, KTS = (a.Fs + 31) / 32;
+  f32x4 acc[RS];
+#pragma unroll
+  for (int s = 0; s < RS; ++s) acc[s] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = z; i < n_list; i += a.splits) {
+    const int e = list[i];
+    const bool shared = e == a.E;
+    const int kts = (shared ? a.Fs : a.F) / 32;           // F and Fs are multiples of 32: an expert's k-tiles are its own
+    const bf16_t* wd = (shared ? a.shared_down + (size_t)(n0 / 16) * KTS * 512 : a.down + ((size_t)(n0 / 16) * KT + e * a.F / 32) * 512) + lane * 8;
+    bool use[RS], on[RS];
+    const bf16_t* mr[RS];
+#pragma unroll
+    for (int s = 0; s < RS; ++s) {
+      const int t = s * 16 + c;
+      use[s] = few_weight(a, t, e) != 0.f;
+      on[s] = __ballot(use[s]) != 0ull;
+      mr[s] = a.mid + (size_t)min(t, a.T - 1) * row + e * a.F + g * 8;
+    }
+    auto step = [&](int kt, u32x4 v) {
+#pragma unroll
+      for (int s = 0; s < RS; ++s) {
+        if (!on[s]) continue;
+        u32x4 b = {0u, 0u, 0u, 0u};
+        if (use[s]) b = *reinterpret_cast<const u32x4*>(mr[s] + kt * 32);
+        acc[s] = mfma16(v, b, acc[s]);
+      }
+    };
+    constexpr int U = 8;
+    int kt = wave;
+    for (; kt + 4 * (U - 1) < kts; kt += 4 * U) {
+      u32x4 v[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) v[u] = *reinterpret_cast<const u32x4*>(wd + (size_t)(kt + 4 * u) * 512);
+#pragma unroll
+      for (int u = 0; u < U; ++u) step(kt + 4 * u, v[u]);
+    }
+    for (; kt < kts; kt += 4) step(kt, *reinterpret_cast<const u32x4*>(wd + (size_t)kt * 512));
+  }
+#pragma unroll
+  for (int s = 0; s < RS; ++s) part[wave][s][lane] = acc[s];
+  __syncthreads();
+  for (int s = wave; s < RS; s += 4) {
+    const int t = s * 16 + c, n = n0 + g * 4;
+    if (t >= a.T) continue;
+    f32x4 o = (part[0][s][lane] + part[1][s][lane]) + (part[2][s][lane] + part[3][s][lane]);
+    if (z == 0 && a.side) {
+      const float id = a.side[2 * (size_t)t];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n + i < a.W) o[i] = fmaf(id, bf16_to_f32(a.x[(size_t)t * a.W + n + i]), o[i]);
+    }
+    store4(a.out + (size_t)z * a.T * a.W, (size_t)t * a.W, n, a.W, o);
+  }
+}
+
 // y[t, c] = the sum of the token's rows of `rows` [R, W], or of the n_base partial rows base[s][t]; with `side` also
 // side[t][0] x[t, c] (the identity experts give the input back) + side[t][1] * (the sum of the shared expert's partial rows).
-template <typename TX>
+template <typename TX, int V>
 __global__ void expert_combine_kernel(const float* __restrict__ rows, const int* __restrict__ token_rows, int top,
                                       const float* __restrict__ base, int n_base, const TX* __restrict__ x, const float* __restrict__ side,
                                       const float* __restrict__ shared, int n_shared, float* __restrict__ y, int T, int W) {
-  const int t = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  const int t = blockIdx.x, c = (blockIdx.y * blockDim.x + threadIdx.x) * V;       // V neighbouring columns a thread (W a multiple of V)
   if (c >= W) return;
   const size_t at = (size_t)t * W + c, all = (size_t)T * W;
-  float s = 0.f;
+  float s[V], u[V];
+#pragma unroll
+  for (int i = 0; i < V; ++i) s[i] = u[i] = 0.f;
+  auto add = [&](float (&d)[V], const float* p) {
+    if constexpr (V == 4) {
+      const float4 v = *reinterpret_cast<const float4*>(p);
+      d[0] += v.x; d[1] += v.y; d[2] += v.z; d[3] += v.w;
+    } else {
+      d[0] += p[0];
+    }
+  };
   if (rows) {
     for (int j = 0; j < top; ++j) {
       const int r = token_rows[(size_t)t * top + j];
-      if (r >= 0) s += rows[(size_t)r * W + c];
+      if (r >= 0) add(s, rows + (size_t)r * W + c);
     }
   }
-  for (int i = 0; i < n_base; ++i) s += base[i * all + at];
+  for (int i = 0; i < n_base; ++i) add(s, base + i * all + at);
   if (side) {
-    s = fmaf(side[2 * (size_t)t], load_f32(x, at), s);
-    if (n_shared > 0) {
-      float u = 0.f;
-      for (int i = 0; i < n_shared; ++i) u += shared[i * all + at];
-      s = fmaf(side[2 * (size_t)t + 1], u, s);
-    }
+    const float id = side[2 * (size_t)t], sg = side[2 * (size_t)t + 1];
+    for (int i = 0; i < n_shared; ++i) add(u, shared + i * all + at);
+#pragma unroll
+    for (int i = 0; i < V; ++i) s[i] = fmaf(sg, u[i], fmaf(id, load_f32(x, at + i), s[i]));
   }
-  y[at] = s;
+  if constexpr (V == 4) *reinterpret_cast<float4*>(y + at) = float4{s[0], s[1], s[2], s[3]};
+  else y[at] = s[0];
+}
+
+// Four columns a thread where rows are whole 16-byte units.
+template <typename TX>
+void launch_combine(const float* rows, const int* token_rows, int top, const float* base, int n_base, const TX* x, const float* side,
+                    const float* shared, int n_shared, float* y, int T, int W, hipStream_t stream) {
+  if (W % 4 == 0 && (((uintptr_t)rows | (uintptr_t)base | (uintptr_t)shared | (uintptr_t)y) & 15) == 0)
+    expert_combine_kernel<TX, 4><<<dim3(T, ceil_div(W, 1024)), 256, 0, stream>>>(rows, token_rows, top, base, n_base, x, side, shared, n_shared, y, T, W);
+  else
+    expert_combine_kernel<TX, 1><<<dim3(T, ceil_div(W, 256)), 256, 0, stream>>>(rows, token_rows, top, base, n_base, x, side, shared, n_shared, y, T, W);
 }
 
 }  // namespace
@@ -385,8 +580,41 @@ extern "C" int alice_expert_products(const void* x, const float* weights, const 
   dim3 g2((unsigned)(R / GROUP_TILE), ceil_div(W, 256));
   expert_down_kernel<4><<<g2, 256, 0, stream>>>((const bf16_t*)mid, (const bf16_t*)down, tile_expert, rows, W, F, E);
   ALICE_LAUNCH_CHECK();
-  dim3 g3(T, ceil_div(W, 256));
-  expert_combine_kernel<bf16_t><<<g3, 256, 0, stream>>>(rows, token_rows, top, nullptr, 0, (const bf16_t*)x, side, shared, n_shared, y, T, W);
+  launch_combine<bf16_t>(rows, token_rows, top, nullptr, 0, (const bf16_t*)x, side, shared, n_shared, y, T, W, stream);
+  ALICE_LAUNCH_CHECK();
+  return 0;
+}
+
+// How many partial sums alice_expert_few leaves: enough blocks for the chip.
+extern "C" int alice_expert_few_splits(int W) {
+  const int s = 512 / ceil_div(W, 16);
+  return s < 1 ? 1 : (s > 8 ? 8 : s);
+}
+
+// The routed feed-forward for at most 64 tokens, see expert_few_*_kernel.  x: [T, W] bfloat16; w: [T, E]; gate_up, down,
+// shared_gate_up, shared_down: fragment layouts (the latter two null and shared_width 0 without a shared expert); side
+// [T, 2] or null; mid: [T, E F + shared_width] bfloat16; out: [alice_expert_few_splits(W), T, W] float32 partial sums.
+extern "C" int alice_expert_few(const void* x, const float* w, const float* side, const void* gate_up, const void* down,
+                                const void* shared_gate_up, const void* shared_down, void* mid, float* out, int T, int W, int F, int E,
+                                int shared_width, float epi, float shared_epi, hipStream_t stream) {
+  ALICE_CHECK(x && w && gate_up && down && mid && out, "expert_few: a pointer is missing");
+  ALICE_CHECK(T >= 1 && T <= 64 && E >= 1 && E <= MAX_EXPERTS, "expert_few: %d tokens (1..64) or %d experts (1..%d)", T, E, MAX_EXPERTS);
+  ALICE_CHECK(W >= 8 && W % 8 == 0 && F >= 32 && F % 32 == 0 && shared_width >= 0 && shared_width % 32 == 0,
+              "expert_few: the width must be a multiple of 8 and the experts' of 32");
+  ALICE_CHECK(shared_width == 0 || (side && shared_gate_up && shared_down), "expert_few: a shared expert needs its matrices and its gate");
+  FewArgs a{(const bf16_t*)x, w, side, (const bf16_t*)gate_up, (const bf16_t*)down, (const bf16_t*)shared_gate_up, (const bf16_t*)shared_down,
+            (bf16_t*)mid, out, T, W, F, E, shared_width, alice_expert_few_splits(W), epi, shared_epi};
+  const dim3 g1(ceil_div(F > shared_width ? F : shared_width, 16), E + (shared_width > 0 ? 1 : 0)), g2(ceil_div(W, 16), a.splits);
+#define GO(RS)                                                      \
+  do {                                                              \
+    expert_few_gate_up_kernel<RS><<<g1, 256, 0, stream>>>(a);       \
+    ALICE_LAUNCH_CHECK();                                           \
+    expert_few_down_kernel<RS><<<g2, 256, 0, stream>>>(a);          \
+  } while (0)
+  if (T <= 16) GO(1);
+  else if (T <= 32) GO(2);
+  else GO(4);
+#undef GO
   ALICE_LAUNCH_CHECK();
   return 0;
 }
@@ -419,9 +647,7 @@ extern "C" int alice_expert_combine(const float* base, int n_base, const void* x
   ALICE_CHECK(base && n_base >= 1 && x && side && y && dtype_ok(x_dtype), "expert_combine: a pointer is missing or the dtype is unknown");
   ALICE_CHECK(T >= 0 && W >= 1 && n_shared >= 0 && (n_shared == 0 || shared), "expert_combine: bad sizes");
   if (T == 0) return 0;
-  const dim3 grid(T, ceil_div(W, 256));
-  DISPATCH_DTYPE(x_dtype, TX, (expert_combine_kernel<TX><<<grid, 256, 0, stream>>>(nullptr, nullptr, 0, base, n_base, (const TX*)x, side, shared,
-                                                                                 n_shared, y, T, W)));
+  DISPATCH_DTYPE(x_dtype, TX, (launch_combine<TX>(nullptr, nullptr, 0, base, n_base, (const TX*)x, side, shared, n_shared, y, T, W, stream)));
   ALICE_LAUNCH_CHECK();
   return 0;
 }

@@ -318,13 +318,13 @@ __global__ __launch_bounds__(256) void latent_tiled_kernel(LatentArgs a) {
   }
 }
 
-// One row a block: out = sum_z exp(m_z - M) o_z / sum_z exp(m_z - M) l_z, M the largest of the m_z.  The splits'
+// 128 elements of one row a block: out = sum_z exp(m_z - M) o_z / sum_z exp(m_z - M) l_z, M the largest of the m_z.  The splits'
 // maxima and sums are read once into LDS, a split's weight is computed once, and the row's elements are added up with
 // several loads in flight.
 __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ part, bf16_t* __restrict__ out,
                                                            int splits, long rows_total, int R) {
   const size_t row = blockIdx.x;
-  const int t = threadIdx.x;
+  const int t = threadIdx.x, e0 = blockIdx.y * 128;
   __shared__ float mz[32], lz[32], wz[32];
   if (t < 32) {
     float m = -INFINITY, l = 0.f;
@@ -347,21 +347,20 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restri
   }
   __syncthreads();
   const size_t stride = (size_t)rows_total * (R + 2);
-  for (int e = t; e < R; e += blockDim.x) {
-    const float* p = part + row * (size_t)(R + 2) + e;
-    float o = 0.f;
-    int z = 0;
-    for (; z + 4 <= splits; z += 4) {                    // four loads in flight
-      const float a0 = p[(size_t)z * stride], a1 = p[(size_t)(z + 1) * stride], a2 = p[(size_t)(z + 2) * stride],
-                  a3 = p[(size_t)(z + 3) * stride];
-      o = fmaf(wz[z], a0, o);
-      o = fmaf(wz[z + 1], a1, o);
-      o = fmaf(wz[z + 2], a2, o);
-      o = fmaf(wz[z + 3], a3, o);
-    }
-    for (; z < splits; ++z) o = fmaf(wz[z], p[(size_t)z * stride], o);
-    out[row * R + e] = f32_to_bf16(o);
+  const int e = e0 + t;
+  if (e >= R) return;
+  const float* p = part + row * (size_t)(R + 2) + e;
+  float o = 0.f;
+  int z = 0;
+  for (; z + 8 <= splits; z += 8) {                      // eight loads in flight
+    float v[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = p[(size_t)(z + i) * stride];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o = fmaf(wz[z + i], v[i], o);
   }
+  for (; z < splits; ++z) o = fmaf(wz[z], p[(size_t)z * stride], o);
+  out[row * R + e] = f32_to_bf16(o);
 }
 
 // ------------------------------------------------------------------------------------- a matrix a head, matrix cores
@@ -541,7 +540,7 @@ extern "C" int alice_latent_tiled(const void* q, const void* pool, void* out, fl
   if (rc) return rc;
   ALICE_LAUNCH_CHECK();
   if (splits > 1) {
-    latent_merge_kernel<<<(unsigned)rows_total, 128, 0, stream>>>(part, (bf16_t*)out, splits, rows_total, kv_rank);
+    latent_merge_kernel<<<dim3((unsigned)rows_total, ceil_div(kv_rank, 128)), 128, 0, stream>>>(part, (bf16_t*)out, splits, rows_total, kv_rank);
     ALICE_LAUNCH_CHECK();
   }
   return 0;

@@ -182,17 +182,29 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
     const int j = tid / 4, k = (tid % 4) * 4;
     pv = raw4<TX>(a, (size_t)(c0 + j) * a.row_w + a.v_col + h * dv + v0 + k, j < len ? dv - v0 - k : 0);
   };
+  // the decays to the chunk's end of the tokens whose keys this thread stages: fixed but for the last, shorter chunk
+  float pwk[NK];
+  auto weights = [&](int len) {
+#pragma unroll
+    for (int u = 0; u < NK; ++u) {
+      const int j = (tid + u * NT) / (DP / 4);
+      pwk[u] = j < len ? pw[len - 1 - j] : 0.f;
+    }
+  };
   fetch(t0);
+  weights(min(CHUNK, t1 - t0));
   for (int c0 = t0; c0 < t1; c0 += CHUNK, ++chunk) {
     const int len = min(CHUNK, t1 - c0);
+    if (len < CHUNK && c0 != t0) weights(len);
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int i = tid + u * NT, j = i / (DP / 4), k = (i % (DP / 4)) * 4;
-      const float w = j < len ? pw[len - 1 - j] : 0.f;
       const float4 x = activated(a, pk[u]);
-      *reinterpret_cast<float4*>(Ks + j * KS + k) = float4{x.x * w, x.y * w, x.z * w, x.w * w};
+      *reinterpret_cast<float4*>(Ks + j * KS + k) = float4{x.x * pwk[u], x.y * pwk[u], x.z * pwk[u], x.w * pwk[u]};
     }
     *reinterpret_cast<float4*>(Vs + (tid / 4) * 16 + (tid % 4) * 4) = activated(a, pv);
+    const float keep = pw[len];
+    if (c0 + CHUNK < t1) fetch(c0 + CHUNK);                // on its way during the products (the barriers wait for LDS only)
     float* dst = a.states + (chunk * H + h) * d * dv;
 #pragma unroll
     for (int i = 0; i < TW; ++i)
@@ -201,9 +213,7 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
         const int r = r0 + i * 16 + e;
         if (col_ok && r < d) dst[(size_t)r * dv + col] = acc[i][e];
       }
-    if (c0 + CHUNK < t1) fetch(c0 + CHUNK);
-    __syncthreads();
-    const float keep = pw[len];
+    lds_barrier();
     f32x4_t c1[TW], c2[TW];
 #pragma unroll
     for (int i = 0; i < TW; ++i) c1[i] = c2[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -222,7 +232,7 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
     for (int i = 0; i < TW; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc[i][e] = fmaf(keep, acc[i][e], c1[i][e] + c2[i][e]);
-    __syncthreads();                                       // the buffers have been read
+    lds_barrier();                                         // the buffers have been read
   }
 #pragma unroll
   for (int i = 0; i < TW; ++i)
@@ -320,19 +330,44 @@ __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) 
 #pragma unroll
       for (int i = 0; i < 4; ++i) acc[c][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
-    const float* qa = Qs + (lane & 15) * QS + (lane >> 4);
-#pragma unroll 4
-    for (int kk = 0; kk < DP; kk += 4) {
-      const int r = kk + (lane >> 4);
-      float b[CT];
+    // four products' elements of the state, then of the values, are fetched while the four before them are multiplied
+    float b[4][CT], bn[4][CT];
+    auto fetch_state = [&](int kk) {
 #pragma unroll
-      for (int c = 0; c < CT; ++c) b[c] = (ok[c] && r < d) ? S0[(size_t)r * dv + col[c]] : 0.f;
+      for (int n = 0; n < 4; ++n) {
+        const int r = kk + n * 4 + (lane >> 4);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float q = qa[i * 16 * QS + kk];
-#pragma unroll
-        for (int c = 0; c < CT; ++c) acc[c][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, b[c], acc[c][i], 0, 0, 0);
+        for (int c = 0; c < CT; ++c) bn[n][c] = (ok[c] && r < d) ? S0[(size_t)r * dv + col[c]] : 0.f;
       }
+    };
+    auto fetch_values = [&](int kk) {
+#pragma unroll
+      for (int n = 0; n < 4; ++n) {
+        const int j = kk + n * 4 + (lane >> 4);
+#pragma unroll
+        for (int c = 0; c < CT; ++c)
+          bn[n][c] = (ok[c] && j < len) ? load_f32(reinterpret_cast<const TX*>(a.rows), (size_t)(c0 + j) * a.row_w + a.v_col + h * dv + col[c]) : 0.f;
+      }
+    };
+    auto take = [&]() {
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) b[n][c] = bn[n][c];
+    };
+    const float* qa = Qs + (lane & 15) * QS + (lane >> 4);
+    fetch_state(0);
+    for (int kk = 0; kk < DP; kk += 16) {
+      take();
+      if (kk + 16 < DP) fetch_state(kk + 16); else fetch_values(0);
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float q = qa[i * 16 * QS + kk + n * 4];
+#pragma unroll
+          for (int c = 0; c < CT; ++c) acc[c][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, b[n][c], acc[c][i], 0, 0, 0);
+        }
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
@@ -344,17 +379,22 @@ __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) 
       }
     const float* pa = Ks + (lane & 15) * PS + (lane >> 4);
 #pragma unroll
-    for (int kk = 0; kk < CHUNK; kk += 4) {
-      const int j = kk + (lane >> 4);
-      float b[CT];
+    for (int g = 0; g < 4; ++g) {
+      take();
+      if (g < 3) fetch_values(g * 16 + 16);
 #pragma unroll
-      for (int c = 0; c < CT; ++c)
-        b[c] = (ok[c] && j < len) ? in1<TX>(a, (size_t)(c0 + j) * a.row_w + a.v_col + h * dv + col[c]) : 0.f;
+      for (int n = 0; n < 4; ++n) {
+        const int kk = g * 16 + n * 4;
+        if (a.act) {
 #pragma unroll
-      for (int i = kk / 16; i < 4; ++i) {
-        const float q = pa[i * 16 * PS + kk];
+          for (int c = 0; c < CT; ++c) b[n][c] = silu_f(b[n][c]);
+        }
 #pragma unroll
-        for (int c = 0; c < CT; ++c) acc[c][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, b[c], acc[c][i], 0, 0, 0);
+        for (int i = g; i < 4; ++i) {
+          const float q = pa[i * 16 * PS + kk];
+#pragma unroll
+          for (int c = 0; c < CT; ++c) acc[c][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, b[n][c], acc[c][i], 0, 0, 0);
+        }
       }
     }
 #pragma unroll

@@ -156,11 +156,6 @@ __global__ void gelu_mul_rows_kernel(const TZ* __restrict__ z, const TW* __restr
 // are read as 2 rows x 16 neighbours only: 16 mod 32.
 __host__ __device__ __forceinline__ int lds_stride18(int d) { return d + ((18 - d % 32 + 32) % 32); }
 
-// A barrier between phases that exchange data through LDS only: it waits for the wave's LDS accesses, not for its
-// loads and stores of global memory (the rows fetched ahead, the read-outs on their way out), which __syncthreads()
-// would also wait for at every phase.
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
 // acc += sum over k < n (a multiple of 16) of A(k) B(k), four k at a time, as four chains of products that do not
 // wait for each other (a product that adds to the one before it waits for its result, about twice the time the
 // matrix unit is busy with it); the chains are added at the end.

@@ -76,6 +76,8 @@ def _declare(lib) -> None:
         "alice_route_topk": [P, P, P, I, I, I, P],
         "alice_scale_columns": [P, I, P, P, I, I, I, I, P],
         "alice_expert_products": [P, P, P, P, P, P, P, P, I, I, I, I, I, F, P, P, I, P],
+        "alice_expert_few_splits": [I],
+        "alice_expert_few": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, F, P],
         "alice_route_scored": [P, I, P, P, P, I, I, I, I, I, I, I, P],
         "alice_expert_combine": [P, I, P, I, P, P, I, P, I, I, P],
         "alice_lightning": [P, I, I, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
@@ -1214,6 +1216,35 @@ def scale_columns(x: torch.Tensor, weights: torch.Tensor, out: torch.Tensor) -> 
 def expert_products_supported(dtype: torch.dtype, width: int, expert_width: int) -> bool:
     """Whether expert_products takes these operands: bfloat16, a width that is a multiple of 8 and experts of a multiple of 32."""
     return dtype == torch.bfloat16 and width >= 8 and width % 8 == 0 and expert_width >= 32 and expert_width % 32 == 0
+
+
+EXPERT_FEW_MAX_TOKENS = 64
+
+
+def expert_few(x: torch.Tensor, weights: torch.Tensor, side: Optional[torch.Tensor], gate_up: torch.Tensor, down: torch.Tensor, *,
+               expert_width: int, epi_param: float, shared_gate_up: Optional[torch.Tensor] = None,
+               shared_down: Optional[torch.Tensor] = None, shared_width: int = 0, shared_epi_param: float = 0.0) -> torch.Tensor:
+    """expert_products for at most EXPERT_FEW_MAX_TOKENS tokens, with every chosen expert's matrices read once; returns
+    float32 partial sums [S, T, W].  With side: plus side[t, 0] x[t], and with the shared expert's matrices (of width
+    shared_width, a multiple of 32) plus side[t, 1] times its output."""
+    T, W = x.shape
+    E, F, Fs = weights.shape[1], int(expert_width), int(shared_width)
+    if not expert_products_supported(x.dtype, W, F) or Fs % 32 or not 1 <= T <= EXPERT_FEW_MAX_TOKENS:
+        raise HipLibraryError("expert_few: bfloat16, a width that is a multiple of 8, experts of a multiple of 32, few tokens")
+    wide = -(-W // 32) * 32
+    _dev(x, "x", torch.bfloat16)
+    _dev(weights, "weights", torch.float32, (T, E))
+    _dev(gate_up, "gate_up", torch.bfloat16, (frag_rows(2 * E * F) * wide,))
+    _dev(down, "down", torch.bfloat16, (frag_rows(W) * (E * F),))
+    if Fs:
+        _dev(shared_gate_up, "shared_gate_up", torch.bfloat16, (2 * Fs * wide,))
+        _dev(shared_down, "shared_down", torch.bfloat16, (frag_rows(W) * Fs,))
+    mid = torch.empty((T, E * F + Fs), dtype=torch.bfloat16, device=x.device)
+    out = torch.empty((library().alice_expert_few_splits(W), T, W), dtype=torch.float32, device=x.device)
+    _call("alice_expert_few", x.data_ptr(), weights.data_ptr(), _opt(side, "side", torch.float32, (T, 2)), gate_up.data_ptr(), down.data_ptr(),
+          _opt(shared_gate_up, "shared_gate_up") if Fs else None, _opt(shared_down, "shared_down") if Fs else None, mid.data_ptr(),
+          out.data_ptr(), T, W, F, E, Fs, float(epi_param), float(shared_epi_param), _stream())
+    return out
 
 
 def expert_products(x: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, y: torch.Tensor, *,

@@ -4,11 +4,12 @@ Router logits z = R h + r in 32-bit; the `top` best-scoring experts serve the to
 wins) and are mixed by a softmax restricted to those `top` logits: y = sum_e w_e down_e(act(gate_e h) * (up_e h)).  Tensors: "router", "router.b", and "e<i>.gate", "e<i>.up", "e<i>.down" for every expert.
 
 The experts' gate and up matrices are stacked into one matrix at load, and their down matrices side by side into
-another.  Steps of few tokens, the 32-bit path and sizes that suit no tile: one gated product gives every expert's
+another.  The 32-bit path, sizes that suit no tile and steps in between: one gated product gives every expert's
 middle activations, each is multiplied by its expert's weight of that token (zero where the token does not use the
 expert), and one down projection over all of them is the weighted sum.  Steps of many tokens in bfloat16: the (token,
 expert) pairs are put in expert order on the device and each pair meets its own expert's matrices only (grouped
-products over the same stacked matrices).  Every kernel's launch depends on sizes only, never on which experts the
+products over the same stacked matrices).  Steps of few tokens in bfloat16, of which many experts serve none: the chosen
+experts' matrices are read, the others' are not.  Every kernel's launch depends on sizes only, never on which experts the
 tokens chose.
 
 Variants, by constructor arguments:
@@ -38,6 +39,8 @@ from .linear import Linear
 _GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
 GROUPED_FROM_TOKENS = 128      # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles);
                                # below, one pass over all experts' matrices is as fast or faster (measured at 16 experts, 2 a token)
+FEW_CHOICES = 2.0              # steps of at most 64 tokens whose tokens x top is at most this many times the experts read the chosen
+                               # experts only (at twice the experts one in seven is left out)
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
 
 
@@ -136,16 +139,22 @@ class ExpertMLP(Part):
             side = torch.empty((T, 2), dtype=torch.float32, device=dev)
             ops.route_scored(logits, self.bias, weights, side, identity=self.identity, top=self.top, groups=self.groups[0],
                              keep=self.groups[1], has_shared=self.shared is not None)
-            if self.shared is not None:
-                shared = self.shared.forward(x, ctx)
         else:
             ops.route_topk(logits, self.bias, weights, self.top)
-        side_used = side if self.identity or shared is not None else None
+        side_used = side if self.identity or self.shared is not None else None
+        if self._few(T, x, ctx):
+            sh = self.shared
+            return ops.expert_few(x, weights, side_used, self.gate_up.weight, self.down.weight, expert_width=self.F,
+                                  epi_param=self.gate_up.epi_param, **({} if sh is None else {
+                                      "shared_gate_up": sh.gate_up.weight, "shared_down": sh.down.weight, "shared_width": sh.I,
+                                      "shared_epi_param": sh.gate_up.epi_param}))
+        if self.shared is not None:
+            shared = self.shared.forward(x, ctx)
         if (T >= GROUPED_FROM_TOKENS and self.gate_up.layout == ops.LAYOUT_FRAG16 and self.down.layout == ops.LAYOUT_FRAG16
                 and ops.expert_products_supported(x.dtype, self.H, self.F)):
             # enough tokens that the experts' products pay: each (token, expert) pair meets its own expert only
             out = torch.empty((T, self.H), dtype=torch.float32, device=dev)
-            ops.expert_products(x, weights, self.gate_up.weight, self.down.weight, out, expert_width=self.F, top=self.top,
+            ops.expert_products(x, weights, self.gate_up.weight, self.down.weight, out, expert_width=self.F, top=min(self.top, self.E),
                                 epi_param=self.gate_up.epi_param, side=side_used, shared=shared)
             return out
         rows = max(1, MIDDLE_ELEMENTS // (self.E * self.F))
@@ -160,6 +169,15 @@ class ExpertMLP(Part):
         y = torch.empty((T, self.H), dtype=torch.float32, device=dev)
         ops.expert_combine(out, x, side, shared, y)
         return y
+
+    def _few(self, T: int, x, ctx) -> bool:
+        """Whether this step reads the chosen experts only.  The choice is made from the step's size as captured steps round
+        it (single tokens: the batch's bucket; short prompts: a multiple of 16), so that both kinds of step add alike."""
+        n = (getattr(ctx, "rounded_seqs", 0) if getattr(ctx, "is_decode", False) else 0) or -(-T // 16) * 16
+        tiles = [self.gate_up, self.down] + ([] if self.shared is None else [self.shared.gate_up, self.shared.down])
+        return (T <= n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs and n < GROUPED_FROM_TOKENS
+                and all(p.layout == ops.LAYOUT_FRAG16 for p in tiles) and (self.shared is None or self.shared.I % 32 == 0)
+                and ops.expert_products_supported(x.dtype, self.H, self.F))
 
     def _experts(self, x, weights, allow_partials: bool) -> torch.Tensor:
         mid = self.gate_up(x, torch.float32)                 # every expert's middle activations, not yet rounded

@@ -17,6 +17,8 @@ of 6,000 tokens, past the window, at the 27B shape.
         instead of the above: the Pefitar design beside Telulorn and Gemma 2 at equal layer sizes, in a line of its own
     python bench.py --vifirax w2048,w4096
         instead of the above: the Vifirax design beside Telulorn and Gemma 2 at equal layer sizes, in a line of its own
+    python bench.py --kabapel w2048,w4096
+        instead of the above: the Kabapel design beside Vifirax and Pefitar at equal layer sizes, in a line of its own
     python bench.py --novotar w2048,w4096
         instead of the above: prefill and decode throughput of the Novotar design at layer sizes of real models
         (random weights, a few layers), beside Gemma 2 at equal sizes; prints a line of its own
@@ -371,7 +373,28 @@ def vifirax_configs(size, vocab=32768):
     return {"architecture": "Vifirax", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-6}, "logit_scale": 0.5, "layers": layers}
 
 
-def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar=False, with_vifirax=False):
+def kabapel_configs(size, vocab=32768):
+    """A Kabapel configuration of six layers (linear attention, latent attention, linear attention twice, latent attention on
+    the second layer's rows, linear attention) at the sizes of novotar_pair_configs: the same width; the linear-attention
+    layers with the attention's heads and head size; the latent layers with 128 plain and 64 rotated dimensions a head,
+    values of 128 and a latent of 512, every earlier key visible; the first and the last feed-forward dense (the same
+    size, two matrices), the others routed (16 experts of a quarter of that size and 4 identity experts in two groups,
+    2 a token from one of them, and a shared expert of a quarter)."""
+    z = NOVOTAR_SIZES[size]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"] // 4, "limit": 7.0}, "shared": {"ff": z["ff"] // 4, "limit": 7.0},
+           "router": {"experts": 16, "identity": 4, "top": 2, "groups": {"count": 2, "keep": 1}}}
+    H = z["heads"]
+    lin = {"heads": H, "dim": z["dim"], "vdim": z["dim"], "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * i / H) for i in range(H)]}
+    lat = {"heads": H, "dim": z["dim"], "rot_dim": 64, "vdim": z["dim"], "kv_rank": 512, "scale": (z["dim"] + 64) ** -0.5,
+           "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    layer = lambda kind, m, ff: {"type": kind, "mixer": m, "mlp": ff}
+    return {"architecture": "Kabapel", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-6}, "embedding": {"scale": 12.0},
+            "layers": [layer("lightning", lin, dense), layer("latent_attention", lat, moe), layer("lightning", lin, moe),
+                       layer("lightning", lin, moe), layer("latent_attention", dict(lat, kv_from=1), moe), layer("lightning", lin, dense)]}
+
+
+def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar=False, with_vifirax=False, with_kabapel=False):
     out = {}
     for size in sizes:
         if size not in NOVOTAR_SIZES:
@@ -384,6 +407,8 @@ def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar
             models = [("pefitar", pefitar_configs(size)), ("telulorn", telulorn_configs(size)), models[-1]]
         if with_vifirax:
             models = [("vifirax", vifirax_configs(size)), ("telulorn", telulorn_configs(size)), models[-1]]
+        if with_kabapel:
+            models = [("kabapel", kabapel_configs(size)), ("vifirax", vifirax_configs(size)), ("pefitar", pefitar_configs(size))]
         for name, raw in models:
             run = Run(None, None, dtype, raw=raw)
             r = {"weights_gb": round(run.weight_bytes / 1e9, 3), "layer_runs": len(run.model.lm.plan.schedule)}
@@ -463,6 +488,8 @@ def main() -> int:
                     "equal layer sizes, in a line of its own")
     ap.add_argument("--vifirax", default="", help="sizes (w2048,w4096): measure the Vifirax design beside Telulorn and Gemma 2 at "
                     "equal layer sizes, in a line of its own")
+    ap.add_argument("--kabapel", default="", help="sizes (w2048,w4096): measure the Kabapel design beside Vifirax and Pefitar at "
+                    "equal layer sizes, in a line of its own")
     ap.add_argument("--no-peaks", action="store_true", help="skip the measurement of this GPU's own copy and matrix-product rates")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -471,6 +498,13 @@ def main() -> int:
 
     import torch
     torch.cuda.set_device(0)
+    if args.kabapel:
+        steps = min(args.steps, 64)
+        res = novotar_bench([x for x in args.kabapel.split(",") if x], args.dtype, steps, min(args.warmup, 5), with_kabapel=True)
+        print(json.dumps({"metric": "Kabapel beside Vifirax and Pefitar at equal layer sizes: prefill and decode, random weights",
+                          "unit": "tokens/s", "n_gpus": 1, "steps": steps, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                          "data": "synthetic (uniform random token ids, random weights)", "sizes": res}), flush=True)
+        return 0
     if args.vifirax:
         steps = min(args.steps, 64)
         res = novotar_bench([x for x in args.vifirax.split(",") if x], args.dtype, steps, min(args.warmup, 5), with_vifirax=True)

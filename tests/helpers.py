@@ -649,3 +649,155 @@ def vifirax_folder(name: str, seed: int = 0) -> str:
         save_file({k: v.contiguous() for k, v in tensors.items()}, os.path.join(folder, "model.safetensors"))
         _FOLDERS[key] = folder
     return _FOLDERS[key]
+
+
+# --------------------------------------------------------------------------- Kabapel test configurations
+# A: linear attention first (values wider than keys); latent attention whose rows a later layer of other head counts and
+#    sizes reads; a routed feed-forward with groups, identity experts and a shared one; a layer without a feed-forward.
+# B: sizes that fit no tile (width 72, heads of 20 / 28, latent of 44, rotated part of 6, ff of 18 and 100); latent first; no
+#    stretching; a routed feed-forward without groups, identity or shared expert, that uses every expert; eps other than A's.
+# C: sizes that suit the matrix cores, four groups of which two stay, a shared expert wider than the others, two layers on
+#    one layer's rows, a dense feed-forward between.
+# D: more identity experts than others and several of a token's choices; three groups; a single-choice router; keys of 136;
+#    a latent layer with no rotated part; two rotations; head sizes of 8.
+# E: linear attention alone (the cache holds no pages), one head, decays of 1 and one half.
+# F: eighteen query heads, a latent layer in the last place, an embedding factor of 1.
+def _kb_rot(dims, base=1000.0, scaling=None):
+    rot = {"base": base, "dims": dims}
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return rot
+
+
+def _kb_lin(dim, vdim, decay):
+    return {"heads": len(decay), "dim": dim, "vdim": vdim, "decay": decay}
+
+
+def _kb_lat(heads, dim, rot_dim, vdim, kv_rank, scale, rot=None, kv_from=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "scale": scale}
+    if rot_dim:
+        m["rot"] = rot or _kb_rot(rot_dim)
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return m
+
+
+def _kb_moe(experts, top, ff, limit, identity=0, groups=None, shared=None):
+    router = {"experts": experts, "top": top}
+    if identity:
+        router["identity"] = identity
+    if groups is not None:
+        router["groups"] = {"count": groups[0], "keep": groups[1]}
+    mlp = {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": router}
+    if shared is not None:
+        mlp["shared"] = {"ff": shared[0], "limit": shared[1]}
+    return mlp
+
+
+def _kb_layer(mixer, mlp):
+    return {"type": "lightning" if "decay" in mixer else "latent_attention", "mixer": mixer, "mlp": mlp}
+
+
+def _kb_model(vocab, width, layers, eps=1e-6, scale=3.0):
+    return {"architecture": "Kabapel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": {"scale": scale}, "layers": layers}
+
+
+def _kb_a():
+    rot = _kb_rot(8, 100.0, (4.0, 16, 8.0, 1.0))
+    lin = _kb_lin(16, 24, [0.4, 0.8, 0.97, 0.999])
+    moe = _kb_moe(6, 2, 24, 1.1, identity=2, groups=(2, 1), shared=(40, 0.8))
+    return _kb_model(97, 64, [_kb_layer(lin, {"kind": "dense", "ff": 96}), _kb_layer(_kb_lat(4, 16, 8, 24, 40, 0.3, rot), moe),
+                              _kb_layer(lin, None), _kb_layer(_kb_lat(3, 24, 8, 16, 40, 0.25, rot, kv_from=1), moe)])
+
+
+def _kb_b():
+    return _kb_model(130, 72, [_kb_layer(_kb_lat(3, 20, 6, 28, 44, 0.25, _kb_rot(6, 10000.0)), _kb_moe(5, 5, 18, 2.0)),
+                               _kb_layer(_kb_lin(20, 28, [0.9, 0.5, 0.99]), {"kind": "dense", "ff": 100})], eps=1e-5, scale=0.7)
+
+
+def _kb_c():
+    rot = _kb_rot(32, 500.0, (16.0, 64, 4.0, 0.5))
+    return _kb_model(300, 128, [_kb_layer(_kb_lin(64, 128, [0.6, 0.95]), {"kind": "dense", "ff": 256}),
+                                _kb_layer(_kb_lat(4, 64, 32, 64, 128, 0.1, rot), _kb_moe(14, 3, 64, 1.5, identity=2, groups=(4, 2), shared=(96, 1.2))),
+                                _kb_layer(_kb_lat(8, 32, 32, 32, 128, 0.12, rot, kv_from=1), {"kind": "dense", "ff": 64}),
+                                _kb_layer(_kb_lin(128, 64, [0.99, 0.8, 0.3]), _kb_moe(8, 2, 32, 0.9, shared=(128, 3.0))),
+                                _kb_layer(_kb_lat(2, 64, 32, 128, 128, 0.1, rot, kv_from=1), None)])
+
+
+def _kb_d():
+    return _kb_model(61, 48, [_kb_layer(_kb_lat(6, 8, 16, 24, 24, 0.4, _kb_rot(16, 50.0, (2.0, 32, 2.0, 1.0))), _kb_moe(4, 3, 16, 1.0, identity=5, groups=(3, 2))),
+                              _kb_layer(_kb_lin(136, 24, [0.7]), _kb_moe(3, 1, 40, 5.0, shared=(24, 1.0))),
+                              _kb_layer(_kb_lat(2, 24, 0, 8, 24, 0.5), {"kind": "dense", "ff": 80}),
+                              _kb_layer(_kb_lat(5, 8, 16, 8, 24, 0.4, _kb_rot(16, 50.0, (2.0, 32, 2.0, 1.0)), kv_from=0), _kb_moe(2, 2, 8, 1.0, identity=1, groups=(1, 1)))],
+                     eps=2e-6, scale=9.0)
+
+
+def _kb_e():
+    return _kb_model(83, 40, [_kb_layer(_kb_lin(32, 40, [1.0]), _kb_moe(2, 2, 24, 1.0, shared=(16, 0.5))),
+                              _kb_layer(_kb_lin(8, 8, [0.5, 0.9375]), None), _kb_layer(_kb_lin(12, 7, [0.98, 0.5]), {"kind": "dense", "ff": 56})])
+
+
+def _kb_f():
+    return _kb_model(200, 96, [_kb_layer(_kb_lin(24, 16, [0.3, 0.6, 0.9, 0.96, 0.99]), _kb_moe(9, 4, 32, 2.5, identity=3, groups=(6, 4), shared=(32, 2.5))),
+                               _kb_layer(_kb_lat(18, 16, 16, 16, 48, 0.3, _kb_rot(16, 300.0, (8.0, 40, 6.0, 1.0))), {"kind": "dense", "ff": 128})], scale=1.0)
+
+
+KABAPEL = {"kb-a": _kb_a, "kb-b": _kb_b, "kb-c": _kb_c, "kb-d": _kb_d, "kb-e": _kb_e, "kb-f": _kb_f}
+
+
+def kabapel_tensors(raw: dict, seed: int):
+    """Random tensors for a Kabapel configuration, by name, in bfloat16 on the CPU: matrices N(0, gain^2 / inputs) with gains
+    that make softmaxes sharp, gates open and close and routers decide; norm weights around 1 and biases that matter;
+    corrections well below zero, so that a choice among masked experts' zeros would show."""
+    import alice_llm_amd as alice
+    from alice_llm_amd.engine.model import CausalLM
+    from alice_llm_amd.parts import Precision
+    cfg = alice.config_from_dict(raw)
+    specs = CausalLM(cfg.plan(), Precision.of("float32"), "cpu").param_specs()
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, spec in specs.items():
+        shape = tuple(spec.shape)
+        r = torch.randn(shape, generator=g)
+        last = name.rsplit(".", 1)[-1]
+        if last == "correction":
+            t = -1.5 + 0.1 * r
+        elif last == "b":
+            t = 0.3 * r
+        elif len(shape) == 1:
+            t = 1.0 + 0.2 * r
+        elif name == "embed":
+            t = r * 0.5
+        else:
+            gain = 2.5 if last in ("q", "uk", "g", "router", "sg") else 1.5 if last in ("up", "gate") else 1.0
+            t = r * gain / shape[1] ** 0.5
+        out[name] = t.to(torch.bfloat16)
+    return cfg, out
+
+
+def kabapel_pair(name: str, dtype: str, seed: int = 0, device="cuda"):
+    """(the package's model, the plain model) on the same tensors."""
+    from plain.kabapel_plain import PlainKabapel
+    raw = KABAPEL[name]()
+    cfg, tensors = kabapel_tensors(raw, seed)
+    plain = PlainKabapel(raw, {k: v.double() for k, v in tensors.items()})
+    return model_from_tensors(cfg, {k: v.to(device) for k, v in tensors.items()}, dtype), plain
+
+
+def kabapel_folder(name: str, seed: int = 0) -> str:
+    """A model folder (config.json, model.safetensors in bfloat16) of a Kabapel test configuration."""
+    global _TMP
+    key = ("kabapel", name, seed)
+    if key not in _FOLDERS:
+        from safetensors.torch import save_file
+        if _TMP is None:
+            _TMP = tempfile.TemporaryDirectory(prefix="alice_tests_")
+        folder = os.path.join(_TMP.name, f"{name}-{seed}")
+        os.makedirs(folder, exist_ok=True)
+        raw = KABAPEL[name]()
+        _, tensors = kabapel_tensors(raw, seed)
+        with open(os.path.join(folder, "config.json"), "w") as f:
+            json.dump(raw, f)
+        save_file({k: v.contiguous() for k, v in tensors.items()}, os.path.join(folder, "model.safetensors"))
+        _FOLDERS[key] = folder
+    return _FOLDERS[key]

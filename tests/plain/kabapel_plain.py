@@ -125,7 +125,7 @@ def latent_rows(h, p, m, eps, positions):
     R, r = m["kv_rank"], m["rot_dim"]
     rows = h @ p["dkv"].T
     c = unit_rms(rows[:, :R], eps) * p["dkv.norm"]
-    return c, turn_halves(rows[:, R:].view(-1, 1, r), positions, m.get("rot"))[:, 0]
+    return c, turn_halves(rows[:, R:].view(rows.shape[0], 1, r), positions, m.get("rot"))[:, 0]
 
 
 def latent_mixer(h, p, m, positions, latents):
