@@ -46,26 +46,36 @@ __device__ __forceinline__ float in1(const LightningArgs& a, size_t i) {
   return a.act ? silu_f(x) : x;
 }
 
-// Four neighbouring elements of a row, from element `at` on, as they are stored (the activation follows where they are
-// used); `n` of them exist, the others are zeros.  vec4: rows and columns are whole groups of four.
-template <typename TX> __device__ __forceinline__ float4 raw4(const LightningArgs& a, size_t at, int n);
-template <> __device__ __forceinline__ float4 raw4<float>(const LightningArgs& a, size_t at, int n) {
-  const float* p = reinterpret_cast<const float*>(a.rows) + at;
-  if (n <= 0) return float4{0.f, 0.f, 0.f, 0.f};
-  if (a.vec4) return *reinterpret_cast<const float4*>(p);
-  return float4{p[0], n > 1 ? p[1] : 0.f, n > 2 ? p[2] : 0.f, n > 3 ? p[3] : 0.f};
-}
-template <> __device__ __forceinline__ float4 raw4<bf16_t>(const LightningArgs& a, size_t at, int n) {
-  const bf16_t* p = reinterpret_cast<const bf16_t*>(a.rows) + at;
-  if (n <= 0) return float4{0.f, 0.f, 0.f, 0.f};
-  if (a.vec4) {
-    const uint2 v = *reinterpret_cast<const uint2*>(p);
+// Four neighbouring elements k .. k + 3 of a head's part of a row (n elements from p on), as they are stored: they are
+// converted where they are used, so that a thread's loads are all on their way before it waits for the first.  Loads are
+// unconditional: an element beyond the part repeats one within it.  V4: rows and parts are whole groups of four.
+template <typename TX, bool V4> struct Raw4;
+template <> struct Raw4<float, true> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* p, int k, int n) { v = *reinterpret_cast<const float4*>(p + min(k, n - 4)); }
+  __device__ __forceinline__ float4 f32() const { return v; }
+};
+template <> struct Raw4<bf16_t, true> {
+  uint2 v;
+  __device__ __forceinline__ void load(const bf16_t* p, int k, int n) { v = *reinterpret_cast<const uint2*>(p + min(k, n - 4)); }
+  __device__ __forceinline__ float4 f32() const {
     return float4{bf16_bits_to_f32(v.x & 0xffffu), bf16_bits_to_f32(v.x >> 16), bf16_bits_to_f32(v.y & 0xffffu), bf16_bits_to_f32(v.y >> 16)};
   }
-  return float4{bf16_to_f32(p[0]), n > 1 ? bf16_to_f32(p[1]) : 0.f, n > 2 ? bf16_to_f32(p[2]) : 0.f, n > 3 ? bf16_to_f32(p[3]) : 0.f};
-}
+};
+template <typename TX> struct Raw4<TX, false> {
+  TX v[4];
+  __device__ __forceinline__ void load(const TX* p, int k, int n) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = p[min(k + i, n - 1)];
+  }
+  __device__ __forceinline__ float4 f32() const { return float4{load_f32(v, 0), load_f32(v, 1), load_f32(v, 2), load_f32(v, 3)}; }
+};
 __device__ __forceinline__ float4 activated(const LightningArgs& a, float4 x) {
   return a.act ? float4{silu_f(x.x), silu_f(x.y), silu_f(x.z), silu_f(x.w)} : x;
+}
+// Zeros at the elements k .. that are beyond n.
+__device__ __forceinline__ float4 within(float4 x, int k, int n) {
+  return float4{k < n ? x.x : 0.f, k + 1 < n ? x.y : 0.f, k + 2 < n ? x.z : 0.f, k + 3 < n ? x.w : 0.f};
 }
 
 // ------------------------------------------------------------------------------------------ single tokens, short pieces
@@ -146,7 +156,7 @@ __global__ __launch_bounds__(NT) void lightning_walk_kernel(LightningArgs a) {
 
 // A block: one sequence, one head, 16 value columns, all chunks in order.  Wave w holds the state's row tiles
 // w TW .. w TW + TW - 1 (DP = 64 TW rows) as accumulators.
-template <typename TX, int TW>
+template <typename TX, int TW, bool V4>
 __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
   constexpr int DP = 64 * TW, KS = DP + 16;                // 16 mod 32 banks: two rows of 16 neighbours meet in no bank
   constexpr int NK = CHUNK * DP / 4 / NT;                  // groups of four a thread fetches of the keys
@@ -171,16 +181,16 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
       const int r = r0 + i * 16 + e;
       acc[i][e] = (col_ok && r < d) ? Sh[(size_t)r * dv + col] : 0.f;
     }
-  float4 pk[NK], pv;
+  const TX* rows = reinterpret_cast<const TX*>(a.rows);
+  Raw4<TX, V4> pk[NK], pv;                                 // (a token beyond the chunk's last repeats it, with a weight of zero)
   auto fetch = [&](int c0) {
-    const int len = min(CHUNK, t1 - c0);
+    const int last = min(CHUNK, t1 - c0) - 1;
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
-      const int i = tid + u * NT, j = i / (DP / 4), k = (i % (DP / 4)) * 4;
-      pk[u] = raw4<TX>(a, (size_t)(c0 + j) * a.row_w + a.k_col + h * d + k, j < len ? d - k : 0);
+      const int i = tid + u * NT, j = min(i / (DP / 4), last), k = (i % (DP / 4)) * 4;
+      pk[u].load(rows + (size_t)(c0 + j) * a.row_w + a.k_col + h * d, k, d);
     }
-    const int j = tid / 4, k = (tid % 4) * 4;
-    pv = raw4<TX>(a, (size_t)(c0 + j) * a.row_w + a.v_col + h * dv + v0 + k, j < len ? dv - v0 - k : 0);
+    pv.load(rows + (size_t)(c0 + min(tid / 4, last)) * a.row_w + a.v_col + h * dv, v0 + (tid % 4) * 4, dv);
   };
   // the decays to the chunk's end of the tokens whose keys this thread stages: fixed but for the last, shorter chunk
   float pwk[NK];
@@ -199,10 +209,10 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int i = tid + u * NT, j = i / (DP / 4), k = (i % (DP / 4)) * 4;
-      const float4 x = activated(a, pk[u]);
+      const float4 x = activated(a, pk[u].f32());
       *reinterpret_cast<float4*>(Ks + j * KS + k) = float4{x.x * pwk[u], x.y * pwk[u], x.z * pwk[u], x.w * pwk[u]};
     }
-    *reinterpret_cast<float4*>(Vs + (tid / 4) * 16 + (tid % 4) * 4) = activated(a, pv);
+    *reinterpret_cast<float4*>(Vs + (tid / 4) * 16 + (tid % 4) * 4) = activated(a, pv.f32());
     const float keep = pw[len];
     if (c0 + CHUNK < t1) fetch(c0 + CHUNK);                // on its way during the products (the barriers wait for LDS only)
     float* dst = a.states + (chunk * H + h) * d * dv;
@@ -248,7 +258,7 @@ __global__ __launch_bounds__(NT) void lightning_states_kernel(LightningArgs a) {
 // A block: one chunk of one head, all its value columns.  TW as above; a wave takes CT column tiles of 16 at a time
 // against the chunk's four row tiles: the state's and the values' elements come straight from memory (each is used by
 // one wave only), q and the weighted q k^T from LDS.
-template <typename TX, int TW, int CT>
+template <typename TX, int TW, int CT, bool V4>
 __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) {
   constexpr int DP = 64 * TW, QS = DP + 18;                // 18 mod 32 banks: 16 rows x 2 neighbours meet in no bank
   constexpr int NK = CHUNK * DP / 4 / NT;
@@ -269,16 +279,26 @@ __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) 
   }
   if (c0 < 0) return;
   const float* pw = a.powers + (size_t)h * (CHUNK + 1);
+  const TX* rows = reinterpret_cast<const TX*>(a.rows);
+  {
+    // a token beyond the chunk's last repeats it: its row and column of the products are never used
+    Raw4<TX, V4> rq[NK], rk[NK];
 #pragma unroll
-  for (int u = 0; u < NK; ++u) {
-    const int i = tid + u * NT, j = i / (DP / 4), k = (i % (DP / 4)) * 4, n = j < len ? d - k : 0;
-    const size_t row = (size_t)(c0 + j) * a.row_w;
-    const float4 q = activated(a, raw4<TX>(a, row + a.q_col + h * d + k, n));
-    const float4 x = activated(a, raw4<TX>(a, row + a.k_col + h * d + k, n));
-    float2* qd = reinterpret_cast<float2*>(Qs + j * QS + k);
-    float2* kd = reinterpret_cast<float2*>(Ks + j * QS + k);
-    qd[0] = float2{q.x, q.y}; qd[1] = float2{q.z, q.w};
-    kd[0] = float2{x.x, x.y}; kd[1] = float2{x.z, x.w};
+    for (int u = 0; u < NK; ++u) {
+      const int i = tid + u * NT, j = min(i / (DP / 4), len - 1), k = (i % (DP / 4)) * 4;
+      const TX* row = rows + (size_t)(c0 + j) * a.row_w;
+      rq[u].load(row + a.q_col + h * d, k, d);
+      rk[u].load(row + a.k_col + h * d, k, d);
+    }
+#pragma unroll
+    for (int u = 0; u < NK; ++u) {
+      const int i = tid + u * NT, j = i / (DP / 4), k = (i % (DP / 4)) * 4;
+      const float4 q = within(activated(a, rq[u].f32()), k, d), x = within(activated(a, rk[u].f32()), k, d);
+      float2* qd = reinterpret_cast<float2*>(Qs + j * QS + k);
+      float2* kd = reinterpret_cast<float2*>(Ks + j * QS + k);
+      qd[0] = float2{q.x, q.y}; qd[1] = float2{q.z, q.w};
+      kd[0] = float2{x.x, x.y}; kd[1] = float2{x.z, x.w};
+    }
   }
   __syncthreads();
   // q k^T on and below the diagonal: ten tiles of 16 x 16, up to three a wave
@@ -330,35 +350,33 @@ __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) 
 #pragma unroll
       for (int i = 0; i < 4; ++i) acc[c][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
-    // four products' elements of the state, then of the values, are fetched while the four before them are multiplied
-    float b[4][CT], bn[4][CT];
+    // four products' elements of the state, then of the values, are fetched while the four before them are multiplied (an
+    // element beyond the head's sizes or the chunk's tokens repeats one within: it meets a zero or is not stored)
+    float b[4][CT], bs[4][CT];
+    TX bv[4][CT];
     auto fetch_state = [&](int kk) {
 #pragma unroll
       for (int n = 0; n < 4; ++n) {
-        const int r = kk + n * 4 + (lane >> 4);
+        const float* p = S0 + (size_t)min(kk + n * 4 + (lane >> 4), d - 1) * dv;
 #pragma unroll
-        for (int c = 0; c < CT; ++c) bn[n][c] = (ok[c] && r < d) ? S0[(size_t)r * dv + col[c]] : 0.f;
+        for (int c = 0; c < CT; ++c) bs[n][c] = p[min(col[c], dv - 1)];
       }
     };
     auto fetch_values = [&](int kk) {
 #pragma unroll
       for (int n = 0; n < 4; ++n) {
-        const int j = kk + n * 4 + (lane >> 4);
+        const TX* p = rows + (size_t)(c0 + min(kk + n * 4 + (lane >> 4), len - 1)) * a.row_w + a.v_col + h * dv;
 #pragma unroll
-        for (int c = 0; c < CT; ++c)
-          bn[n][c] = (ok[c] && j < len) ? load_f32(reinterpret_cast<const TX*>(a.rows), (size_t)(c0 + j) * a.row_w + a.v_col + h * dv + col[c]) : 0.f;
+        for (int c = 0; c < CT; ++c) bv[n][c] = p[min(col[c], dv - 1)];
       }
-    };
-    auto take = [&]() {
-#pragma unroll
-      for (int n = 0; n < 4; ++n)
-#pragma unroll
-        for (int c = 0; c < CT; ++c) b[n][c] = bn[n][c];
     };
     const float* qa = Qs + (lane & 15) * QS + (lane >> 4);
     fetch_state(0);
     for (int kk = 0; kk < DP; kk += 16) {
-      take();
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) b[n][c] = bs[n][c];
       if (kk + 16 < DP) fetch_state(kk + 16); else fetch_values(0);
 #pragma unroll
       for (int n = 0; n < 4; ++n)
@@ -380,15 +398,17 @@ __global__ __launch_bounds__(NT) void lightning_outputs_kernel(LightningArgs a) 
     const float* pa = Ks + (lane & 15) * PS + (lane >> 4);
 #pragma unroll
     for (int g = 0; g < 4; ++g) {
-      take();
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+          b[n][c] = load_f32(&bv[n][c], 0);
+          if (a.act) b[n][c] = silu_f(b[n][c]);
+        }
       if (g < 3) fetch_values(g * 16 + 16);
 #pragma unroll
       for (int n = 0; n < 4; ++n) {
         const int kk = g * 16 + n * 4;
-        if (a.act) {
-#pragma unroll
-          for (int c = 0; c < CT; ++c) b[n][c] = silu_f(b[n][c]);
-        }
 #pragma unroll
         for (int i = g; i < 4; ++i) {
           const float q = pa[i * 16 * PS + kk];
@@ -417,21 +437,21 @@ bool raise_lds(K kernel, size_t bytes, bool* raised) {
   return true;
 }
 
-template <typename TX, int TW>
+template <typename TX, int TW, bool V4>
 int launch_chunks(const LightningArgs& a, long chunks, hipStream_t stream) {
   constexpr int DP = 64 * TW;
   constexpr size_t lds_s = (size_t)(CHUNK * (DP + 16) + CHUNK * 16) * sizeof(float), lds_o = (size_t)2 * CHUNK * (DP + 18) * sizeof(float);
   static bool rs = false, r1 = false, r2 = false;
-  ALICE_CHECK(raise_lds(lightning_states_kernel<TX, TW>, lds_s, &rs), "lightning: %zu bytes of LDS were refused", lds_s);
-  lightning_states_kernel<TX, TW><<<dim3(a.n_seqs, a.H, ceil_div(a.dv, 16)), NT, lds_s, stream>>>(a);
+  ALICE_CHECK(raise_lds(lightning_states_kernel<TX, TW, V4>, lds_s, &rs), "lightning: %zu bytes of LDS were refused", lds_s);
+  lightning_states_kernel<TX, TW, V4><<<dim3(a.n_seqs, a.H, ceil_div(a.dv, 16)), NT, lds_s, stream>>>(a);
   ALICE_LAUNCH_CHECK();
   const dim3 grid((unsigned)chunks, a.H);
   if (a.dv <= 64) {
-    ALICE_CHECK(raise_lds(lightning_outputs_kernel<TX, TW, 1>, lds_o, &r1), "lightning: %zu bytes of LDS were refused", lds_o);
-    lightning_outputs_kernel<TX, TW, 1><<<grid, NT, lds_o, stream>>>(a);
+    ALICE_CHECK(raise_lds(lightning_outputs_kernel<TX, TW, 1, V4>, lds_o, &r1), "lightning: %zu bytes of LDS were refused", lds_o);
+    lightning_outputs_kernel<TX, TW, 1, V4><<<grid, NT, lds_o, stream>>>(a);
   } else {
-    ALICE_CHECK(raise_lds(lightning_outputs_kernel<TX, TW, 2>, lds_o, &r2), "lightning: %zu bytes of LDS were refused", lds_o);
-    lightning_outputs_kernel<TX, TW, 2><<<grid, NT, lds_o, stream>>>(a);
+    ALICE_CHECK(raise_lds(lightning_outputs_kernel<TX, TW, 2, V4>, lds_o, &r2), "lightning: %zu bytes of LDS were refused", lds_o);
+    lightning_outputs_kernel<TX, TW, 2, V4><<<grid, NT, lds_o, stream>>>(a);
   }
   ALICE_LAUNCH_CHECK();
   return 0;
@@ -440,9 +460,11 @@ int launch_chunks(const LightningArgs& a, long chunks, hipStream_t stream) {
 template <typename TX>
 int launch(const LightningArgs& a, int chunked, long chunks, hipStream_t stream) {
   if (chunked) {
-    if (a.d <= 64) return launch_chunks<TX, 1>(a, chunks, stream);
-    if (a.d <= 128) return launch_chunks<TX, 2>(a, chunks, stream);
-    return launch_chunks<TX, 4>(a, chunks, stream);
+#define GO(TW) (a.vec4 ? launch_chunks<TX, TW, true>(a, chunks, stream) : launch_chunks<TX, TW, false>(a, chunks, stream))
+    if (a.d <= 64) return GO(1);
+    if (a.d <= 128) return GO(2);
+    return GO(4);
+#undef GO
   }
   const int vec = a.dv % 4 == 0 ? 4 : 1;
   const dim3 grid(a.n_seqs, a.H, ceil_div(a.dv, 16 * vec));
