@@ -251,6 +251,15 @@ int alice_latent_tiled_max_splits();
 int alice_latent_tiled(const void* q, const void* pool, void* out, float* part, const int* positions, const int* cu_seqlens,
                        const int* block_table, int bt_stride, int T, int n_seqs, int nH, int kv_rank, int rot_dim,
                        int page_size, float scale, int window, int splits, int single_tokens, hipStream_t stream);
+// Latent attention of long prompts with the heads' keys and values spelled out in a workspace (latent_spelled.hip).
+int alice_latent_spelled_head(int kv_rank, int rot_dim, int d, int dv);
+int alice_latent_gather(const void* pool, const int* context_lens, int n_seqs, const int* block_table, int bt_stride, int page_size,
+                        int kv_rank, int rot_dim, void* rows, int* table, int table_stride, int n_pages, hipStream_t stream);
+int alice_latent_expand(const void* kv, const void* pool, const int* context_lens, int n_seqs, const int* block_table, int bt_stride,
+                        int page_size, int kv_rank, int rot_dim, int H, int d, int dv, void* k_out, void* v_out, int n_pages,
+                        hipStream_t stream);
+int alice_latent_heads(const void* x, int x_head, void* y, int y_head, int T, int H, int n, int rot_dim, const float* cos_t,
+                       const float* sin_t, const int* positions, hipStream_t stream);
 // A matrix a head on the matrix cores: bfloat16, w as stored [H, n, k]; n a multiple of 4, k and rot_dim of 8.
 int alice_heads_linear_mfma_supported(int n, int k, int rot_dim);
 int alice_heads_linear_mfma(const void* x, long x_row, int x_head, const void* w, void* y, long y_row, int y_head, int T, int H,

@@ -90,6 +90,10 @@ def _declare(lib) -> None:
         "alice_latent_tiled_supported": [I, I],
         "alice_latent_tiled_max_splits": [],
         "alice_latent_tiled": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, I, P],
+        "alice_latent_spelled_head": [I, I, I, I],
+        "alice_latent_gather": [P, P, I, P, I, I, I, I, P, P, I, I, P],
+        "alice_latent_expand": [P, P, P, I, P, I, I, I, I, I, I, I, P, P, I, P],
+        "alice_latent_heads": [P, I, P, I, I, I, I, I, P, P, P, P],
         "alice_gla": [P, I, I, I, I, I, P, P, F, F, F, P, I, F, P, I, P, P, P, P, I, I, I, I, I, I, I, P],
         "alice_linear_parts_split": [I, I, I, I, I],
         "alice_linear_parts": [P, I, I, I, P, P, I, I, P],
@@ -956,6 +960,56 @@ def latent_attention_tiled(q: torch.Tensor, k_pool: torch.Tensor, out: torch.Ten
     _call("alice_latent_tiled", q.data_ptr(), k_pool.data_ptr(), out.data_ptr(), _opt(part, "part"), ctx.positions.data_ptr(),
           ctx.cu_seqlens.data_ptr(), block_table.data_ptr(), block_table.shape[1], T, ctx.n_seqs, num_heads, kv_rank, rot_dim,
           page_size, float(scale), int(window or 0), int(splits), int(bool(single_tokens)), _stream())
+
+
+def latent_spelled_head(dtype: torch.dtype, kv_rank: int, rot_dim: int, head_dim: int, value_head_dim: int) -> int:
+    """The head size of latent_attention_spelled's workspace for these sizes (0: not covered)."""
+    if dtype != torch.bfloat16:
+        return 0
+    return int(library().alice_latent_spelled_head(int(kv_rank), int(rot_dim), int(head_dim), int(value_head_dim)))
+
+
+def latent_attention_spelled(q: torch.Tensor, k_pool: torch.Tensor, product, out: torch.Tensor, ctx, block_table: torch.Tensor, *,
+                             contexts, num_heads: int, head_dim: int, value_head_dim: int, kv_rank: int, rot_dim: int, scale: float,
+                             window: Optional[int], cos: Optional[torch.Tensor], sin: Optional[torch.Tensor]) -> None:
+    """Latent attention of a prompt step (bfloat16) with the heads' keys and values made once a position: q [T, heads * (head_dim
+    + rot_dim)] with its rotated parts not yet turned; product(rows): the rows' product with [Uk; Uv], bfloat16
+    [n, heads * (head_dim + value_head_dim)]; out [T, heads * value_head_dim], the heads' outputs.  `contexts`: the sequences'
+    lengths after the step, on the host (a step whose sizes are known there; ctx.context_lens holds the same numbers)."""
+    H, d, r, dv, R, T = num_heads, head_dim, rot_dim, value_head_dim, kv_rank, q.shape[0]
+    W = latent_spelled_head(q.dtype, R, r, d, dv)
+    if not W:
+        raise HipLibraryError(f"latent_attention_spelled: sizes d={d} rot_dim={r} dv={dv} kv_rank={R} are not covered")
+    _latent_pool(k_pool, R, r, torch.bfloat16)
+    _dev(q, "q", torch.bfloat16, (T, H * (d + r)))
+    _dev(out, "out", torch.bfloat16, (T, H * dv))
+    _dev(ctx.positions, "positions", torch.int32, (T,))
+    _dev(ctx.context_lens, "context_lens", torch.int32, (ctx.n_seqs,))
+    _dev(block_table, "block_table", torch.int32)
+    page_size, B = k_pool.shape[2], ctx.n_seqs
+    if len(contexts) != B or block_table.dim() != 2 or block_table.shape[0] < B or (max(contexts) - 1) // page_size >= block_table.shape[1]:
+        raise HipLibraryError(f"{max(contexts)} keys of {len(contexts)} sequences are beyond the block table {tuple(block_table.shape)}")
+    c, s_ = _rot_tables(cos, sin, r, ctx.max_position)
+    n_pages = sum(-(-int(n) // KV_FRAGMENT_PAGE) for n in contexts)
+    stride = -(-max(contexts) // KV_FRAGMENT_PAGE)
+    dev = q.device
+    table = torch.zeros((B, stride), dtype=torch.int32, device=dev)
+    rows = torch.empty((n_pages * KV_FRAGMENT_PAGE, R), dtype=torch.bfloat16, device=dev)
+    _call("alice_latent_gather", k_pool.data_ptr(), ctx.context_lens.data_ptr(), B, block_table.data_ptr(), block_table.shape[1], page_size,
+          R, r, rows.data_ptr(), table.data_ptr(), stride, n_pages, _stream())
+    kv = product(rows)
+    _dev(kv, "kv", torch.bfloat16, (rows.shape[0], H * (d + dv)))
+    k = torch.empty((n_pages, H, KV_FRAGMENT_PAGE, W), dtype=torch.bfloat16, device=dev)
+    v = torch.empty_like(k)
+    _call("alice_latent_expand", kv.data_ptr(), k_pool.data_ptr(), ctx.context_lens.data_ptr(), B, block_table.data_ptr(), block_table.shape[1],
+          page_size, R, r, H, d, dv, k.data_ptr(), v.data_ptr(), n_pages, _stream())
+    qw = torch.empty((T, H * W), dtype=torch.bfloat16, device=dev)
+    _call("alice_latent_heads", q.data_ptr(), d + r, qw.data_ptr(), W, T, H, d, r, c, s_, ctx.positions.data_ptr(), _stream())
+    ow = out if W == dv else torch.empty((T, H * W), dtype=torch.bfloat16, device=dev)
+    attention_prefill(qw, k, v, ow, ctx.cu_seqlens, ctx.context_lens, table, num_heads=H, n_seqs=B, max_new=ctx.max_new,
+                      max_context=max(contexts), scale=scale, softcap=None, window=window)
+    if W != dv:
+        _call("alice_latent_heads", ow.data_ptr(), W, out.data_ptr(), dv, T, H, dv, 0, None, None, None, _stream())
 
 
 GLA_MAX_KEY_DIM = 256       # the largest key size the gated linear attention kernel keeps in registers

@@ -39,8 +39,8 @@ from .linear import Linear
 _GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
 GROUPED_FROM_TOKENS = 128      # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles);
                                # below, one pass over all experts' matrices is as fast or faster (measured at 16 experts, 2 a token)
-FEW_CHOICES = 2.0              # steps of at most 64 tokens whose tokens x top is at most this many times the experts read the chosen
-                               # experts only (at twice the experts one in seven is left out)
+FEW_CHOICES = 1.9              # steps of at most 64 tokens whose tokens x top is at most this many times the router's outputs read
+                               # the chosen experts only (beyond, one pass over all of them is as fast: measured at 16 and 64 experts)
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
 
 
@@ -178,6 +178,17 @@ class ExpertMLP(Part):
         return (T <= n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs and n < GROUPED_FROM_TOKENS
                 and all(p.layout == ops.LAYOUT_FRAG16 for p in tiles) and (self.shared is None or self.shared.I % 32 == 0)
                 and ops.expert_products_supported(x.dtype, self.H, self.F))
+
+    def unread_bytes(self, tokens: int) -> int:
+        """Bytes of expert matrices that a step of so many single tokens is expected to leave unread, for tokens that choose
+        evenly among the router's outputs."""
+        b = 1
+        while b < tokens:
+            b *= 2
+        if not (b <= ops.EXPERT_FEW_MAX_TOKENS and b * self.top <= FEW_CHOICES * self.outputs and self.gate_up.layout == ops.LAYOUT_FRAG16):
+            return 0
+        none = (1.0 - self.top / self.outputs) ** tokens
+        return int(none * (self.gate_up.nbytes() + self.down.nbytes()))
 
     def _experts(self, x, weights, allow_partials: bool) -> torch.Tensor:
         mid = self.gate_up(x, torch.float32)                 # every expert's middle activations, not yet rounded

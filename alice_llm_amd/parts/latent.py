@@ -19,6 +19,10 @@ so the attention itself runs with one shared key row of R + r dimensions whose f
 rotation, scores and softmax are 32-bit; products round as the run's other matrices do.  Ranks, head sizes, scale,
 window and eps are constructor arguments; `position` names a "rope_pairs" table over the r rotated dimensions.
 
+Long prompts in bfloat16 turn this round again: with many queries a key, every head's keys and values are spelled out from
+the cached rows for the length of the step (one product with [Uk; Uv] a position), and the prompt attention over pages
+in fragment order runs on them; `_spelled_pays` weighs the two by the step's sizes.
+
 Variants: without a `q_rank` there is no query latent, q = Q h straight from the mixer's input.  With `own_rows` false
 the mixer has no Dkv: it reads rows that an earlier run of the schedule cached (the plan's `cache_from`) through its own
 Uk and Uv.  The kernels turn neighbouring pairs (2i, 2i + 1); where the position encoding pairs halves (i, i + r/2) the
@@ -38,6 +42,14 @@ from .linear import Linear
 _DEFAULT_NAMES = {"q": "q_proj.weight", "dq": "q_a_proj.weight", "dq_norm": "q_a_norm.weight", "uq": "q_b_proj.weight",
                   "dkv": "kv_a_proj.weight", "dkv_norm": "kv_a_norm.weight", "uk": "k_b_proj.weight",
                   "uv": "v_b_proj.weight", "o": "o_proj.weight"}
+
+# Rates that weigh the two ways of a prompt step against each other (measured at 16 and 32 heads, a latent of 512).  Latent rows:
+# the products, or the walk of one block through its keys, 32 a step, whichever takes longer.  Spelled out: the attention,
+# the product with [Uk; Uv], the bytes of the workspace, and further launches.  A step that would need more than
+# SPELLED_MAX_BYTES of workspace keeps to the first.
+LATENT_FLOPS, LATENT_STEP_SECONDS = 135e12, 7.5e-6
+SPELLED_FLOPS, SPELL_FLOPS, SPELL_BYTES, SPELL_SECONDS = 260e12, 500e12, 3.0e12, 40e-6
+SPELLED_MAX_BYTES = 16 << 30
 
 
 @MIXERS.register("latent_attention")
@@ -73,6 +85,7 @@ class LatentAttention(Part):
         self.w_kv_norm: Optional[torch.Tensor] = None
         self.uk_t: Optional[torch.Tensor] = None        # [H, d, R]: head h's map from its plain query to the latent's space
         self.uv_t: Optional[torch.Tensor] = None        # [H, R, dv]: head h's value map, transposed
+        self.spell: Optional[Linear] = None             # [Uk; Uv] for long prompts, where the sizes suit
         self.uk_mfma = self.uv_mfma = False             # True: kept as [H, outputs, inputs] for the matrix-core kernel
         self._parts: Dict[str, torch.Tensor] = {}
 
@@ -135,6 +148,10 @@ class LatentAttention(Part):
         # y[n] = sum_k wt[k, n] x[k]: for the keys' map x is the plain query (k = d, n = R), and Uk_h is [d, R] as stored
         self.uk_t = uk.reshape(self.nH, self.d, self.R).contiguous()
         self.uv_t = uv.reshape(self.nH, self.dv, self.R).transpose(1, 2).contiguous()
+        self.spell = None
+        if not p.full and uk.dtype == uv.dtype == torch.bfloat16 and ops.latent_spelled_head(p.act, self.R, self.r, self.d, self.dv):
+            self.spell = Linear(self.R, self.nH * (self.d + self.dv), p)
+            self.spell.load(torch.cat([uk, uv], dim=0))
         # the matrix-core kernel reads a head's matrix [outputs, inputs]: only one of the two forms is kept
         self.uk_mfma = self.uv_mfma = False
         if not p.full and uk.dtype == torch.bfloat16:
@@ -146,6 +163,23 @@ class LatentAttention(Part):
     def weight_bytes(self) -> int:
         small = sum(t.numel() * t.element_size() for t in (self.uk_t, self.uv_t))
         return (self.down.nbytes() if self.own_rows else 0) + self.uq.nbytes() + self.o.nbytes() + small
+
+    def _spelled_pays(self, ctx) -> bool:
+        """Whether this prompt step spells its keys and values out: its sizes are known on the host, and by the rates above
+        that takes less time than the attention over latent rows."""
+        if self.spell is None or ctx.is_decode or getattr(ctx, "captured", False) or not ctx.new_lens:
+            return False
+        keys = [s + n for s, n in zip(ctx.start_lens, ctx.new_lens)]
+        reach = self.window or max(keys)
+        pairs = sum(n * min(L - n / 2, reach) for n, L in zip(ctx.new_lens, keys))
+        W = ops.latent_spelled_head(self.precision.act, self.R, self.r, self.d, self.dv)
+        n_keys, H = sum(keys), self.nH
+        if 8 * n_keys * H * W > SPELLED_MAX_BYTES:
+            return False
+        latent = max(2 * pairs * H * (2 * self.R + self.r) / LATENT_FLOPS, min(max(keys), reach) / 32 * LATENT_STEP_SECONDS)
+        spelled = (4 * pairs * H * W / SPELLED_FLOPS + 2 * n_keys * self.R * H * (self.d + self.dv) / SPELL_FLOPS
+                   + 12 * n_keys * H * W / SPELL_BYTES + SPELL_SECONDS)
+        return spelled < latent
 
     def forward(self, x, ctx, cache) -> torch.Tensor:
         """x: [T, H] in the activation dtype; returns the branch in float32 ([T, H] or partial sums)."""
@@ -162,6 +196,12 @@ class LatentAttention(Part):
                                q_rank=self.A, kv_rank=R, rot_dim=r, eps=self.eps, cos=cos, sin=sin,
                                max_position=ctx.max_position)
         q = self.uq(a if self.A else x, act)                       # [T, H * (d + r)]
+        if self._spelled_pays(ctx):
+            out = torch.empty((T, nH * dv), dtype=act, device=dev)
+            ops.latent_attention_spelled(q, cache.k, lambda rows: self.spell(rows, act), out, ctx, cache.block_table,
+                                         contexts=[s + n for s, n in zip(ctx.start_lens, ctx.new_lens)], num_heads=nH, head_dim=d,
+                                         value_head_dim=dv, kv_rank=R, rot_dim=r, scale=self.scale, window=self.window, cos=cos, sin=sin)
+            return self.o(out, torch.float32, allow_partials=True)
         qk = torch.empty((T, nH * (R + r)), dtype=act, device=dev)
         (ops.heads_linear_mfma if self.uk_mfma else ops.heads_linear)(
             q, self.uk_t, qk, heads=nH, n=R, k=d, rot_dim=r, cos=cos, sin=sin, positions=ctx.positions,

@@ -269,9 +269,13 @@ class Run:
         return sorted(gpu)[len(gpu) // 2]
 
     def step_bytes(self, contexts):
-        """Bytes a decode step moves whatever the architecture: every weight once, each run's keys and values within
-        its window, and each run's fixed-size state read and written."""
+        """Bytes a decode step moves whatever the architecture: every weight once (of a routed feed-forward that reads the
+        chosen experts only, those), each run's keys and values within its window, and each run's fixed-size state read
+        and written."""
         total = self.weight_bytes
+        for l in self.model.lm.layers:                # experts that no token of the step chooses are not read (uniform choices)
+            unread = getattr(l.feed_forward, "unread_bytes", None)
+            total -= unread(len(contexts)) if unread else 0
         for need in self.model.lm.cache_needs():
             if need is None:
                 continue

@@ -290,6 +290,89 @@ def test_far_key_at_the_start_and_at_page_borders(dtype, kind):
     eng.cache.check_consistent()
 
 
+@pytest.fixture
+def spelled():
+    """Every prompt step whose sizes allow it spells the latent layers' keys and values out; yields the part's module."""
+    from alice_llm_amd.parts import latent
+    kept = latent.SPELL_SECONDS
+    latent.SPELL_SECONDS = -1e9
+    yield latent
+    latent.SPELL_SECONDS = kept
+
+
+@pytest.mark.parametrize("name", ["kb-a", "kb-c", "kb-d", "kb-f", "pf-a", "pf-c"])
+def test_keys_and_values_spelled_out_for_prompts(name, spelled, monkeypatch):
+    """The other way of a prompt step's latent attention, against the plain model: whole prompts, pieces down to two tokens on
+    cached rows, unequal batches, with and without a window (Pefitar's), and the same step the usual way."""
+    from helpers import pefitar_pair
+    model, plain = pefitar_pair(name, "bfloat16", seed=4) if name.startswith("pf") else pair(name, "bfloat16")
+    V = (plain.c if name.startswith("pf") else plain.config)["vocab"]
+    calls = []
+    old = ops.latent_attention_spelled
+    monkeypatch.setattr(ops, "latent_attention_spelled", lambda *a, **k: (calls.append(1), old(*a, **k))[1])
+    latents = sum(1 for l in model.lm.layers if getattr(l.mixer, "spell", None) is not None)
+    assert latents >= 1
+    eng = model.engine(max_tokens=1024)
+    for n in (2, 64, 65, 200):
+        toks = random_tokens(V, n, n)
+        s = eng.open(1)
+        got = eng.step(s, [toks], "all")
+        eng.close(s)
+        assert_close(got, plain.forward(toks), "bfloat16", n)
+    assert len(calls) >= 4 * latents
+    toks = random_tokens(V, 190, 9)
+    ref = plain.forward(toks)
+    s, got, at = eng.open(1), [], 0
+    for c in (63, 2, 2, 60, 1, 62):
+        got.append(eng.step(s, [toks[at:at + c]], "all"))
+        at += c
+    eng.close(s)
+    assert_close(torch.cat(got), ref, "bfloat16")
+    lens = [1, 130, 64, 7]
+    seqs = [random_tokens(V, n, 70 + n) for n in lens]
+    slots = eng.open(4)[::-1]
+    first = eng.step(slots, [t[:(n + 1) // 2] for t, n in zip(seqs, lens)], "all")
+    rest = eng.step(slots[1:], [t[(n + 1) // 2:] for t, n in list(zip(seqs, lens))[1:]], "all")
+    a = b = 0
+    for i, n in enumerate(lens):
+        h = (n + 1) // 2
+        rows = [first[a:a + h]] + ([rest[b:b + n - h]] if i else [])
+        a, b = a + h, b + (n - h if i else 0)
+        assert_close(torch.cat(rows), plain.forward(seqs[i]), "bfloat16", i)
+    eng.close(slots)
+    spelled.SPELL_SECONDS = 1e9
+    done = len(calls)
+    s = eng.open(1)
+    other = eng.step(s, [toks], "all")
+    eng.close(s)
+    assert len(calls) == done
+    assert_close(other, ref, "bfloat16")
+    eng.cache.check_consistent()
+
+
+def test_spelling_out_pays_for_long_prompts_and_long_contexts_only():
+    raw = dict(KABAPEL["kb-c"]())
+    cfg, t = kabapel_tensors(raw, 1)
+    mix = model_from_tensors(cfg, {k: v.to(DEV) for k, v in t.items()}, "bfloat16").lm.layers[1].mixer
+
+    class Step:
+        is_decode, captured = False, False
+
+        def __init__(self, start, new):
+            self.start_lens, self.new_lens = start, new
+
+    assert not mix._spelled_pays(Step([0], [64])) and not mix._spelled_pays(Step([30, 0], [2, 90]))
+    assert mix._spelled_pays(Step([0], [60000])) and mix._spelled_pays(Step([4000], [2]))
+    one = Step([0], [60000])
+    one.captured = True
+    assert not mix._spelled_pays(one)
+    assert model_from_tensors(cfg, {k: v.to(DEV) for k, v in t.items()}, "float32").lm.layers[1].mixer.spell is None
+
+
+def test_far_key_spelled_out(spelled):
+    test_far_key_at_the_start_and_at_page_borders(kind="tiles", dtype="bfloat16")
+
+
 # ------------------------------------------------------------------ the model through the engine
 
 @pytest.mark.parametrize("name,dtype", CASES)
