@@ -14,13 +14,13 @@
 // the token does not use), so that one down projection over all parts gives the weighted sum of the experts.
 //
 // The grouped products (bfloat16, weights in the matrix cores' fragment layout): the (token, expert) pairs of a step are
-// put in the order of their experts, every expert's run padded to whole tiles of 64 rows (route_groups_kernel: one
-// block counts, places and labels; which row is whose is device data, so a launch depends on sizes only).  A block of
-// expert_gate_up_kernel takes one tile of rows, all of one expert, and 128 of that expert's middle columns: each of its
-// four waves holds 32 columns of the gate and of the up matrix against the tile's four row fragments, gathered from the
-// tokens' rows, and writes act(gate) * up * routing weight, rounded once.  expert_down_kernel is the same walk over
-// the expert's slice of the inner dimension of the side-by-side down matrices; expert_combine_kernel adds a token's
-// rows.  Only the experts that tokens chose are read, and each row meets only its own expert.
+// put in the order of their experts and tokens, every expert's run padded to whole tiles of 64 or 128 rows (a block an
+// expert: route_count_kernel counts, route_place_kernel places and labels; which row is whose is device data, so a launch
+// depends on sizes only).  A block of expert_tile_kernel takes one tile of rows, all of one expert, and 128 of that expert's
+// middle columns (gate and up, then act(gate) * up * routing weight, rounded once) or 256 outputs of its slice of the
+// side-by-side down matrices: the rows, gathered from the tokens', are staged in LDS two k-tiles at a time and shared by the
+// four waves, each of which streams its own weight tiles, a stage ahead.  expert_combine_kernel adds a token's rows.  Only
+// the experts that tokens chose are read, and each row meets only its own expert.
 //
 // Steps of few tokens read every chosen expert's matrices once and do little else (expert_few_*): a block of the first
 // kernel takes one expert and 16 of its middle columns, and ends at once if no token of the step chose it; its four waves
@@ -162,172 +162,218 @@ __global__ void scale_columns_kernel(const TI* __restrict__ x, const float* __re
   }
 }
 
-constexpr int GROUP_TILE = 64;      // rows of a tile: four row fragments of 16
+// ------------------------------------------------------------------------------------------ grouped products
 
-// One block.  w: [T, E] routing weights (zero: not chosen).  row_token / row_weight [R]: the pairs in expert order, every
-// expert's run padded to whole tiles (token -1, weight 0); tile_expert [R / 64] (-1: no rows); token_rows [T, top]:
-// where each token's rows went (-1: fewer than top).
-__global__ __launch_bounds__(1024) void route_groups_kernel(const float* __restrict__ w, int T, int E, int top, int R,
-                                                            int* __restrict__ row_token, float* __restrict__ row_weight,
-                                                            int* __restrict__ tile_expert, int* __restrict__ token_rows) {
-  __shared__ int cnt[MAX_EXPERTS], fill[MAX_EXPERTS], off[MAX_EXPERTS + 1];
-  const int tid = threadIdx.x;
-  for (int e = tid; e < E; e += blockDim.x) cnt[e] = fill[e] = 0;
+// count[e]: the tokens that use expert e.  w: [T, E] routing weights (zero: not chosen).
+__global__ __launch_bounds__(1024) void route_count_kernel(const float* __restrict__ w, int T, int E, int* __restrict__ count) {
+  __shared__ int part[16];
+  const int e = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  int n = 0;
+  for (int t = threadIdx.x; t < T; t += 1024) n += w[(size_t)t * E + e] > 0.f;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) n += __shfl_xor(n, o, 64);
+  if (lane == 0) part[wave] = n;
   __syncthreads();
-  for (long i = tid; i < (long)T * E; i += blockDim.x)
-    if (w[i] > 0.f) atomicAdd(&cnt[i % E], 1);
+  if (threadIdx.x == 0) {
+    int total = 0;
+    for (int i = 0; i < 16; ++i) total += part[i];
+    count[e] = total;
+  }
+}
+
+// A block an expert: its tokens in order into its run of rows.  row_token / row_weight [R] (padding: -1, 0); tile_expert
+// [R / tile] (-1: no rows); token_rows [T, top]: where each token's rows went, in the order of the experts (-1: fewer).
+__global__ __launch_bounds__(1024) void route_place_kernel(const float* __restrict__ w, const int* __restrict__ count, int T, int E, int top,
+                                                           int R, int tile, int* __restrict__ row_token, float* __restrict__ row_weight,
+                                                           int* __restrict__ tile_expert, int* __restrict__ token_rows) {
+  __shared__ int part[17];
+  const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  auto padded = [&](int i) { return (count[i] + tile - 1) / tile * tile; };
+  int before = 0;
+  for (int i = tid; i < e; i += 1024) before += padded(i);
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) before += __shfl_xor(before, o, 64);
+  if (lane == 0) part[wave] = before;
   __syncthreads();
-  if (tid == 0) {
-    int at = 0;
-    for (int e = 0; e < E; ++e) {
-      off[e] = at;
-      at += (cnt[e] + GROUP_TILE - 1) / GROUP_TILE * GROUP_TILE;
+  int off = 0;
+  for (int i = 0; i < 16; ++i) off += part[i];
+  const int mine = count[e], run = padded(e);
+  for (int i = tid; i < run / tile; i += 1024) tile_expert[off / tile + i] = e;
+  if (e == E - 1)
+    for (int i = (off + run) / tile + tid; i < R / tile; i += 1024) tile_expert[i] = -1;
+  for (int i = mine + tid; i < run; i += 1024) {
+    row_token[off + i] = -1;
+    row_weight[off + i] = 0.f;
+  }
+  int base = off;
+  for (int t0 = 0; t0 < T; t0 += 1024) {
+    const int t = t0 + tid;
+    const float x = t < T ? w[(size_t)t * E + e] : 0.f;
+    const unsigned long long m = __ballot(x > 0.f);
+    __syncthreads();                                   // the last round's counts have been read
+    if (lane == 0) part[wave] = __popcll(m);
+    __syncthreads();
+    int at = base, all = 0;
+    for (int i = 0; i < 16; ++i) {
+      const int n = part[i];
+      at += i < wave ? n : 0;
+      all += n;
     }
-    off[E] = at;
-  }
-  __syncthreads();
-  for (int r = tid; r < R; r += blockDim.x) {
-    row_token[r] = -1;
-    row_weight[r] = 0.f;
-  }
-  for (int t = tid; t < R / GROUP_TILE; t += blockDim.x) {
-    const int r = t * GROUP_TILE;
-    int e = -1;
-    if (r < off[E]) {
-      int lo = 0, hi = E - 1;                       // the last expert whose run starts at or before r and is not empty there
-      while (lo < hi) {
-        const int mid = (lo + hi + 1) >> 1;
-        if (off[mid] <= r) lo = mid; else hi = mid - 1;
-      }
-      e = lo;
-    }
-    tile_expert[t] = e;
-  }
-  __syncthreads();
-  for (int t = tid; t < T; t += blockDim.x) {
-    int j = 0;
-    for (int e = 0; e < E && j < top; ++e) {
-      const float x = w[(size_t)t * E + e];
+    base += all;
+    if (t < T) {
+      int slot = 0;                                    // how many of the token's experts come before this one
+      if (x > 0.f || e == E - 1)
+        for (int i = 0; i < e; ++i) slot += w[(size_t)t * E + i] > 0.f;
       if (x > 0.f) {
-        const int r = off[e] + atomicAdd(&fill[e], 1);
+        const int r = at + __popcll(m & ((1ull << lane) - 1ull));
         row_token[r] = t;
         row_weight[r] = x;
-        token_rows[(size_t)t * top + j++] = r;
+        if (slot < top) token_rows[(size_t)t * top + slot] = r;
+        ++slot;
       }
-    }
-    for (; j < top; ++j) token_rows[(size_t)t * top + j] = -1;
-  }
-}
-
-// mid[r, f] = act(gate_e x[token r]) * (up_e x[token r]) * weight r, for the tile's expert e; wf: the fragment layout of
-// [all gates; all ups] ([2 E F, W]); mid: [R, F] bfloat16.  A wave takes CW tiles of 16 columns against the tile's four
-// row fragments: 4 + 2 CW loads for 8 CW products a k-tile.
-template <int CW>
-__global__ __launch_bounds__(256) void expert_gate_up_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ wf,
-                                                             const int* __restrict__ row_token, const float* __restrict__ row_weight,
-                                                             const int* __restrict__ tile_expert, bf16_t* __restrict__ mid,
-                                                             int W, int F, int E, float epi) {
-  constexpr int RS = GROUP_TILE / 16;
-  const int e = tile_expert[blockIdx.x];
-  if (e < 0) return;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
-  const int f0 = (blockIdx.y * 4 + wave) * 16 * CW;
-  if (f0 >= F) return;
-  const int KT = (W + 31) / 32;
-  const bf16_t *wg[CW], *wu[CW];
-#pragma unroll
-  for (int j = 0; j < CW; ++j) {
-    const int f = min(f0 + j * 16, F - 16);           // (a tile beyond the expert's columns repeats the last one; it is not stored)
-    wg[j] = wf + (size_t)((e * F + f) / 16) * KT * 512 + lane * 8;
-    wu[j] = wf + (size_t)(((size_t)E * F + (size_t)e * F + f) / 16) * KT * 512 + lane * 8;
-  }
-  const bf16_t* xr[RS];
-  const int r0 = blockIdx.x * GROUP_TILE;
-#pragma unroll
-  for (int s = 0; s < RS; ++s) xr[s] = x + (size_t)max(row_token[r0 + s * 16 + c], 0) * W;     // (a padded row reads token 0's; its weight is 0)
-  f32x4 ag[CW][RS], au[CW][RS];
-#pragma unroll
-  for (int j = 0; j < CW; ++j)
-#pragma unroll
-    for (int s = 0; s < RS; ++s) ag[j][s] = au[j][s] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int kt = 0; kt < KT; ++kt) {
-    const int k = min(kt * 32 + g * 8, W - 8);       // a row's last, partial k-tile: the weights are zero there
-    u32x4 b[RS], a_g[CW], a_u[CW];
-#pragma unroll
-    for (int j = 0; j < CW; ++j) {
-      a_g[j] = *reinterpret_cast<const u32x4*>(wg[j] + (size_t)kt * 512);
-      a_u[j] = *reinterpret_cast<const u32x4*>(wu[j] + (size_t)kt * 512);
-    }
-#pragma unroll
-    for (int s = 0; s < RS; ++s) b[s] = *reinterpret_cast<const u32x4*>(xr[s] + k);
-#pragma unroll
-    for (int j = 0; j < CW; ++j)
-#pragma unroll
-      for (int s = 0; s < RS; ++s) {
-        ag[j][s] = mfma16(a_g[j], b[s], ag[j][s]);
-        au[j][s] = mfma16(a_u[j], b[s], au[j][s]);
-      }
-  }
-#pragma unroll
-  for (int s = 0; s < RS; ++s) {
-    const int r = r0 + s * 16 + c;
-    const float wr = row_weight[r];
-#pragma unroll
-    for (int j = 0; j < CW; ++j) {
-      if (f0 + j * 16 >= F) continue;
-      f32x4 o;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] = wr == 0.f ? 0.f : gated_act(ag[j][s][i], au[j][s][i], epi, false) * wr;
-      store4(mid, (size_t)r * F, f0 + j * 16 + g * 4, F, o);
+      if (e == E - 1)
+        for (; slot < top; ++slot) token_rows[(size_t)t * top + slot] = -1;
     }
   }
 }
 
-// out[r, n] = sum_f mid[r, f] down_e[n, f] for the tile's expert e; wf: the fragment layout of the down matrices side
-// by side ([W, E F]); out: [R, W] float32.  A wave takes CW tiles of 16 outputs against the tile's four row fragments.
-template <int CW>
-__global__ __launch_bounds__(256) void expert_down_kernel(const bf16_t* __restrict__ mid, const bf16_t* __restrict__ wf,
-                                                          const int* __restrict__ tile_expert, float* __restrict__ out,
-                                                          int W, int F, int E) {
-  constexpr int RS = GROUP_TILE / 16;
-  const int e = tile_expert[blockIdx.x];
-  if (e < 0) return;
+struct GroupArgs {
+  const bf16_t* x;                     // DOWN false: the tokens' rows [T, K]; true: the middle rows [R, K]
+  const bf16_t* wf;                    // fragment layout of [all gates; all ups] ([2 E F, W]) or of the down matrices ([W, E F])
+  const int* row_token; const float* row_weight; const int* tile_expert;
+  bf16_t* mid;                         // [R, F]
+  float* out;                          // [R, W]
+  int K, W, F, E, gx, gy;
+  float epi;
+};
+
+// One tile of 16 TM rows against 4 weight tiles of 16 a wave (gate, up, gate, up; or four of the down matrices).
+template <bool DOWN, int TM>
+__global__ __launch_bounds__(256, 2) void expert_tile_kernel(GroupArgs a) {
+  constexpr int WN = 4, KC = 2, XJ = TM / 4;
+  __shared__ __align__(16) u32x4 xs[2][KC][TM][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
-  const int n0 = (blockIdx.y * 4 + wave) * 16 * CW;
-  if (n0 >= W) return;
-  const int KT = (E * F + 31) / 32, kt0 = e * F / 32, kts = F / 32;      // F is a multiple of 32: an expert's k-tiles are its own
-  const int n_tiles = (W + 15) / 16;
-  const bf16_t* wd[CW];
+  // blocks that share weight tiles (neighbouring row tiles of one expert) run on the same XCD
+  const int id = blockIdx.x, per = (a.gx * a.gy + 7) >> 3, item = (id & 7) * per + (id >> 3);
+  if ((id >> 3) >= per || item >= a.gx * a.gy) return;
+  const int bx = item / a.gy, by = item % a.gy, e = a.tile_expert[by], r0 = by * 16 * TM;
+  if (e < 0) return;
+  const int KT = (a.K + 31) / 32;                          // (DOWN: F is a multiple of 32, an expert's k-tiles are its own)
+  const bf16_t* wsrc[WN];
+  int col[WN];                                             // the first column of the wave's tile i; the matrix's width or more: none
 #pragma unroll
-  for (int j = 0; j < CW; ++j) wd[j] = wf + ((size_t)min(n0 / 16 + j, n_tiles - 1) * KT + kt0) * 512 + lane * 8;
-  const int r0 = blockIdx.x * GROUP_TILE;
-  const bf16_t* mr[RS];
-#pragma unroll
-  for (int s = 0; s < RS; ++s) mr[s] = mid + (size_t)(r0 + s * 16 + c) * F + g * 8;
-  f32x4 acc[CW][RS];
-#pragma unroll
-  for (int j = 0; j < CW; ++j)
-#pragma unroll
-    for (int s = 0; s < RS; ++s) acc[j][s] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int kt = 0; kt < kts; ++kt) {
-    u32x4 a[CW], b[RS];
-#pragma unroll
-    for (int j = 0; j < CW; ++j) a[j] = *reinterpret_cast<const u32x4*>(wd[j] + (size_t)kt * 512);
-#pragma unroll
-    for (int s = 0; s < RS; ++s) b[s] = *reinterpret_cast<const u32x4*>(mr[s] + kt * 32);
-#pragma unroll
-    for (int j = 0; j < CW; ++j)
-#pragma unroll
-      for (int s = 0; s < RS; ++s) acc[j][s] = mfma16(a[j], b[s], acc[j][s]);
+  for (int i = 0; i < WN; ++i) {
+    if (DOWN) {
+      const int n = (bx * 4 + wave) * WN + i, n_tiles = (a.W + 15) / 16;
+      col[i] = n * 16;
+      wsrc[i] = a.wf + ((size_t)min(n, n_tiles - 1) * ((size_t)a.E * a.F / 32) + (size_t)e * a.F / 32) * 512 + lane * 8;
+    } else {
+      const int p = (bx * 4 + wave) * (WN / 2) + (i >> 1), f = min(p, a.F / 16 - 1);
+      col[i] = p * 16;
+      wsrc[i] = a.wf + (((i & 1) ? (size_t)a.E * a.F / 16 : 0) + (size_t)e * a.F / 16 + f) * KT * 512 + lane * 8;
+    }
   }
+  const bf16_t* xsrc[XJ];
 #pragma unroll
-  for (int j = 0; j < CW; ++j) {
-    if (n0 + j * 16 >= W) continue;
-#pragma unroll
-    for (int s = 0; s < RS; ++s) store4(out, (size_t)(r0 + s * 16 + c) * W, n0 + j * 16 + g * 4, W, acc[j][s]);
+  for (int j = 0; j < XJ; ++j) {
+    const int r = r0 + (XJ * wave + j) * 16 + c;
+    xsrc[j] = a.x + (size_t)(DOWN ? r : max(a.row_token[r], 0)) * a.K;       // (a padded row reads token 0's; its weight is 0)
   }
+  f32x4 acc[WN][TM];
+#pragma unroll
+  for (int i = 0; i < WN; ++i)
+#pragma unroll
+    for (int j = 0; j < TM; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const bf16_t* zero = reinterpret_cast<const bf16_t*>(g_zero_tile) + lane * 8;
+  u32x4 xr[KC][XJ], wk[KC][WN];
+  auto stage_load = [&](int s) {                           // beyond the last k-tile the weights are zeros
+#pragma unroll
+    for (int kc = 0; kc < KC; ++kc)
+#pragma unroll
+      for (int j = 0; j < XJ; ++j) xr[kc][j] = *reinterpret_cast<const u32x4*>(xsrc[j] + min((s * KC + kc) * 32 + g * 8, a.K - 8));
+  };
+  auto stage_store = [&](int buf) {
+#pragma unroll
+    for (int kc = 0; kc < KC; ++kc)
+#pragma unroll
+      for (int j = 0; j < XJ; ++j) xs[buf][kc][XJ * wave + j][lane] = xr[kc][j];
+  };
+  const int S = (KT + KC - 1) / KC;
+  stage_load(0);
+  stage_store(0);
+#pragma unroll
+  for (int kc = 0; kc < KC; ++kc)
+#pragma unroll
+    for (int i = 0; i < WN; ++i) wk[kc][i] = *reinterpret_cast<const u32x4*>(kc < KT ? wsrc[i] + (size_t)kc * 512 : zero);
+  auto stage_mfma = [&](int s, bool more) {
+#pragma unroll
+    for (int kc = 0; kc < KC; ++kc) {
+      u32x4 xf[TM];
+#pragma unroll
+      for (int j = 0; j < TM; ++j) xf[j] = xs[s & 1][kc][j][lane];
+      const int next = (s + 1) * KC + kc;
+#pragma unroll
+      for (int i = 0; i < WN; ++i) {
+#pragma unroll
+        for (int j = 0; j < TM; ++j) acc[i][j] = mfma16(wk[kc][i], xf[j], acc[i][j]);
+        if (more) {                                        // this tile's registers are free: the same tile of the next stage
+          __builtin_amdgcn_sched_barrier(0);
+          wk[kc][i] = *reinterpret_cast<const u32x4*>(next < KT ? wsrc[i] + (size_t)next * 512 : zero);
+          __builtin_amdgcn_sched_barrier(0);
+        }
+      }
+    }
+  };
+  for (int s = 0; s + 1 < S; ++s) {
+    stage_load(s + 1);
+    __builtin_amdgcn_sched_barrier(0);
+    __syncthreads();
+    stage_mfma(s, true);
+    stage_store((s + 1) & 1);
+  }
+  __syncthreads();
+  stage_mfma(S - 1, false);
+#pragma unroll
+  for (int j = 0; j < TM; ++j) {
+    const int r = r0 + j * 16 + c;
+    if (DOWN) {
+#pragma unroll
+      for (int i = 0; i < WN; ++i)
+        if (col[i] < a.W) store4(a.out, (size_t)r * a.W, col[i] + g * 4, a.W, acc[i][j]);
+    } else {
+      const float wr = a.row_weight[r];
+#pragma unroll
+      for (int p = 0; p < WN / 2; ++p) {
+        if (col[2 * p] >= a.F) continue;
+        f32x4 o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = wr == 0.f ? 0.f : gated_act(acc[2 * p][j][i], acc[2 * p + 1][j][i], a.epi, false) * wr;
+        store4(a.mid, (size_t)r * a.F, col[2 * p] + g * 4, a.F, o);
+      }
+    }
+  }
+}
+
+// Rows of a tile: 128 where the experts' runs are long enough on average, else 64.
+int group_tile(int T, int E, int top) { return (long)T * top >= 96L * E ? 128 : 64; }
+
+template <int TM>
+int launch_group(GroupArgs a, const void* gate_up, const void* down, const void* x, int R, hipStream_t stream) {
+  const int W = a.W, F = a.F;
+  a.gy = R / (16 * TM);
+  a.x = (const bf16_t*)x;
+  a.wf = (const bf16_t*)gate_up;
+  a.K = W;
+  a.gx = ceil_div(F, 128);
+  expert_tile_kernel<false, TM><<<8 * ceil_div((long)a.gx * a.gy, 8), 256, 0, stream>>>(a);
+  ALICE_LAUNCH_CHECK();
+  a.x = a.mid;
+  a.wf = (const bf16_t*)down;
+  a.K = F;
+  a.gx = ceil_div(W, 256);
+  expert_tile_kernel<true, TM><<<8 * ceil_div((long)a.gx * a.gy, 8), 256, 0, stream>>>(a);
+  ALICE_LAUNCH_CHECK();
+  return 0;
 }
 
 // ------------------------------------------------------------------------------------------ few tokens
@@ -550,14 +596,15 @@ void launch_combine(const float* rows, const int* token_rows, int top, const flo
 
 // Rows that the grouped products of a step of T tokens need: every pair and every expert's padding, in whole tiles.
 extern "C" long alice_expert_rows(int T, int E, int top) {
-  return ((long)T * top + (long)E * (GROUP_TILE - 1) + GROUP_TILE - 1) / GROUP_TILE * GROUP_TILE;
+  const int tile = group_tile(T, E, top);
+  return ((long)T * top + (long)E * (tile - 1) + tile - 1) / tile * tile;
 }
 
 // The routed feed-forward by grouped products, see the top of the file.  x: [T, W] bfloat16; weights: [T, E] float32 of
 // alice_route_topk; gate_up, down: fragment layouts of [2 E F, W] and [W, E F]; y: [T, W] float32.  Workspaces for
 // side, shared: null, or what alice_expert_combine adds (the identity experts' weight and the shared expert's gate a token,
-// the shared expert's partial rows).  R = alice_expert_rows(T, E, top): ints [2 R + R / 64 + T top] (row_token, tile_expert, token_rows; the row weights
-// share the ints' buffer as floats), mid [R, F] bfloat16, rows [R, W] float32.
+// the shared expert's partial rows).  R = alice_expert_rows(T, E, top): ints [2 R + R / 64 + T top + E] (row_token, tile_expert, token_rows, the experts' counts; the row
+// weights share the ints' buffer as floats), mid [R, F] bfloat16, rows [R, W] float32.
 extern "C" int alice_expert_products(const void* x, const float* weights, const void* gate_up, const void* down, float* y, int* ints,
                                      void* mid, float* rows, int T, int W, int F, int E, int top, float epi, const float* side,
                                      const float* shared, int n_shared, hipStream_t stream) {
@@ -566,20 +613,28 @@ extern "C" int alice_expert_products(const void* x, const float* weights, const 
   ALICE_CHECK(T >= 1 && E >= 1 && E <= MAX_EXPERTS && top >= 1 && top <= E, "expert_products: 1 <= top <= experts <= %d", MAX_EXPERTS);
   ALICE_CHECK(W >= 8 && W % 8 == 0 && F >= 32 && F % 32 == 0, "expert_products: the width must be a multiple of 8 and the experts' a multiple of 32");
   const long R = alice_expert_rows(T, E, top);
-  ALICE_CHECK(R / GROUP_TILE <= 2147483647L / 2 && (long)T * E < (1L << 40), "expert_products: too many rows for one launch");
+  const int tile = group_tile(T, E, top);
+  ALICE_CHECK(R < (1L << 30) && (long)T * E < (1L << 40) && R / tile * (long)ceil_div(F > W ? F : W, 128) < (1L << 28), "expert_products: too many rows for one launch");
   int* row_token = ints;
   float* row_weight = reinterpret_cast<float*>(ints + R);
   int* tile_expert = ints + 2 * R;
-  int* token_rows = tile_expert + R / GROUP_TILE;
-  route_groups_kernel<<<1, 1024, 0, stream>>>(weights, T, E, top, (int)R, row_token, row_weight, tile_expert, token_rows);
+  int* token_rows = tile_expert + R / tile;
+  int* count = token_rows + (long)T * top;
+  route_count_kernel<<<E, 1024, 0, stream>>>(weights, T, E, count);
   ALICE_LAUNCH_CHECK();
-  dim3 g1((unsigned)(R / GROUP_TILE), ceil_div(F, 128));
-  expert_gate_up_kernel<2><<<g1, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, row_token, row_weight, tile_expert,
-                                                (bf16_t*)mid, W, F, E, epi);
+  route_place_kernel<<<E, 1024, 0, stream>>>(weights, count, T, E, top, (int)R, tile, row_token, row_weight, tile_expert, token_rows);
   ALICE_LAUNCH_CHECK();
-  dim3 g2((unsigned)(R / GROUP_TILE), ceil_div(W, 256));
-  expert_down_kernel<4><<<g2, 256, 0, stream>>>((const bf16_t*)mid, (const bf16_t*)down, tile_expert, rows, W, F, E);
-  ALICE_LAUNCH_CHECK();
+  GroupArgs a{};
+  a.row_token = row_token;
+  a.row_weight = row_weight;
+  a.tile_expert = tile_expert;
+  a.mid = (bf16_t*)mid;
+  a.out = rows;
+  a.W = W;
+  a.F = F;
+  a.E = E;
+  a.epi = epi;
+  if (const int rc = tile == 128 ? launch_group<8>(a, gate_up, down, x, (int)R, stream) : launch_group<4>(a, gate_up, down, x, (int)R, stream)) return rc;
   launch_combine<bf16_t>(rows, token_rows, top, nullptr, 0, (const bf16_t*)x, side, shared, n_shared, y, T, W, stream);
   ALICE_LAUNCH_CHECK();
   return 0;

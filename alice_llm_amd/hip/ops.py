@@ -1319,7 +1319,7 @@ def expert_products(x: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tenso
     _dev(down, "down", torch.bfloat16, (frag_rows(W) * (-(-(E * F) // 32) * 32),))
     _dev(y, "y", torch.float32, (T, W))
     R = library().alice_expert_rows(T, E, int(top))
-    ints = torch.empty((2 * R + R // 64 + T * top,), dtype=torch.int32, device=x.device)
+    ints = torch.empty((2 * R + R // 64 + T * top + E,), dtype=torch.int32, device=x.device)
     mid = torch.empty((R, F), dtype=torch.bfloat16, device=x.device)
     rows = torch.empty((R, W), dtype=torch.float32, device=x.device)
     _call("alice_expert_products", x.data_ptr(), weights.data_ptr(), gate_up.data_ptr(), down.data_ptr(), y.data_ptr(),

@@ -37,8 +37,8 @@ from .feedforward import GatedMLP
 from .linear import Linear
 
 _GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
-GROUPED_FROM_TOKENS = 128      # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles);
-                               # below, one pass over all experts' matrices is as fast or faster (measured at 16 experts, 2 a token)
+GROUPED_FROM_TOKENS = 64       # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles): as
+                               # fast as one pass over all experts' matrices with 16 experts, faster with 64 (2 a token)
 FEW_CHOICES = 1.9              # steps of at most 64 tokens whose tokens x top is at most this many times the router's outputs read
                                # the chosen experts only (beyond, one pass over all of them is as fast: measured at 16 and 64 experts)
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
@@ -185,7 +185,7 @@ class ExpertMLP(Part):
         b = 1
         while b < tokens:
             b *= 2
-        if not (b <= ops.EXPERT_FEW_MAX_TOKENS and b * self.top <= FEW_CHOICES * self.outputs and self.gate_up.layout == ops.LAYOUT_FRAG16):
+        if not (b < GROUPED_FROM_TOKENS and b * self.top <= FEW_CHOICES * self.outputs and self.gate_up.layout == ops.LAYOUT_FRAG16):
             return 0
         none = (1.0 - self.top / self.outputs) ** tokens
         return int(none * (self.gate_up.nbytes() + self.down.nbytes()))
