@@ -41,10 +41,10 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const bf16_t* __rest
   int p = 0;
   const int v = blockIdx.x, s = page_owner(v, context_lens, n_seqs, p);
   if (s < 0) return;
-  if (threadIdx.x == 0) table[(size_t)s * table_stride + p] = v;
+  if (threadIdx.x == 0 && blockIdx.y == 0) table[(size_t)s * table_stride + p] = v;
   const int len = context_lens[s], per = R / 8;
   const int* bt = block_table + (size_t)s * bt_stride;
-  for (int i = threadIdx.x; i < PAGE * per; i += 256) {
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < PAGE * per; i += 256 * gridDim.y) {
     const int t = i / per, e = (i % per) * 8, pos = p * PAGE + t;
     u32x4 x = {0u, 0u, 0u, 0u};
     if (pos < len) x = *reinterpret_cast<const u32x4*>(cached_row(pool, bt, page_size, D, pos) + e);
@@ -139,7 +139,7 @@ extern "C" int alice_latent_gather(const void* pool, const int* context_lens, in
               rot_dim >= 0 && rot_dim % 8 == 0, "latent_gather: bad sizes");
   ALICE_CHECK(aligned16(pool) && aligned16(rows), "latent_gather: operands are not aligned");
   if (n_pages == 0) return 0;
-  latent_gather_kernel<<<n_pages, 256, 0, stream>>>((const bf16_t*)pool, context_lens, n_seqs, block_table, bt_stride, page_size, kv_rank,
+  latent_gather_kernel<<<dim3(n_pages, 8), 256, 0, stream>>>((const bf16_t*)pool, context_lens, n_seqs, block_table, bt_stride, page_size, kv_rank,
                                                     kv_rank + rot_dim, (bf16_t*)rows, table, table_stride);
   ALICE_LAUNCH_CHECK();
   return 0;
