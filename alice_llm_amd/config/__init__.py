@@ -7,6 +7,7 @@ from .telulorn import TelulornConfig
 from .pefitar import PefitarConfig
 from .vifirax import VifiraxConfig
 from .kabapel import KabapelConfig
+from .vazilorn import VazilornConfig
 from . import presets
 
 register_architecture("Gemma2ForCausalLM", Gemma2Config, model_type="gemma2")
@@ -15,3 +16,4 @@ register_architecture("Telulorn", TelulornConfig)
 register_architecture("Pefitar", PefitarConfig)
 register_architecture("Vifirax", VifiraxConfig)
 register_architecture("Kabapel", KabapelConfig)
+register_architecture("Vazilorn", VazilornConfig)

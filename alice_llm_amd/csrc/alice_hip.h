@@ -4,7 +4,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 
-#define ALICE_ABI_VERSION 13
+#define ALICE_ABI_VERSION 14
 
 #define ALICE_EPI_NONE 0
 #define ALICE_EPI_GEGLU 1     // W = [gate; up] stacked; epi_param 0: y = gelu_tanh(gate x) * (up x); epi_param = limit > 0:
@@ -51,6 +51,12 @@ int alice_add_norm(float* resid, const float* branch, int n_partials, long parti
                    const void* w_post, const void* w_pre, const void* b_pre, int w_dtype, void* out, int out_dtype,
                    const int* rows, int T, int H, float eps_post, float eps_pre, float off_post,
                    float off_pre, int full_precision, int out_layout, hipStream_t stream);
+
+// The same with norms that act element by element, tanh(a v) * w + b (no mean, no variance): resid += post(sum of the branch's
+// partial results), out = pre(resid).  post, pre: float32 weight and bias [H] with a factor a, each pair null for none.
+int alice_add_dyntanh(float* resid, const float* branch, int n_partials, long partial_stride, const float* w_post,
+                      const float* b_post, float a_post, const float* w_pre, const float* b_pre, float a_pre, void* out,
+                      int out_dtype, const int* rows, int T, int H, int full_precision, int out_layout, hipStream_t stream);
 
 // resid += sum over n branches of norm_j(sum of the branch's partial results), norm_j(b) = b / sqrt(mean(b^2) +
 // eps_j) * (offsets_j + weights_j) where weights_j is given and b itself where it is null; out (optional): the new
@@ -157,10 +163,11 @@ int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width, const flo
                       void* v_pool, int out_dtype, const float* cos_t, const float* sin_t, int rotary_dim,
                       int interleaved, const float* vcos, const float* vsin, const int* positions,
                       const int* seq_of_token, const int* block_table, int bt_stride, int T, int nH, int nKV,
-                      int d, int dv, int page_size, int n_pages, const float* norm_w, float norm_eps, float* inv_rms,
-                      hipStream_t stream);
+                      int d, int dv, int page_size, int n_pages, const float* norm_w, int norm_heads, float norm_eps,
+                      float* inv_rms, hipStream_t stream);
 // (norm_w: float32 [nH d + nKV d] or null: the q columns and the k columns are each RMS-normed over the whole
-// projection, after the bias and before the rotation; inv_rms: float32 [T, 2] workspace.)
+// projection, after the bias and before the rotation; inv_rms: float32 [T, 2] workspace.  With norm_heads: float32 [2, d],
+// every q head and every k head by its own root mean square times the first or second row; no workspace.)
 // x[t, c] += a[t, c] + v[c] (either may be null)
 int alice_add_rows(float* x, const float* a, const float* v, int T, int W, hipStream_t stream);
 // Gated linear attention over a step's tokens, see gla.hip.
@@ -212,12 +219,14 @@ long alice_expert_rows(int T, int E, int top);
 int alice_expert_products(const void* x, const float* weights, const void* gate_up, const void* down, float* y, int* ints,
                           void* mid, float* rows, int T, int W, int F, int E, int top, float epi, const float* side, const float* shared,
                           int n_shared, hipStream_t stream);
-// A router that scores all n = experts + identity outputs by a softmax: z [T, z_w] float32; choice = score + correction [n]; of
-// `groups` equal runs of neighbours the `keep` with the largest choice stay, of those the `top` largest choices serve the
-// token, weighted by score / (sum of the chosen scores + 1e-20).  w [T, experts] (zero: not chosen); side [T, 2]: the weight
-// of the identity outputs together, and with has_shared sigmoid(z[t, n]) (else 0).
+// A router that scores all n = experts + identity outputs by a softmax (or, with `sigmoid`, each by its own sigmoid): z [T, z_w]
+// float32; choice = score + correction [n]; of `groups` equal runs of neighbours the `keep` with the largest choice (group_best
+// 1) or the largest sum of their two largest choices (2) stay, of those the `top` largest choices serve the token, weighted by
+// weight_scale * score / (sum of the chosen scores + 1e-20).  w [T, experts] (zero: not chosen); side [T, 2]: the weight
+// of the identity outputs together, and the shared expert's factor: shared_mode 0: 0, 1: sigmoid(z[t, n]), 2: 1.
 int alice_route_scored(const float* z, int z_w, const float* correction, float* w, float* side, int T, int experts, int identity,
-                       int top, int groups, int keep, int has_shared, hipStream_t stream);
+                       int top, int groups, int keep, int shared_mode, int sigmoid, int group_best, float weight_scale,
+                       hipStream_t stream);
 // The routed feed-forward for at most 64 tokens: only the chosen experts' matrices are read, the shared expert is one more.
 int alice_expert_few_splits(int W);
 int alice_expert_few(const void* x, const float* w, const float* side, const void* gate_up, const void* down, const void* shared_gate_up,

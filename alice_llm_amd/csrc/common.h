@@ -136,6 +136,13 @@ __device__ __forceinline__ float unary_act(float v, float p, bool full) {
 }
 __device__ __forceinline__ float sigmoid_f(float z, bool full) { return 1.f / (1.f + (full ? expf(-z) : __expf(-z))); }
 
+// Where element (row r, column i) of a [T, H] bfloat16 output goes: row-major, or fragment order for the
+// matrix-core kernels ([T/16][H/32][64][8], see linear_mfma.hip).
+__device__ __forceinline__ size_t out_index(int layout, int r, int i, int H) {
+  if (layout == 0) return (size_t)r * H + i;
+  return ((size_t)((size_t)(r >> 4) * (H >> 5) + (i >> 5)) * 64 + ((i & 31) >> 3) * 16 + (r & 15)) * 8 + (i & 7);
+}
+
 // ---- host side -------------------------------------------------------------------------
 void alice_set_error(const char* fmt, ...);
 

@@ -51,13 +51,6 @@ extern "C" int alice_embed(const int* tokens, const void* table, int table_dtype
   return 0;
 }
 
-// Where element (row r, column i) of a [T, H] bfloat16 output goes: row-major, or fragment order for the
-// matrix-core kernels ([T/16][H/32][64][8], see linear_mfma.hip).
-__device__ __forceinline__ size_t out_index(int layout, int r, int i, int H) {
-  if (layout == 0) return (size_t)r * H + i;
-  return ((size_t)((size_t)(r >> 4) * (H >> 5) + (i >> 5)) * 64 + ((i & 31) >> 3) * 16 + (r & 15)) * 8 + (i & 7);
-}
-
 // ---------------------------------------------------------------- residual add + norms
 // One block per row r (source row rows ? rows[r] : r):
 //   b   = sum over `n_partials` slices of `branch` (slice stride `partial_stride` elements)

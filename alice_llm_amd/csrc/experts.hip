@@ -4,10 +4,11 @@
 // it picks the `top` largest (of equal logits the lower index), takes the softmax over the picked logits only, and
 // writes a dense row of weights [E]: the picked experts' weights, zero elsewhere.  All in 32-bit.
 //
-// route_scored_kernel: a router whose scores are a softmax over all its outputs, the last of which may be identity experts
-// (they give the token's own input back and have no matrices).  A correction is added to the scores for the choice
-// only; the outputs form equal groups of neighbours, and only experts of the groups with the largest choice in them can
-// be chosen; the chosen experts' scores, divided by their sum, are the weights.  A wave per token, all in 32-bit.
+// route_scored_kernel: a router whose scores are a softmax over all its outputs, or a sigmoid of each.  The last outputs may
+// be identity experts (they give the token's own input back and have no matrices).  A correction is added to the scores
+// for the choice only; the outputs form equal groups of neighbours, and only experts of the groups with the largest choice
+// in them (or the largest sum of their two largest choices) can be chosen; the chosen experts' scores, divided by their
+// sum and times a constant, are the weights.  A wave per token, all in 32-bit.
 //
 // scale_columns_kernel: y[t, e F + j] = x[t, e F + j] * w[t, e] for rows made of E parts of F columns: the experts'
 // middle activations side by side, each multiplied by its expert's weight of that token (a zero for an expert that
@@ -80,21 +81,27 @@ __device__ __forceinline__ void wave_argmax(float& best, int& at) {
 
 __global__ __launch_bounds__(64) void route_scored_kernel(const float* __restrict__ z, int z_w, const float* __restrict__ correction,
                                                           float* __restrict__ w, float* __restrict__ side, int E, int n, int top,
-                                                          int groups, int keep, int has_shared) {
+                                                          int groups, int keep, int shared_mode, int sigmoid, int group_best,
+                                                          float weight_scale) {
   __shared__ float score[MAX_EXPERTS], choice[MAX_EXPERTS], wt[MAX_EXPERTS], best_of[MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* zt = z + (size_t)t * z_w;
-  float m = -INFINITY;
-  for (int e = lane; e < n; e += 64) m = fmaxf(m, zt[e]);
-  m = wave_max(m);
-  float sum = 0.f;
-  for (int e = lane; e < n; e += 64) {
-    const float x = expf(zt[e] - m);
-    score[e] = x;
-    sum += x;
+  float sum = 1.f;
+  if (sigmoid) {
+    for (int e = lane; e < n; e += 64) score[e] = 1.f / (1.f + expf(-zt[e]));
+  } else {
+    float m = -INFINITY;
+    for (int e = lane; e < n; e += 64) m = fmaxf(m, zt[e]);
+    m = wave_max(m);
+    sum = 0.f;
+    for (int e = lane; e < n; e += 64) {
+      const float x = expf(zt[e] - m);
+      score[e] = x;
+      sum += x;
+    }
+    sum = wave_sum(sum);
   }
-  sum = wave_sum(sum);
-  for (int e = lane; e < n; e += 64) {
+  for (int e = lane; e < n; e += 64) {                 // (a lane reads the scores that it wrote itself)
     const float x = score[e] / sum;
     score[e] = x;
     choice[e] = x + (correction ? correction[e] : 0.f);
@@ -104,9 +111,13 @@ __global__ __launch_bounds__(64) void route_scored_kernel(const float* __restric
   if (keep < groups) {
     const int gs = n / groups;
     for (int g = lane; g < groups; g += 64) {
-      float b = -INFINITY;
-      for (int e = g * gs; e < (g + 1) * gs; ++e) b = fmaxf(b, choice[e]);
-      best_of[g] = b;
+      float b = -INFINITY, second = -INFINITY;
+      for (int e = g * gs; e < (g + 1) * gs; ++e) {
+        const float x = choice[e];
+        second = fmaxf(second, fminf(b, x));
+        b = fmaxf(b, x);
+      }
+      best_of[g] = group_best == 2 && gs > 1 ? b + second : b;
     }
     __syncthreads();
     for (int k = 0; k < keep; ++k) {                   // the kept groups are marked by +infinity
@@ -139,7 +150,7 @@ __global__ __launch_bounds__(64) void route_scored_kernel(const float* __restric
     }
     __syncthreads();
   }
-  const float inv = 1.f / (total + 1e-20f);
+  const float inv = weight_scale / (total + 1e-20f);
   float id = 0.f;
   for (int e = lane; e < n; e += 64) {
     const float x = wt[e] * inv;
@@ -149,7 +160,7 @@ __global__ __launch_bounds__(64) void route_scored_kernel(const float* __restric
   id = wave_sum(id);
   if (lane == 0) {
     side[2 * (size_t)t] = id;
-    side[2 * (size_t)t + 1] = has_shared ? 1.f / (1.f + expf(-zt[n])) : 0.f;
+    side[2 * (size_t)t + 1] = shared_mode == 1 ? 1.f / (1.f + expf(-zt[n])) : (shared_mode == 2 ? 1.f : 0.f);
   }
 }
 
@@ -684,15 +695,17 @@ extern "C" int alice_route_topk(const float* z, const float* bias, float* w, int
 }
 
 extern "C" int alice_route_scored(const float* z, int z_w, const float* correction, float* w, float* side, int T, int experts,
-                                  int identity, int top, int groups, int keep, int has_shared, hipStream_t stream) {
+                                  int identity, int top, int groups, int keep, int shared_mode, int sigmoid, int group_best,
+                                  float weight_scale, hipStream_t stream) {
   ALICE_CHECK(z && w && side, "route_scored: a pointer is missing");
   const int n = experts + identity;
   ALICE_CHECK(T >= 0 && experts >= 1 && identity >= 0 && n <= MAX_EXPERTS && top >= 1 && top <= n, "route_scored: 1 <= top <= outputs <= %d", MAX_EXPERTS);
   ALICE_CHECK(groups >= 1 && n % groups == 0 && keep >= 1 && keep <= groups && (long)keep * (n / groups) >= top,
               "route_scored: %d groups must divide %d outputs, and the kept ones hold at least `top` of them", groups, n);
-  ALICE_CHECK(z_w >= n + (has_shared ? 1 : 0), "route_scored: rows of %d logits are too short", z_w);
+  ALICE_CHECK(shared_mode >= 0 && shared_mode <= 2 && (group_best == 1 || group_best == 2), "route_scored: unknown shared_mode %d or group_best %d", shared_mode, group_best);
+  ALICE_CHECK(z_w >= n + (shared_mode == 1 ? 1 : 0), "route_scored: rows of %d logits are too short", z_w);
   if (T == 0) return 0;
-  route_scored_kernel<<<T, 64, 0, stream>>>(z, z_w, correction, w, side, experts, n, top, groups, keep, has_shared);
+  route_scored_kernel<<<T, 64, 0, stream>>>(z, z_w, correction, w, side, experts, n, top, groups, keep, shared_mode, sigmoid, group_best, weight_scale);
   ALICE_LAUNCH_CHECK();
   return 0;
 }

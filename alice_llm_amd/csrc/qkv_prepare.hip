@@ -11,7 +11,9 @@
 //
 // With norm weights the q columns (all heads together) and the k columns (likewise) are each divided by their root
 // mean square over the whole projection, eps inside the root, and multiplied by a weight of that length, after the
-// bias and before the rotation; projection_rms_kernel finds the two factors of every token first, in 32-bit.
+// bias and before the rotation; projection_rms_kernel finds the two factors of every token first, in 32-bit.  With a norm a
+// head instead, every q head and every k head is divided by its own root mean square and multiplied by a weight of d numbers
+// that the q heads share (and one that the k heads share): qkv_prepare_heads_kernel, a wave a head, the head in registers.
 #include "common.h"
 #include "alice_hip.h"
 #include "kv_layout.h"
@@ -104,6 +106,82 @@ __global__ void qkv_prepare_kernel(const TI* __restrict__ rows, int row_w, const
   }
 }
 
+// A wave per (token, head), four heads a block; a lane holds up to two pairs of the head (d <= 256): the rotation's pairs
+// first, then the unrotated dimensions two by two (of an odd number the last alone).  norm_w: [2, d], the q heads' weight and
+// the k heads'.
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void qkv_prepare_heads_kernel(const TI* __restrict__ rows, int row_w, const float* __restrict__ bias,
+                                                                const float* __restrict__ norm_w, float eps,
+                                                                TO* __restrict__ q_out, TO* __restrict__ k_pool, TO* __restrict__ v_pool,
+                                                                const float* __restrict__ cos_t, const float* __restrict__ sin_t, int R,
+                                                                int interleaved, const int* __restrict__ positions,
+                                                                const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
+                                                                int bt_stride, int nH, int nKV, int d, int dv, int page_size, int n_pages,
+                                                                int n_heads) {
+  const int t = blockIdx.x, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (h >= n_heads) return;
+  const int pos = positions[t];
+  const TI* row = rows + (size_t)t * row_w;
+  int page = -1;
+  if (k_pool) {
+    page = block_table[(size_t)seq_of_token[t] * bt_stride + pos / page_size];
+    if (page < 0 || page >= n_pages) page = -1;
+  }
+  const int tp = pos % page_size;
+  if (h >= nH + nKV) {                                          // a value head: as it is
+    if (page < 0) return;
+    const int hv = h - nH - nKV;
+    const size_t col0 = (size_t)(nH + nKV) * d + (size_t)hv * dv;
+    TO* dst = v_pool + (((size_t)page * nKV + hv) * page_size + tp) * dv;
+    for (int e = lane; e < dv; e += 64) {
+      float x = load_f32(row, col0 + e);
+      if (bias) x += bias[col0 + e];
+      store_f32(dst, e, x);
+    }
+    return;
+  }
+  const bool is_q = h < nH;
+  const size_t col0 = (size_t)h * d;
+  const float* w = norm_w + (is_q ? 0 : d);
+  const int half = R >> 1, n_pairs = half + (d - R + 1) / 2;
+  int e0[2], e1[2];
+  bool on0[2], on1[2];
+  float x0[2], x1[2], w0[2], w1[2], cs[2], sn[2];
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {                                 // every load before the first use
+    const int i = lane + 64 * k;
+    const bool turned = i < half;
+    e0[k] = turned ? (interleaved ? 2 * i : i) : R + 2 * (i - half);
+    e1[k] = turned ? (interleaved ? 2 * i + 1 : i + half) : e0[k] + 1;
+    on0[k] = i < n_pairs;
+    on1[k] = on0[k] && e1[k] < d;
+    x0[k] = on0[k] ? load_f32(row, col0 + e0[k]) : 0.f;
+    x1[k] = on1[k] ? load_f32(row, col0 + e1[k]) : 0.f;
+    w0[k] = on0[k] ? w[e0[k]] : 0.f;
+    w1[k] = on1[k] ? w[e1[k]] : 0.f;
+    cs[k] = turned ? cos_t[(size_t)pos * half + i] : 1.f;
+    sn[k] = turned ? sin_t[(size_t)pos * half + i] : 0.f;
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    if (bias && on0[k]) x0[k] += bias[col0 + e0[k]];
+    if (bias && on1[k]) x1[k] += bias[col0 + e1[k]];
+    ss = fmaf(x0[k], x0[k], fmaf(x1[k], x1[k], ss));
+  }
+  ss = wave_sum(ss);
+  if (!is_q && page < 0) return;
+  const float inv = 1.f / sqrtf(ss / (float)d + eps);
+  TO* dst = is_q ? q_out + ((size_t)t * nH + h) * d : k_pool + (((size_t)page * nKV + (h - nH)) * page_size + tp) * d;
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    float y0, y1;
+    rotate_pair(x0[k] * inv * w0[k], x1[k] * inv * w1[k], cs[k], sn[k], y0, y1);
+    if (on0[k]) store_f32(dst, e0[k], y0);
+    if (on1[k]) store_f32(dst, e1[k], y1);
+  }
+}
+
 // x[t, c] += (a ? a[t, c] : 0) + (v ? v[c] : 0)
 __global__ void add_rows_kernel(float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ v, long n, int W) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
@@ -120,10 +198,11 @@ extern "C" int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width
                                  void* v_pool, int out_dtype, const float* cos_t, const float* sin_t, int rotary_dim,
                                  int interleaved, const float* vcos, const float* vsin, const int* positions,
                                  const int* seq_of_token, const int* block_table, int bt_stride, int T, int nH, int nKV,
-                                 int d, int dv, int page_size, int n_pages, const float* norm_w, float norm_eps, float* inv_rms,
-                                 hipStream_t stream) {
+                                 int d, int dv, int page_size, int n_pages, const float* norm_w, int norm_heads, float norm_eps,
+                                 float* inv_rms, hipStream_t stream) {
   ALICE_CHECK(dtype_ok(rows_dtype) && dtype_ok(out_dtype), "qkv_prepare: unknown dtype");
-  ALICE_CHECK(norm_w == nullptr || (inv_rms != nullptr && norm_eps > 0.f), "qkv_prepare: the projection norm needs its workspace and a positive eps");
+  ALICE_CHECK(norm_w == nullptr || (norm_eps > 0.f && (norm_heads || inv_rms != nullptr)), "qkv_prepare: the norm needs a positive eps, and over the whole projection its workspace");
+  ALICE_CHECK(norm_w == nullptr || !norm_heads || (d <= 256 && vcos == nullptr), "qkv_prepare: the norm a head takes heads of up to 256 and values as they are");
   ALICE_CHECK(rows_dtype == DT_F32 || rows_dtype == out_dtype, "qkv_prepare: rows are float32 or in the outputs' dtype");
   ALICE_CHECK(T >= 0 && nH >= 1 && nKV >= 0 && d >= 1 && dv >= 1, "qkv_prepare: bad sizes T=%d nH=%d nKV=%d d=%d dv=%d", T, nH, nKV, d, dv);
   ALICE_CHECK(rotary_dim >= 0 && rotary_dim <= d && rotary_dim % 2 == 0, "qkv_prepare: rotated width %d must be even and at most %d", rotary_dim, d);
@@ -136,6 +215,19 @@ extern "C" int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width
   ALICE_CHECK(nH + 2 * nKV <= 65535, "qkv_prepare: too many heads for one launch");
   if (T == 0) return 0;
   dim3 grid(T, nH + (k_pool ? 2 * nKV : 0));
+  if (norm_w && norm_heads) {
+    const int n_heads = nH + (k_pool ? 2 * nKV : 0);
+    const dim3 g(T, ceil_div(n_heads, 4));
+#define GO(TI, TO)                                                                                                          \
+  qkv_prepare_heads_kernel<TI, TO><<<g, 256, 0, stream>>>((const TI*)rows, row_width, bias, norm_w, norm_eps, (TO*)q_out, (TO*)k_pool, (TO*)v_pool, \
+      cos_t, sin_t, rotary_dim, interleaved, positions, seq_of_token, block_table, bt_stride, nH, nKV, d, dv, page_size > 0 ? page_size : 1, n_pages, n_heads)
+    if (rows_dtype == DT_F32 && out_dtype == DT_F32) GO(float, float);
+    else if (rows_dtype == DT_F32) GO(float, bf16_t);
+    else GO(bf16_t, bf16_t);
+#undef GO
+    ALICE_LAUNCH_CHECK();
+    return 0;
+  }
   const int threads = 64;
   if (norm_w) {
     dim3 g0(T, k_pool ? 2 : 1);

@@ -18,7 +18,7 @@ from ..csrc import build as _build
 EPI_NONE, EPI_GEGLU, EPI_SOFTCAP = 0, 1, 2
 LAYOUT_ROW, LAYOUT_FRAG16 = 0, 1
 LINEAR_AUTO, LINEAR_GENERIC, LINEAR_SKINNY, LINEAR_MFMA, LINEAR_TILED_W16, LINEAR_TILED_W32 = 0, 1, 2, 3, 4, 5
-ABI_VERSION = 13
+ABI_VERSION = 14
 GATED_SILU = -1.0        # epi_param of EPI_GEGLU that picks silu(gate) * up
 UNARY_RELU2 = -1.0       # epi_param of EPI_SOFTCAP that picks the square of max(y, 0) instead of the capped form
 UNARY_SILU = -2.0        # likewise y * sigmoid(y)
@@ -41,6 +41,7 @@ def _declare(lib) -> None:
     sigs = {
         "alice_embed": [P, P, I, I, P, I, I, I, F, P],
         "alice_add_norm": [P, P, I, L, P, P, P, I, P, I, P, I, I, F, F, F, F, I, I, P],
+        "alice_add_dyntanh": [P, P, I, L, P, P, F, P, P, F, P, I, P, I, I, I, I, P],
         "alice_softcap": [P, L, F, I, P],
         "alice_add_branches": [P, I, P, P, P, P, I, P, P, P, I, I, I, I, P],
         "alice_linear": [P, I, P, I, I, P, I, I, I, I, I, F, I, I, I, I, I, P],
@@ -66,7 +67,7 @@ def _declare(lib) -> None:
         "alice_attention_split_supported": [I, I, I, I, I],
         "alice_attention_split_runs": [I],
         "alice_mix_heads": [P, P, P, I, F, P, I, I, I, I, I, I, P],
-        "alice_qkv_prepare": [P, I, I, P, P, P, P, I, P, P, I, I, P, P, P, P, P, I, I, I, I, I, I, I, I, P, F, P, P],
+        "alice_qkv_prepare": [P, I, I, P, P, P, P, I, P, P, I, I, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, F, P, P],
         "alice_short_conv": [P, I, I, I, I, P, P, P, P, I, P, P, P, I, I, P],
         "alice_ssm_prepare": [P, I, I, P, P, P, P, I, I, P],
         "alice_delta_prepare": [P, I, I, I, I, F, F, P, P, P, P, I, I, P, I, I, P],
@@ -78,7 +79,7 @@ def _declare(lib) -> None:
         "alice_expert_products": [P, P, P, P, P, P, P, P, I, I, I, I, I, F, P, P, I, P],
         "alice_expert_few_splits": [I],
         "alice_expert_few": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, F, F, P],
-        "alice_route_scored": [P, I, P, P, P, I, I, I, I, I, I, I, P],
+        "alice_route_scored": [P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, P],
         "alice_expert_combine": [P, I, P, I, P, P, I, P, I, I, P],
         "alice_lightning": [P, I, I, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
         "alice_add_rows": [P, P, P, I, I, P],
@@ -285,6 +286,37 @@ def add_norm(resid: torch.Tensor, branch: Optional[torch.Tensor], w_post: Option
           _opt(out, "out"), dtype_code(out.dtype if out is not None else torch.float32),
           _opt(rows, "rows"), T, H, float(eps_post), float(eps_pre), float(off_post), float(off_pre),
           int(full_precision), int(out_layout), _stream())
+
+
+def add_dyntanh(resid: torch.Tensor, branch: Optional[torch.Tensor], post, pre, out: Optional[torch.Tensor], *,
+                rows: Optional[torch.Tensor] = None, n_partials: int = 1, full_precision: bool,
+                out_layout: int = LAYOUT_ROW) -> None:
+    """resid += post(sum of branch partials); out = pre(resid), post and pre each (factor a, weight, bias) of a norm that acts
+    element by element, tanh(a v) * weight + bias (float32 [H]), or None: the sum, or the stream, as it is.  `rows`: only
+    these rows are normed into `out` (no branch).  out_layout: as add_norm's."""
+    if resid.dim() != 2:
+        raise HipLibraryError("resid must be [T, H]")
+    Tres, H = resid.shape
+    _dev(resid, "resid", torch.float32)
+    T = Tres if rows is None else rows.numel()
+    if branch is not None:
+        _dev(branch, "branch", torch.float32, (n_partials, Tres, H) if n_partials > 1 else (Tres, H))
+    elif n_partials != 1 or post is not None:
+        raise HipLibraryError("partial sums and a norm behind them need a branch")
+    if pre is not None and out is None:
+        raise HipLibraryError("a norm of the stream needs an output")
+    args = []
+    for norm, nm in ((post, "post"), (pre, "pre")):
+        a, w, b = norm if norm is not None else (0.0, None, None)
+        args += [_opt(w, nm + " weight", torch.float32, (H,)), _opt(b, nm + " bias", torch.float32, (H,)), float(a)]
+    if out is not None and out_layout == LAYOUT_FRAG16:
+        _dev(out, "out", torch.bfloat16, (frag_rows(T) * H,))
+    elif out is not None:
+        _dev(out, "out", None, (T, H))
+    if rows is not None:
+        _dev(rows, "rows", torch.int32)
+    _call("alice_add_dyntanh", resid.data_ptr(), _opt(branch, "branch"), n_partials, Tres * H, *args, _opt(out, "out"),
+          dtype_code(out.dtype if out is not None else torch.float32), _opt(rows, "rows"), T, H, int(full_precision), int(out_layout), _stream())
 
 
 MAX_BRANCHES = 4
@@ -734,14 +766,15 @@ def qkv_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], q_out: torch.T
                 value_head_dim: int, max_position: int, cos: Optional[torch.Tensor] = None,
                 sin: Optional[torch.Tensor] = None, rotary_dim: int = 0, interleaved: bool = True,
                 value_cos: Optional[torch.Tensor] = None, value_sin: Optional[torch.Tensor] = None,
-                norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0) -> None:
+                norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0, norm_heads: bool = False) -> None:
     """From the rows [q | k | v | ...] of a fused projection (float32, or q_out's dtype): bias [>= q, k, v columns]
     added, q and k heads rotated over their first rotary_dim dimensions in pairs ((2i, 2i + 1) if interleaved, else
     (i, i + rotary_dim / 2)) from tables [positions, rotary_dim / 2], values turned over all their dimensions where
     value tables [positions, dv / 2] are given; q to q_out, k and v into the row-major pools at their positions.
     norm_weight: float32 [q columns + k columns (where a cache is written)]: after the bias and before the rotation, the q
     columns (all heads together) and the k columns are each divided by their root mean square over the whole projection
-    (norm_eps inside the root) and multiplied by this weight."""
+    (norm_eps inside the root) and multiplied by this weight.  norm_heads: float32 [2, head_dim] instead: every q head and
+    every k head by its own root mean square, times the first row (q) or the second (k)."""
     T = rows.shape[0]
     dt = q_out.dtype
     d, dv = head_dim, value_head_dim
@@ -780,16 +813,17 @@ def qkv_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], q_out: torch.T
     inv_rms = None
     if norm_weight is not None:
         n_norm = num_heads * d + (num_kv_heads * d if k_pool is not None else 0)
-        _dev(norm_weight, "norm_weight", torch.float32, (n_norm,))
+        _dev(norm_weight, "norm_weight", torch.float32, (2, d) if norm_heads else (n_norm,))
         if not norm_eps > 0:
-            raise HipLibraryError("the projection norm needs a positive eps")
-        inv_rms = torch.empty((T, 2), dtype=torch.float32, device=rows.device)
+            raise HipLibraryError("the norm of the projection needs a positive eps")
+        if not norm_heads:
+            inv_rms = torch.empty((T, 2), dtype=torch.float32, device=rows.device)
     _call("alice_qkv_prepare", rows.data_ptr(), dtype_code(rows.dtype), rows.shape[1], _opt(bias, "bias"), q_out.data_ptr(),
           _opt(k_pool, "k_pool"), _opt(v_pool, "v_pool"), dtype_code(dt), _opt(cos, "cos"), _opt(sin, "sin"),
           int(rotary_dim if cos is not None else 0), int(interleaved), _opt(value_cos, "value_cos"), _opt(value_sin, "value_sin"),
           positions.data_ptr(), _opt(seq_of_token, "seq_of_token"), _opt(block_table, "block_table"), bt_stride, T,
           num_heads, num_kv_heads if k_pool is not None else 0, d, dv, page_size, n_pages,
-          _opt(norm_weight, "norm_weight"), float(norm_eps), _opt(inv_rms, "inv_rms"), _stream())
+          _opt(norm_weight, "norm_weight"), int(norm_heads), float(norm_eps), _opt(inv_rms, "inv_rms"), _stream())
 
 
 def add_rows(x: torch.Tensor, rows: Optional[torch.Tensor], vector: Optional[torch.Tensor]) -> None:
@@ -1220,21 +1254,25 @@ def route_topk(logits: torch.Tensor, bias: Optional[torch.Tensor], weights: torc
 
 
 def route_scored(logits: torch.Tensor, correction: Optional[torch.Tensor], weights: torch.Tensor, side: torch.Tensor, *,
-                 identity: int, top: int, groups: int = 1, keep: int = 1, has_shared: bool = False) -> None:
-    """A router whose scores are a softmax over all n = experts + identity columns of logits (float32 [T, >= n]).  The
-    choice is score + correction (float32 [n]); of `groups` equal runs of neighbours the `keep` with the largest choice
-    stay, and of those the `top` largest choices serve the token, weighted by their scores divided by the scores' sum.
+                 identity: int, top: int, groups: int = 1, keep: int = 1, has_shared: bool = False, shared_gate: bool = True,
+                 sigmoid: bool = False, group_best: int = 1, weight_scale: float = 1.0) -> None:
+    """A router whose scores are a softmax over all n = experts + identity columns of logits (float32 [T, >= n]), or with
+    `sigmoid` the sigmoid of each.  The choice is score + correction (float32 [n]); of `groups` equal runs of neighbours the
+    `keep` with the largest choice (group_best 1) or the largest sum of their two largest choices (group_best 2) stay, and of
+    those the `top` largest choices serve the token, weighted by weight_scale times their scores divided by the scores' sum.
     weights (float32 [T, experts]): zero where not chosen; side (float32 [T, 2]): the identity outputs' weight together,
-    and with has_shared sigmoid(logits[:, n])."""
+    and with has_shared the shared expert's factor, sigmoid(logits[:, n]) or without shared_gate 1."""
     T, E = weights.shape
     n = E + int(identity)
     _dev(logits, "logits", torch.float32)
-    if logits.dim() != 2 or logits.shape[0] != T or logits.shape[1] < n + int(bool(has_shared)):
-        raise HipLibraryError(f"logits must be [{T}, >= {n + int(bool(has_shared))}], found {tuple(logits.shape)}")
+    shared_mode = 0 if not has_shared else 1 if shared_gate else 2
+    if logits.dim() != 2 or logits.shape[0] != T or logits.shape[1] < n + int(shared_mode == 1):
+        raise HipLibraryError(f"logits must be [{T}, >= {n + int(shared_mode == 1)}], found {tuple(logits.shape)}")
     _dev(weights, "weights", torch.float32)
     _dev(side, "side", torch.float32, (T, 2))
     _call("alice_route_scored", logits.data_ptr(), logits.shape[1], _opt(correction, "correction", torch.float32, (n,)),
-          weights.data_ptr(), side.data_ptr(), T, E, int(identity), int(top), int(groups), int(keep), int(bool(has_shared)), _stream())
+          weights.data_ptr(), side.data_ptr(), T, E, int(identity), int(top), int(groups), int(keep), shared_mode,
+          int(bool(sigmoid)), int(group_best), float(weight_scale), _stream())
 
 
 def _partial_rows(t: Optional[torch.Tensor], name: str, T: int, W: int) -> int:

@@ -25,7 +25,8 @@ until the bias is added and the rotation done):
                   one more than the sum of the exponentials)
   qk_norm         "projection": q (all heads together) and k (likewise) are each divided by their root mean square over
                   the whole projection (qk_norm_eps inside the root) and multiplied by a weight of that length ("q_norm",
-                  "k_norm"), after the bias and before the rotation
+                  "k_norm"), after the bias and before the rotation.  "head": every q head and every k head by its own root
+                  mean square, times a weight of the head's size that the heads share
   output_bias     the output matrix has a bias ("o_bias")
   own_keys        False: the mixer has no k and v matrices (nor their biases and norm); it reads the keys and values that
                   another run of the schedule cached and brings its own queries, gate and output matrix
@@ -92,8 +93,10 @@ class Attention(Part):
         self.bias, self.chunk, self.keep_first = bool(bias), chunk, int(keep_first)
         if sink not in (False, True, None, "zero"):
             raise ValueError(f"attention: sink '{sink}' is not known (False, True or 'zero')")
-        if qk_norm not in (None, "projection"):
-            raise ValueError(f"attention: qk_norm '{qk_norm}' is not known (None or 'projection')")
+        if qk_norm not in (None, "projection", "head"):
+            raise ValueError(f"attention: qk_norm '{qk_norm}' is not known (None, 'projection' or 'head')")
+        if qk_norm == "head" and getattr(positions.get(position), "value_cos", None) is not None:
+            raise ValueError("attention: qk_norm 'head' takes values as they are, not turned by their position")
         self.has_sink, self.has_talk, self.output_scale = bool(sink), bool(talk), float(output_scale)
         self.zero_sink = sink == "zero"
         self.qk_norm, self.qk_norm_eps = qk_norm, float(qk_norm_eps)
@@ -146,9 +149,10 @@ class Attention(Part):
                 specs[n["k"] + ".b"] = ParamSpec((self.kv_dim,), init_std=0.1)
                 specs[n["v"] + ".b"] = ParamSpec((self.v_dim,), init_std=0.1)
         if self.qk_norm:
-            specs[n["q_norm"]] = ParamSpec((self.q_dim,), init_std=0.3)
+            head = self.qk_norm == "head"                   # (a head's weight is shared by the heads)
+            specs[n["q_norm"]] = ParamSpec((self.d,), init_std=0.1, init_mean=1.0) if head else ParamSpec((self.q_dim,), init_std=0.3)
             if self.own_keys:
-                specs[n["k_norm"]] = ParamSpec((self.kv_dim,), init_std=0.3)
+                specs[n["k_norm"]] = ParamSpec((self.d,), init_std=0.1, init_mean=1.0) if head else ParamSpec((self.kv_dim,), init_std=0.3)
         if self.output_bias:
             specs[n["o_bias"]] = ParamSpec((self.H,), init_std=0.1)
         if self.has_sink and not self.zero_sink:
@@ -194,8 +198,9 @@ class Attention(Part):
         if self.bias:
             self.qkv_bias = torch.cat([self._bias_parts.pop(self.names[c] + ".b").float() for c in self._mats if c != "g"]).contiguous()
         if self.qk_norm:
-            self.qk_norm_w = torch.cat([self._norm_parts.pop(self.names[c]).float()
-                                        for c in (("q_norm", "k_norm") if self.own_keys else ("q_norm",))]).contiguous()
+            parts = [self._norm_parts.pop(self.names[c]).float() for c in (("q_norm", "k_norm") if self.own_keys else ("q_norm",))]
+            # a head's norm: one row for the q heads, one for the k heads (a mixer without keys of its own never reads the second)
+            self.qk_norm_w = (torch.stack([parts[0], parts[-1]]) if self.qk_norm == "head" else torch.cat(parts)).contiguous()
         if self.zero_sink:
             self.sink = torch.zeros(self.nH, dtype=torch.float32, device=w.device)
         if self.pair_order:
@@ -266,7 +271,7 @@ class Attention(Part):
         if write and not self.own_keys:
             raise RuntimeError("attention: a mixer without keys of its own reads the cache of another run of the schedule")
         norm_w = self.qk_norm_w
-        if norm_w is not None and self.own_keys and not write:
+        if norm_w is not None and self.qk_norm == "projection" and self.own_keys and not write:
             norm_w = norm_w[:self.q_dim]                      # the keys are another run's: only the queries are normed here
         ops.qkv_prepare(rows, self.qkv_bias, q, cache.k if write else None, cache.v if write else None, ctx.positions,
                         ctx.seq_of_token if write else None, cache.block_table if write else None,
@@ -274,7 +279,7 @@ class Attention(Part):
                         max_position=ctx.max_position, cos=getattr(pos, "cos", None), sin=getattr(pos, "sin", None),
                         rotary_dim=getattr(pos, "rotary_dim", 0), interleaved=getattr(pos, "interleaved", True),
                         value_cos=getattr(pos, "value_cos", None), value_sin=getattr(pos, "value_sin", None),
-                        norm_weight=norm_w, norm_eps=self.qk_norm_eps)
+                        norm_weight=norm_w, norm_eps=self.qk_norm_eps, norm_heads=self.qk_norm == "head")
         gate = None
         if self.n_gate:
             g0 = self.q_dim + self.kv_dim + self.v_dim

@@ -85,12 +85,13 @@ class FragmentActs:
 
 @dataclass(frozen=True)
 class ParamSpec:
-    """A tensor a part wants: its shape, the standard deviation of its random initialisation, and
+    """A tensor a part wants: its shape, the standard deviation (and mean) of its random initialisation, and
     whether it is a floating-point weight (kept bfloat16 or float32 as stored) or an integer table
     (kept int32)."""
     shape: Tuple[int, ...]
     init_std: float = 0.02
     integer: bool = False
+    init_mean: float = 0.0
 
 
 class Part:

@@ -21,14 +21,15 @@ class Embedding(Part):
     graph_safe = True
 
     def __init__(self, precision: Precision, *, vocab_size: int, dim: int, scale: float = 1.0,
-                 tensor_name: str = "weight"):
+                 tensor_name: str = "weight", init_std: float = 0.02):
         self.tensor_name = tensor_name
         self.precision = precision
         self.V, self.dim, self.scale = vocab_size, dim, float(scale)
+        self.init_std = float(init_std)                     # of random weights: a design that norms nothing by its size wants rows of order one
         self.table = Linear(dim, vocab_size, precision)     # stored as the head reads it
 
     def param_specs(self) -> Dict[str, ParamSpec]:
-        return {self.tensor_name: ParamSpec((self.V, self.dim))}
+        return {self.tensor_name: ParamSpec((self.V, self.dim), init_std=self.init_std)}
 
     def assign(self, name: str, tensor: torch.Tensor) -> None:
         if name != self.tensor_name:

@@ -17,12 +17,16 @@ Variants, by constructor arguments:
                     output) is added for the choice only; the weights are the chosen scores divided by their sum (+ 1e-20).
                     The outputs may form `groups` = (count, keep): equal runs of neighbours of which only the `keep` with the
                     largest choice in them can serve the token.  No router bias.
+  `scoring="sigmoid"`  the same with the sigmoid of each router output as its score.
+  `group_best=2`    a group counts by the sum of the two largest choices in it instead of the largest one.
+  `weight_scale`    a constant factor of the chosen experts' weights.
   `identity=Z`      the last Z router outputs (behind the experts) are experts without matrices that give the token's own
                     input back (with scoring "all").
   `shared`          a further feed-forward of the same gated form, with sizes and constants of its own ("shared.gate" and so
-                    on), that serves every token, times sigmoid(s . h) ("shared.sg"; with scoring "all").
+                    on), that serves every token, times sigmoid(s . h) ("shared.sg"; with scoring "all" or "sigmoid"), or, with
+                    `shared_gate=False`, as it is.
   `activation="swish_limited"` with `limit`: the experts' bounded gated form.
-The shared expert's gate is one more row of the router's matrix, and its output and the identity experts' are added in
+The shared expert's gate, where it has one, is one more row of the router's matrix, and its output and the identity experts' are added in
 the kernel that adds up a token's experts.
 """
 from __future__ import annotations
@@ -50,15 +54,18 @@ class ExpertMLP(Part):
 
     def __init__(self, precision: Precision, *, hidden_size: int, intermediate_size: int, experts: int, top: int,
                  activation: str = "silu", limit: Optional[float] = None, router_bias: bool = True, scoring: str = "chosen",
-                 identity: int = 0, groups: Optional[Tuple[int, int]] = None, shared: Optional[Mapping] = None):
+                 identity: int = 0, groups: Optional[Tuple[int, int]] = None, shared: Optional[Mapping] = None,
+                 group_best: int = 1, weight_scale: float = 1.0, shared_gate: bool = True):
         if activation not in _GATED:
             raise ValueError(f"expert_mlp has no kernel for activation '{activation}'; available: {sorted(_GATED)}")
         if (activation == "swish_limited") != (limit is not None) or (limit is not None and not limit > 0):
             raise ValueError("expert_mlp: 'swish_limited' takes a positive limit, and only it does")
-        if scoring not in ("chosen", "all"):
-            raise ValueError(f"expert_mlp: scoring '{scoring}' is not known; available: 'chosen', 'all'")
-        if scoring == "chosen" and (identity or groups or shared):
-            raise ValueError("expert_mlp: identity experts, groups and a shared expert come with scoring 'all'")
+        if scoring not in ("chosen", "all", "sigmoid"):
+            raise ValueError(f"expert_mlp: scoring '{scoring}' is not known; available: 'chosen', 'all', 'sigmoid'")
+        if scoring == "chosen" and (identity or groups or shared or weight_scale != 1.0):
+            raise ValueError("expert_mlp: identity experts, groups, a shared expert and a factor of the weights come with scoring 'all' or 'sigmoid'")
+        if group_best not in (1, 2) or not weight_scale > 0:
+            raise ValueError(f"expert_mlp: group_best is 1 or 2 and weight_scale positive, found {group_best} and {weight_scale}")
         outputs = int(experts) + int(identity)
         if experts < 1 or identity < 0 or not 1 <= top <= outputs <= ops.ROUTER_MAX_EXPERTS:
             raise ValueError(f"expert_mlp: 1 <= top <= experts <= {ops.ROUTER_MAX_EXPERTS}, found top {top} of {outputs}")
@@ -67,12 +74,14 @@ class ExpertMLP(Part):
             raise ValueError(f"expert_mlp: {count} groups must divide {outputs} outputs, and the {keep} kept ones hold at least {top}")
         self.precision = precision
         self.H, self.F, self.E, self.top = hidden_size, int(intermediate_size), int(experts), int(top)
-        self.identity, self.groups, self.scored = int(identity), (int(count), int(keep)), scoring == "all"
+        self.identity, self.groups, self.scored = int(identity), (int(count), int(keep)), scoring != "chosen"
+        self.sigmoid, self.group_best, self.weight_scale = scoring == "sigmoid", int(group_best), float(weight_scale)
         self.outputs = outputs
         self.router_bias = bool(router_bias) and not self.scored
         self.shared = None if shared is None else GatedMLP(precision, hidden_size=hidden_size, tensor_names={
             "gate": "gate", "up": "up", "down": "down"}, **shared)
-        self.router = Linear(hidden_size, outputs + (self.shared is not None), precision)      # the last row: the shared expert's gate
+        self.shared_gate = bool(shared_gate) and self.shared is not None
+        self.router = Linear(hidden_size, outputs + self.shared_gate, precision)               # the last row: the shared expert's gate
         self.gate_up = Linear(hidden_size, self.E * self.F, precision, epilogue=ops.EPI_GEGLU,
                               epi_param=float(limit) if limit is not None else _GATED[activation])
         self.down = Linear(self.E * self.F, hidden_size, precision)
@@ -89,10 +98,11 @@ class ExpertMLP(Part):
         if self.router_bias:
             specs["router.b"] = ParamSpec((self.outputs,), init_std=0.1)
         if self.scored:
-            specs["correction"] = ParamSpec((self.outputs,), init_std=0.1)
+            specs["correction"] = ParamSpec((self.outputs,), init_std=0.02 if self.sigmoid else 0.1)
         if self.shared is not None:
             specs.update({f"shared.{n}": spec for n, spec in self.shared.param_specs().items()})
-            specs["shared.sg"] = ParamSpec((1, self.H), init_std=0.1)
+            if self.shared_gate:
+                specs["shared.sg"] = ParamSpec((1, self.H), init_std=0.1)
         return specs
 
     def assign(self, name: str, tensor: torch.Tensor) -> None:
@@ -109,6 +119,7 @@ class ExpertMLP(Part):
         router = self.precision.matrix(self._parts.pop("router"))
         if self.shared is not None:
             self.shared.finalize()
+        if self.shared_gate:
             sg = self.precision.matrix(self._parts.pop("shared.sg"))
             if sg.dtype != router.dtype:
                 router, sg = router.float(), sg.float()
@@ -138,7 +149,8 @@ class ExpertMLP(Part):
         if self.scored:
             side = torch.empty((T, 2), dtype=torch.float32, device=dev)
             ops.route_scored(logits, self.bias, weights, side, identity=self.identity, top=self.top, groups=self.groups[0],
-                             keep=self.groups[1], has_shared=self.shared is not None)
+                             keep=self.groups[1], has_shared=self.shared is not None, shared_gate=self.shared_gate, sigmoid=self.sigmoid,
+                             group_best=self.group_best, weight_scale=self.weight_scale)
         else:
             ops.route_topk(logits, self.bias, weights, self.top)
         side_used = side if self.identity or self.shared is not None else None

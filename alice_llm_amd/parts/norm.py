@@ -1,5 +1,6 @@
 """Norms.  RMSNorm: y = x / sqrt(mean(x^2) + eps) * (weight_offset + w), all in 32-bit.  LayerNorm:
-y = (x - m) / sqrt(mean((x - m)^2) + eps) * w + b with m = mean(x), likewise.
+y = (x - m) / sqrt(mean((x - m)^2) + eps) * w + b with m = mean(x), likewise.  DynamicTanh: y = tanh(a x) * w + b, element
+by element, with one stored number a.
 
 The reference multiplies by the stored weight (llama3.rs:5244-5256), its files holding 1 + w; a
 safetensors file holds w, so Gemma 2 passes weight_offset = 1.  The offset, eps and the width are
@@ -98,4 +99,45 @@ class LayerNorm(Part):
         out = torch.empty((n, self.dim), dtype=out_dtype, device=x.device)
         ops.add_norm(x, None, None, self.weight, out, eps_pre=self.eps, b_pre=self.bias, rows=rows,
                      full_precision=self.precision.full)
+        return out
+
+
+@NORMS.register("dynamic_tanh")
+class DynamicTanh(Part):
+    """y = tanh(alpha x) * w + b: no mean, no variance, every element by itself.  Weight and bias are kept in 32-bit, the one
+    number alpha (`alpha_name`, a tensor without dimensions) is read to the host once, at load.  It rides on the residual
+    add behind a part and ahead of one alike (`pointwise`)."""
+    graph_safe = True
+
+    def __init__(self, precision: Precision, *, dim: int, tensor_name: str = "weight", bias_name: str = "bias", alpha_name: str = "alpha"):
+        self.precision = precision
+        self.dim = dim
+        self.tensor_name, self.bias_name, self.alpha_name = tensor_name, bias_name, alpha_name
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+        self.alpha: Optional[float] = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return {self.tensor_name: ParamSpec((self.dim,), init_std=0.1, init_mean=1.0), self.bias_name: ParamSpec((self.dim,), init_std=0.02),
+                self.alpha_name: ParamSpec((), init_std=0.05, init_mean=0.5)}
+
+    def assign(self, name: str, tensor: torch.Tensor) -> None:
+        if name == self.tensor_name:
+            self.weight = tensor.float().contiguous()
+        elif name == self.bias_name:
+            self.bias = tensor.float().contiguous()
+        elif name == self.alpha_name:
+            self.alpha = float(tensor)
+        else:
+            raise KeyError(name)
+
+    def pointwise(self) -> Tuple[float, torch.Tensor, torch.Tensor]:
+        """(alpha, weight, bias) for the residual add whose norms act element by element."""
+        return self.alpha, self.weight, self.bias
+
+    def forward(self, x: torch.Tensor, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """x: float32 [T, dim]; with `rows` only these rows are normed (in their order)."""
+        n = x.shape[0] if rows is None else rows.numel()
+        out = torch.empty((n, self.dim), dtype=out_dtype, device=x.device)
+        ops.add_dyntanh(x, None, None, self.pointwise(), out, rows=rows, full_precision=self.precision.full)
         return out

@@ -92,7 +92,11 @@ class RotaryPairs(Part):
     `scaling` (factor s, original length L, fast, slow) stretches the frequencies of the q and k rotation for
     contexts beyond L, the slow ones most: with D(t) = R ln(L / (2 pi t)) / (2 ln theta), lo = max(floor D(fast), 0),
     hi = min(ceil D(slow), R - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), the frequency becomes
-    f_i / s * r_i + f_i (1 - r_i), and cos and sin are multiplied by 0.1 ln(s) + 1 (which the tables hold)."""
+    f_i / s * r_i + f_i (1 - r_i), and cos and sin are multiplied by 0.1 ln(s) + 1 (which the tables hold).
+
+    `scaling` with (factor s, low, high, original length L) instead stretches by how often a frequency turns within L
+    positions, t_i = L f_i / (2 pi): f_i stays where t_i > high, becomes f_i / s where t_i < low, and between the two
+    m f_i + (1 - m) f_i / s with m = (t_i - low) / (high - low); cos and sin keep their size."""
     graph_safe = True
 
     def __init__(self, precision: Precision, device, *, dim: int, theta: float, max_positions: int,
@@ -106,9 +110,13 @@ class RotaryPairs(Part):
             raise ValueError(f"turned values need an even size, found {value_dim}")
         self.theta, self.max_positions = float(theta), max_positions
         self.value_dim, self.interleaved = value_dim, bool(interleaved)
-        self.scaling = None if not scaling else {k: float(scaling[k]) for k in ("factor", "original", "fast", "slow")}
+        banded = bool(scaling) and "low" in scaling
+        keys = ("factor", "original", "low", "high") if banded else ("factor", "original", "fast", "slow")
+        self.scaling = None if not scaling else {k: float(scaling[k]) for k in keys}
         if self.scaling is not None and min(self.scaling.values()) <= 0:
-            raise ValueError(f"stretched frequencies need positive factor, original, fast and slow, found {self.scaling}")
+            raise ValueError(f"stretched frequencies need positive {', '.join(keys)}, found {self.scaling}")
+        if banded and not self.scaling["low"] < self.scaling["high"]:
+            raise ValueError(f"frequencies stretched by bands need low below high, found {self.scaling}")
         self.cos, self.sin = self._tables(self.rotary_dim, device, self.scaling) if self.rotary_dim else (None, None)
         self.value_cos, self.value_sin = self._tables(value_dim, device) if value_dim else (None, None)
 
@@ -119,6 +127,10 @@ class RotaryPairs(Part):
         if scaling is None:
             return f, 1.0
         s, L = scaling["factor"], scaling["original"]
+        if "low" in scaling:
+            turns = L * f / (2.0 * math.pi)
+            m = torch.clamp((turns - scaling["low"]) / (scaling["high"] - scaling["low"]), 0.0, 1.0)
+            return m * f + (1.0 - m) * f / s, 1.0
         at = lambda t: width * math.log(L / (2.0 * math.pi * t)) / (2.0 * math.log(self.theta))
         lo = max(math.floor(at(scaling["fast"])), 0)
         hi = min(math.ceil(at(scaling["slow"])), width - 1)

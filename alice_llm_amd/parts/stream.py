@@ -3,7 +3,8 @@
 Blocks push a branch output (with the norm that applies to it before the add, if any) and ask
 for the normed stream that feeds their next part.  The add of the pending branch and the next
 norm run as one kernel when both norms can be fused; otherwise the same result is computed in
-separate kernels.  The stream itself is only ever added to, in 32-bit
+separate kernels.  Norms that act element by element (`pointwise`, on either side of the add) have such a kernel of
+their own.  The stream itself is only ever added to, in 32-bit
 (llama3.rs:14468-14470, 14555-14557).
 """
 from __future__ import annotations
@@ -27,6 +28,11 @@ def _fused_pre(norm):
         return norm.fused_pre()
     f = norm.fused() if hasattr(norm, "fused") else None
     return None if f is None else (*f, None)
+
+
+def _pointwise(norm):
+    """(alpha, weight, bias) of a norm that acts element by element, else None."""
+    return norm.pointwise() if norm is not None and hasattr(norm, "pointwise") else None
 
 
 class ResidualStream:
@@ -83,7 +89,9 @@ class ResidualStream:
         n, b = self._partials()
         post = self._post
         fused = post.fused() if post is not None and hasattr(post, "fused") else None
-        if post is None or fused is not None:
+        if _pointwise(post) is not None:
+            self._add_pointwise(None, None)
+        elif post is None or fused is not None:
             w, eps, off = fused if fused is not None else (None, 0.0, 0.0)
             ops.add_norm(self.x, b, w, None, None, eps_post=eps, off_post=off, n_partials=n,
                          full_precision=self.precision.full)
@@ -92,6 +100,14 @@ class ResidualStream:
                 b = b.sum(dim=0)
             normed = post.forward(b.contiguous(), torch.float32)
             ops.add_norm(self.x, normed, None, None, None, full_precision=self.precision.full)
+        self._branch = None
+        self._post = None
+
+    def _add_pointwise(self, norm, out, out_layout: int = ops.LAYOUT_ROW) -> None:
+        """The pending add (none, or with no norm behind the branch or one that acts element by element) and norm(x), likewise."""
+        n, b = self._partials() if self._branch is not None else (1, None)
+        ops.add_dyntanh(self.x, b, _pointwise(self._post) if b is not None else None, _pointwise(norm), out.data if out_layout else out,
+                        n_partials=n, full_precision=self.precision.full, out_layout=out_layout)
         self._branch = None
         self._post = None
 
@@ -106,6 +122,13 @@ class ResidualStream:
                 self._flush_many(out)
                 return out
             self._flush_many()
+        if _pointwise(norm) is not None:
+            if self._branch is not None and self._post is not None and _pointwise(self._post) is None:
+                self.flush()
+            frag = fragments and out_dtype == torch.bfloat16 and FragmentActs.possible(self.precision, T, H)
+            out = FragmentActs.empty(T, H, self.x.device) if frag else torch.empty((T, H), dtype=out_dtype, device=self.x.device)
+            self._add_pointwise(norm, out, ops.LAYOUT_FRAG16 if frag else ops.LAYOUT_ROW)
+            return out
         pre = _fused_pre(norm)
         if fragments and pre is not None and out_dtype == torch.bfloat16 and FragmentActs.possible(self.precision, T, H):
             post = self._post
@@ -144,6 +167,11 @@ class ResidualStream:
         """norm(x[rows]) after all pending adds: what the output head reads."""
         self.flush()
         out_dtype = out_dtype or self.precision.act
+        point = _pointwise(norm)
+        if fragments and point is not None and out_dtype == torch.bfloat16 and FragmentActs.possible(self.precision, rows.numel(), self.x.shape[1]):
+            out = FragmentActs.empty(rows.numel(), self.x.shape[1], self.x.device)
+            ops.add_dyntanh(self.x, None, None, point, out.data, rows=rows, full_precision=self.precision.full, out_layout=ops.LAYOUT_FRAG16)
+            return out
         pre = _fused_pre(norm)
         if fragments and pre is not None and out_dtype == torch.bfloat16 and \
                 FragmentActs.possible(self.precision, rows.numel(), self.x.shape[1]):

@@ -111,7 +111,7 @@ def load_weights(model, folder: str, strict: bool = True) -> List[str]:
 # --------------------------------------------------------------------------- random weights
 
 def random_tensors(specs: Dict[str, ParamSpec], seed: int, dtype: torch.dtype, device="cpu") -> Iterator[Tuple[str, torch.Tensor]]:
-    """Tensors in the order of `specs` from one generator seeded with `seed`: N(0, init_std) drawn in
+    """Tensors in the order of `specs` from one generator seeded with `seed`: N(init_mean, init_std) drawn in
     float32 (on the host unless a device is given, whose generator draws other values), then cast to
     `dtype`; integer tables are zeros."""
     gen = torch.Generator(device=device)
@@ -121,7 +121,7 @@ def random_tensors(specs: Dict[str, ParamSpec], seed: int, dtype: torch.dtype, d
             yield name, torch.zeros(spec.shape, dtype=torch.int32, device=device)
         else:
             t = torch.empty(spec.shape, dtype=torch.float32, device=device)
-            t.normal_(0.0, spec.init_std, generator=gen)
+            t.normal_(spec.init_mean, spec.init_std, generator=gen)
             yield name, t.to(dtype)
 
 
