@@ -4,7 +4,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 
-#define ALICE_ABI_VERSION 14
+#define ALICE_ABI_VERSION 15
 
 #define ALICE_EPI_NONE 0
 #define ALICE_EPI_GEGLU 1     // W = [gate; up] stacked; epi_param 0: y = gelu_tanh(gate x) * (up x); epi_param = limit > 0:
@@ -113,12 +113,14 @@ int alice_attention_generic(const void* q, int dtype, const void* k_pool, const 
                             int dv, const void* gate, int gate_stride, hipStream_t stream);
 
 // bfloat16 attention on the matrix cores over a cache in the fragment layout (kv_layout 1 of
-// alice_rope_cache_write): prompts, and single tokens with the keys split over `splits` blocks.
+// alice_rope_cache_write): prompts, and single tokens with the keys split over `splits` blocks.  sink (float32 [nH] or null):
+// exp(sink[h]) joins the softmax's denominator of head h.
 int alice_attention_mfma_supported(int d);
 int alice_attention_prefill(const void* q, const void* k_pool, const void* v_pool, void* out,
                             const int* cu_seqlens, const int* context_lens, const int* block_table,
                             int bt_stride, int B, int max_new, int nH, int nKV, int d, int page_size,
-                            float scale, float softcap, int window, int variant, int out_layout, hipStream_t stream);
+                            float scale, float softcap, int window, int variant, int out_layout, const float* sink,
+                            hipStream_t stream);
 // out[t, h, :] *= sigmoid(gate[t * gate_stride + h]) in place on a bfloat16 attention output in either layout.
 // alice_attention_generic with further parameters of the mask and the softmax (0 / null: off): gate: float32 rows,
 // gate_mode 1: a number a head, 2: a number an output element ([T, nH dv]); out_scale: a constant factor of the
@@ -164,10 +166,11 @@ int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width, const flo
                       int interleaved, const float* vcos, const float* vsin, const int* positions,
                       const int* seq_of_token, const int* block_table, int bt_stride, int T, int nH, int nKV,
                       int d, int dv, int page_size, int n_pages, const float* norm_w, int norm_heads, float norm_eps,
-                      float* inv_rms, hipStream_t stream);
+                      float* inv_rms, int kv_layout, hipStream_t stream);
 // (norm_w: float32 [nH d + nKV d] or null: the q columns and the k columns are each RMS-normed over the whole
 // projection, after the bias and before the rotation; inv_rms: float32 [T, 2] workspace.  With norm_heads: float32 [2, d],
-// every q head and every k head by its own root mean square times the first or second row; no workspace.)
+// every q head and every k head by its own root mean square times the first or second row; no workspace; kv_layout 1: the
+// pools are in the fragment layout.)
 // x[t, c] += a[t, c] + v[c] (either may be null)
 int alice_add_rows(float* x, const float* a, const float* v, int T, int W, hipStream_t stream);
 // Gated linear attention over a step's tokens, see gla.hip.
@@ -285,7 +288,7 @@ long alice_attention_decode_workspace(int B, int nH, int d, int splits);
 int alice_attention_decode(const void* q, const void* k_pool, const void* v_pool, void* out, float* parts,
                            const int* context_lens, const int* block_table, int bt_stride, int B, int nH,
                            int nKV, int d, int page_size, float scale, float softcap, int window, int splits,
-                           int out_layout, const void* gate, int gate_stride, hipStream_t stream);
+                           int out_layout, const void* gate, int gate_stride, const float* sink, hipStream_t stream);
 
 // The output projection straight from the parts of alice_attention_decode (at most 16 sequences and 16 splits, weights in the
 // fragment layout, [N, nH d]): y[slices][M][N] float32 partial sums, slices = alice_linear_parts_split(...), which

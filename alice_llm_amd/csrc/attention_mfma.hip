@@ -5,7 +5,7 @@
 // Order of operations as in the reference (llama3.rs:5622-5688): dot product, times scale, softcap
 // cap * tanh(s / cap), mask to the keys max(0, pos + 1 - window) .. pos (llama3.rs:5444-5451),
 // softmax with a running maximum (llama3.rs:5568-5620), weighted sum of the values; the kv head of
-// query head h is h / (nH / nKV).
+// query head h is h / (nH / nKV).  A sink (one number a head, optional) is one more term of the softmax's denominator.
 //
 // Cache layout ("fragment" layout, written by rope_cache_write): a page holds 64 positions of one kv
 // head.  Keys:   [key tile t (4)][d tile (d/32)][lane 64][8]: lane g*16 + r holds K[16 t + r][32 dt + 8g ..+8].
@@ -77,6 +77,13 @@ struct Core {
 #pragma unroll
       for (int t = 0; t < 2 * DT; ++t) o[b][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
+  }
+  // A sink: one more term exp(v) of the column's denominator, without a key and a value.  The running softmax starts from
+  // it (maximum v, sum 1, output 0); where the keys of a column are split, in one of its parts only.  The four lanes of a
+  // column share its maximum and hold shares of its sum.
+  __device__ __forceinline__ void start_at_sink(int b, float v, int lane) {
+    m[b] = v * LOG2E;
+    l[b] = lane < 16 ? 1.f : 0.f;
   }
 
   // The fragments of one block of 32 keys: kpage/vpage point at the page of one kv head, kb is the block
@@ -262,7 +269,7 @@ __global__ __launch_bounds__(256, GH == 1 ? 2 : 1) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool,
     bf16_t* __restrict__ out, const int* __restrict__ cu_seqlens, const int* __restrict__ context_lens,
     const int* __restrict__ block_table, int bt_stride, int nH, int nKV, float scale, float cap, int window,
-    int out_layout) {
+    int out_layout, const float* __restrict__ sink) {
   constexpr int D = DT * 32;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int col = lane & 15, g = lane >> 4;
@@ -290,6 +297,7 @@ __global__ __launch_bounds__(256, GH == 1 ? 2 : 1) void attn_prefill_kernel(
     const int head = kvh * group + h0 + hh;
     const bool ok = tok_ok && (h0 + hh) < group;
     pos[hh] = ok ? my_pos : -1;
+    if (sink && ok) c.start_at_sink(hh, sink[head], lane);
     const bf16_t* qrow = q + ((size_t)(t_begin + (tok_ok ? my_tok : 0)) * nH + (ok ? head : kvh * group)) * D;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -353,7 +361,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_split_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool,
     bf16_t* __restrict__ out, const int* __restrict__ cu_seqlens, const int* __restrict__ context_lens,
     const int* __restrict__ block_table, int bt_stride, int nH, int nKV, float scale, float cap, int window,
-    int out_layout) {
+    int out_layout, const float* __restrict__ sink) {
   constexpr int D = DT * 32;
   __shared__ float sm[4][16], sl[4][16];
   extern __shared__ __align__(16) float so[];                // [3 waves][16 columns][D + 4]
@@ -379,6 +387,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_split_kernel(
 
   Core<DT, 1> c;
   c.init();
+  if (sink && wave == 0) c.start_at_sink(0, sink[head], lane);
   {
     const bf16_t* qrow = q + ((size_t)(t_begin + (tok_ok ? my_tok : 0)) * nH + head) * D;
 #pragma unroll
@@ -446,7 +455,7 @@ __global__ __launch_bounds__(64 * NW * KS, NW * KS == 4 ? 2 : 1) void attn_prefi
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool,
     bf16_t* __restrict__ out, const int* __restrict__ cu_seqlens, const int* __restrict__ context_lens,
     const int* __restrict__ block_table, int bt_stride, int nH, int nKV, float scale, float cap, int window, int HB,
-    int out_layout, int xcd_map) {
+    int out_layout, int xcd_map, const float* __restrict__ sink) {
   // KS = 2: two sets of NW waves, the second takes the later half of the block's keys (its own buffers in LDS);
   // at the end the first set adds the second's part to its own, each scaled to the common maximum.  Halves the
   // longest block's run when there are too few blocks to fill the chip.
@@ -502,6 +511,7 @@ __global__ __launch_bounds__(64 * NW * KS, NW * KS == 4 ? 2 : 1) void attn_prefi
 
   Core<DT, 1> c;
   c.init();
+  if (sink && set == 0 && hh < group) c.start_at_sink(0, sink[kvh * group + hh], lane);
   {
     const bf16_t* qrow = q + ((size_t)(t_begin + (tok_ok ? my_tok : 0)) * nH + kvh * group + (hh < group ? hh : 0)) * D;
 #pragma unroll
@@ -593,7 +603,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool,
     bf16_t* __restrict__ out, float* __restrict__ parts, const int* __restrict__ context_lens,
     const int* __restrict__ block_table, int bt_stride, int nH, int nKV, float scale, float cap, int window, int splits,
-    int out_layout) {
+    int out_layout, const float* __restrict__ sink) {
   constexpr int D = DT * 32;
   __shared__ float sm[4][16], sl[4][16];
   extern __shared__ __align__(16) float so[];            // [4 waves][group][D + 4]
@@ -616,6 +626,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   const ScoreConsts sc(scale, cap);
   const bool head_ok = col < group;
   int cpos[1] = {head_ok ? pos : -1};
+  if (sink && me == 0 && head_ok) c.start_at_sink(0, sink[kvh * group + col], lane);
   {
     const bf16_t* qrow = q + ((size_t)b * nH + kvh * group + (head_ok ? col : 0)) * D;
 #pragma unroll
@@ -758,7 +769,8 @@ extern "C" int alice_head_gate(void* out, int out_layout, const void* gate, int 
 extern "C" int alice_attention_prefill(const void* q, const void* k_pool, const void* v_pool, void* out,
                                        const int* cu_seqlens, const int* context_lens, const int* block_table,
                                        int bt_stride, int B, int max_new, int nH, int nKV, int d, int page_size,
-                                       float scale, float softcap, int window, int variant, int out_layout, hipStream_t stream) {
+                                       float scale, float softcap, int window, int variant, int out_layout, const float* sink,
+                                       hipStream_t stream) {
   ALICE_CHECK(alice_attention_mfma_supported(d), "attention (matrix cores): head_dim %d is not covered (64, 128 or 256)", d);
   ALICE_CHECK(out_layout == 0 || (out_layout == 1 && (nH * d) % 32 == 0), "attention: unknown output layout %d", out_layout);
   ALICE_CHECK(nKV >= 1 && nH % nKV == 0, "attention: bad head counts nH=%d nKV=%d", nH, nKV);
@@ -777,10 +789,10 @@ extern "C" int alice_attention_prefill(const void* q, const void* k_pool, const 
   do {                                                                                                                      \
     if (softcap > 0.f)                                                                                                      \
       attn_prefill_kernel<DT, GH, true><<<grid, 256, 0, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout);     \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout, sink);     \
     else                                                                                                                    \
       attn_prefill_kernel<DT, GH, false><<<grid, 256, 0, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout);     \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout, sink);     \
   } while (0)
 #define GOS(DT)                                                                                                             \
   do {                                                                                                                      \
@@ -788,10 +800,10 @@ extern "C" int alice_attention_prefill(const void* q, const void* k_pool, const 
     const size_t lds = (size_t)3 * 16 * (DT * 32 + 4) * sizeof(float);                                                      \
     if (softcap > 0.f)                                                                                                      \
       attn_prefill_split_kernel<DT, true><<<sgrid, 256, lds, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout);     \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout, sink);     \
     else                                                                                                                    \
       attn_prefill_split_kernel<DT, false><<<sgrid, 256, lds, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout);     \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, out_layout, sink);     \
   } while (0)
   // Few waves (one prompt of a few thousand tokens): split every tile's keys over four waves.  Many: whole
   // tiles per wave, two heads a wave where the group is even.
@@ -814,10 +826,10 @@ extern "C" int alice_attention_prefill(const void* q, const void* k_pool, const 
     }                                                                                                                       \
     if (softcap > 0.f)                                                                                                      \
       attn_prefill_shared_kernel<DT, true, NW, KS><<<lgrid, 64 * NW * KS, lds, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, hb, out_layout, xcd_map); \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, hb, out_layout, xcd_map, sink); \
     else                                                                                                                    \
       attn_prefill_shared_kernel<DT, false, NW, KS><<<lgrid, 64 * NW * KS, lds, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, \
-          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, hb, out_layout, xcd_map); \
+          (bf16_t*)out, cu_seqlens, context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, hb, out_layout, xcd_map, sink); \
   } while (0)
   // Which form (measured on Gemma 2 shapes): with many blocks, four waves sharing their keys; with fewer, eight
   // (half as many blocks, half the key traffic); with too few blocks to fill the chip, the keys of a block split
@@ -861,7 +873,7 @@ extern "C" long alice_attention_decode_workspace(int B, int nH, int d, int split
 extern "C" int alice_attention_decode(const void* q, const void* k_pool, const void* v_pool, void* out, float* parts,
                                       const int* context_lens, const int* block_table, int bt_stride, int B, int nH,
                                       int nKV, int d, int page_size, float scale, float softcap, int window, int splits,
-                                      int out_layout, const void* gate, int gate_stride, hipStream_t stream) {
+                                      int out_layout, const void* gate, int gate_stride, const float* sink, hipStream_t stream) {
   ALICE_CHECK(alice_attention_mfma_supported(d), "attention (matrix cores): head_dim %d is not covered (64, 128 or 256)", d);
   ALICE_CHECK(nKV >= 1 && nH % nKV == 0 && nH / nKV <= 16, "attention (decode): %d query heads per kv head are more than the 16 this kernel takes", nKV ? nH / nKV : 0);
   ALICE_CHECK(page_size == 64, "attention (matrix cores): pages must hold 64 positions, found %d", page_size);
@@ -888,7 +900,7 @@ extern "C" int alice_attention_decode(const void* q, const void* k_pool, const v
       }                                                                                                                     \
     }                                                                                                                       \
     kern<<<grid, 256, lds, stream>>>((const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool, (bf16_t*)out, parts,   \
-                                     context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, splits, out_layout); \
+                                     context_lens, block_table, bt_stride, nH, nKV, scale, softcap, window, splits, out_layout, sink); \
   } while (0)
 #define GO(DT)                          \
   do {                                  \

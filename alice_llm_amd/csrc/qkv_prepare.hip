@@ -13,7 +13,8 @@
 // mean square over the whole projection, eps inside the root, and multiplied by a weight of that length, after the
 // bias and before the rotation; projection_rms_kernel finds the two factors of every token first, in 32-bit.  With a norm a
 // head instead, every q head and every k head is divided by its own root mean square and multiplied by a weight of d numbers
-// that the q heads share (and one that the k heads share): qkv_prepare_heads_kernel, a wave a head, the head in registers.
+// that the q heads share (and one that the k heads share): qkv_prepare_heads_kernel, a wave a head, the head in registers; it
+// also writes pages in the matrix-core kernels' fragment order.
 #include "common.h"
 #include "alice_hip.h"
 #include "kv_layout.h"
@@ -106,80 +107,180 @@ __global__ void qkv_prepare_kernel(const TI* __restrict__ rows, int row_w, const
   }
 }
 
-// A wave per (token, head), four heads a block; a lane holds up to two pairs of the head (d <= 256): the rotation's pairs
-// first, then the unrotated dimensions two by two (of an odd number the last alone).  norm_w: [2, d], the q heads' weight and
-// the k heads'.
+// A wave takes one head of R consecutive tokens, four heads a block; a lane holds up to NP pairs of the head (d <= 128 NP): the
+// rotation's pairs first, then the unrotated dimensions two by two (of an odd number the last alone).  VEC: all pairs are
+// neighbours and go to and from memory as one.  norm_w: [2, d], the q heads' weight and the k heads'.
+// Values in the fragment layout: eight positions of one dimension are neighbours in memory (see kv_layout.h), so where a step
+// brings all eight, the wave of the first of them writes for all.
+struct HeadsArgs {
+  int row_w, R, interleaved, bt_stride, T, nH, nKV, d, dv, page_size, n_pages, n_heads, layout;
+  float eps;
+  const float *bias, *norm_w, *cos_t, *sin_t;
+  const int *positions, *seq_of_token, *block_table;
+};
+
+template <typename TI> __device__ __forceinline__ void load_pair(const TI* p, size_t i, float& x, float& y);
+template <> __device__ __forceinline__ void load_pair<float>(const float* p, size_t i, float& x, float& y) {
+  const float2 v = *reinterpret_cast<const float2*>(p + i);
+  x = v.x;
+  y = v.y;
+}
+template <> __device__ __forceinline__ void load_pair<bf16_t>(const bf16_t* p, size_t i, float& x, float& y) {
+  const uint32_t v = *reinterpret_cast<const uint32_t*>(p + i);
+  x = bf16_bits_to_f32(v & 0xffffu);
+  y = bf16_bits_to_f32(v >> 16);
+}
+__device__ __forceinline__ void store_pair(float* p, size_t i, float x, float y) { *reinterpret_cast<float2*>(p + i) = float2{x, y}; }
+__device__ __forceinline__ void store_pair(bf16_t* p, size_t i, float x, float y) { *reinterpret_cast<uint32_t*>(p + i) = pack_bf16x2(x, y); }
+
+template <typename TI>
+__device__ __forceinline__ float value_of(const TI* rows, const HeadsArgs& a, int t, size_t col) {
+  const float x = load_f32(rows, (size_t)t * a.row_w + col);
+  return a.bias ? x + a.bias[col] : x;
+}
+
+// One token's value head by one wave.
 template <typename TI, typename TO>
-__global__ __launch_bounds__(256) void qkv_prepare_heads_kernel(const TI* __restrict__ rows, int row_w, const float* __restrict__ bias,
-                                                                const float* __restrict__ norm_w, float eps,
-                                                                TO* __restrict__ q_out, TO* __restrict__ k_pool, TO* __restrict__ v_pool,
-                                                                const float* __restrict__ cos_t, const float* __restrict__ sin_t, int R,
-                                                                int interleaved, const int* __restrict__ positions,
-                                                                const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
-                                                                int bt_stride, int nH, int nKV, int d, int dv, int page_size, int n_pages,
-                                                                int n_heads) {
-  const int t = blockIdx.x, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (h >= n_heads) return;
-  const int pos = positions[t];
-  const TI* row = rows + (size_t)t * row_w;
-  int page = -1;
-  if (k_pool) {
-    page = block_table[(size_t)seq_of_token[t] * bt_stride + pos / page_size];
-    if (page < 0 || page >= n_pages) page = -1;
-  }
-  const int tp = pos % page_size;
-  if (h >= nH + nKV) {                                          // a value head: as it is
-    if (page < 0) return;
-    const int hv = h - nH - nKV;
-    const size_t col0 = (size_t)(nH + nKV) * d + (size_t)hv * dv;
-    TO* dst = v_pool + (((size_t)page * nKV + hv) * page_size + tp) * dv;
-    for (int e = lane; e < dv; e += 64) {
-      float x = load_f32(row, col0 + e);
-      if (bias) x += bias[col0 + e];
-      store_f32(dst, e, x);
-    }
+__device__ __forceinline__ void put_values(const TI* rows, TO* v_pool, const HeadsArgs& a, int t, int hv, int pos, int page, int lane) {
+  const size_t col0 = (size_t)(a.nH + a.nKV) * a.d + (size_t)hv * a.dv;
+  TO* dst = v_pool + ((size_t)page * a.nKV + hv) * a.page_size * a.dv;
+  const int tp = pos % a.page_size;
+  if (a.layout == 0) {
+    for (int e = lane; e < a.dv; e += 64) store_f32(dst, (size_t)tp * a.dv + e, value_of(rows, a, t, col0 + e));
     return;
   }
-  const bool is_q = h < nH;
-  const size_t col0 = (size_t)h * d;
-  const float* w = norm_w + (is_q ? 0 : d);
-  const int half = R >> 1, n_pairs = half + (d - R + 1) / 2;
-  int e0[2], e1[2];
-  bool on0[2], on1[2];
-  float x0[2], x1[2], w0[2], w1[2], cs[2], sn[2];
+  if constexpr (sizeof(TO) == 2) {
+    const int back = (pos & 31) - (pos & 12), lead = t - back, last = lead + 19;       // the unit's first token and its last, if here
+    bool whole = lead >= 0 && last < a.T;
+    if (whole) {
+      const int s = a.seq_of_token[t];
+      whole = a.seq_of_token[lead] == s && a.seq_of_token[last] == s && a.positions[lead] == pos - back && a.positions[last] == pos - back + 19;
+    }
+    if (!whole) {
+      for (int e = lane; e < a.dv; e += 64) store_f32(dst, v_offset(1, tp, e, a.dv), value_of(rows, a, t, col0 + e));
+      return;
+    }
+    if (back) return;
+    for (int e = lane; e < a.dv; e += 64) {
+      float x[8];
 #pragma unroll
-  for (int k = 0; k < 2; ++k) {                                 // every load before the first use
+      for (int j = 0; j < 8; ++j) x[j] = value_of(rows, a, t + (j & 3) + 16 * (j >> 2), col0 + e);
+      *reinterpret_cast<uint4*>(dst + v_offset(1, tp, e, a.dv)) =
+          uint4{pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]), pack_bf16x2(x[4], x[5]), pack_bf16x2(x[6], x[7])};
+    }
+  }
+}
+
+template <typename TI, typename TO, int NP, int NR, bool VEC>
+__global__ __launch_bounds__(256) void qkv_prepare_heads_kernel(const TI* __restrict__ rows, TO* __restrict__ q_out, TO* __restrict__ k_pool,
+                                                                TO* __restrict__ v_pool, HeadsArgs a) {
+  const int t0 = blockIdx.x * NR, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (h >= a.n_heads) return;
+  const int d = a.d;
+  int pos[NR], page[NR];
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const int t = min(t0 + r, a.T - 1);
+    pos[r] = a.positions[t];
+    page[r] = -1;
+    if (k_pool && h >= a.nH) {
+      page[r] = a.block_table[(size_t)a.seq_of_token[t] * a.bt_stride + pos[r] / a.page_size];
+      if (page[r] < 0 || page[r] >= a.n_pages || t0 + r >= a.T) page[r] = -1;
+    }
+  }
+  if (h >= a.nH + a.nKV) {
+#pragma unroll
+    for (int r = 0; r < NR; ++r)
+      if (page[r] >= 0) put_values<TI, TO>(rows, v_pool, a, t0 + r, h - a.nH - a.nKV, pos[r], page[r], lane);
+    return;
+  }
+  const bool is_q = h < a.nH;
+  const size_t col0 = (size_t)h * d;
+  const float* w = a.norm_w + (is_q ? 0 : d);
+  const int half = a.R >> 1, n_pairs = half + (d - a.R + 1) / 2;
+  int e0[NP], e1[NP];
+  bool on0[NP], on1[NP];
+  float w0[NP], w1[NP], x0[NR][NP], x1[NR][NP], cs[NR][NP], sn[NR][NP];
+#pragma unroll
+  for (int k = 0; k < NP; ++k) {                                // every load before the first use
     const int i = lane + 64 * k;
     const bool turned = i < half;
-    e0[k] = turned ? (interleaved ? 2 * i : i) : R + 2 * (i - half);
-    e1[k] = turned ? (interleaved ? 2 * i + 1 : i + half) : e0[k] + 1;
+    e0[k] = VEC ? 2 * i : turned ? (a.interleaved ? 2 * i : i) : a.R + 2 * (i - half);
+    e1[k] = VEC ? 2 * i + 1 : turned ? (a.interleaved ? 2 * i + 1 : i + half) : e0[k] + 1;
     on0[k] = i < n_pairs;
     on1[k] = on0[k] && e1[k] < d;
-    x0[k] = on0[k] ? load_f32(row, col0 + e0[k]) : 0.f;
-    x1[k] = on1[k] ? load_f32(row, col0 + e1[k]) : 0.f;
-    w0[k] = on0[k] ? w[e0[k]] : 0.f;
-    w1[k] = on1[k] ? w[e1[k]] : 0.f;
-    cs[k] = turned ? cos_t[(size_t)pos * half + i] : 1.f;
-    sn[k] = turned ? sin_t[(size_t)pos * half + i] : 0.f;
-  }
-  float ss = 0.f;
+    w0[k] = w1[k] = 0.f;
+    if constexpr (VEC) {
+      if (on0[k]) load_pair<float>(w, e0[k], w0[k], w1[k]);
+    } else {
+      if (on0[k]) w0[k] = w[e0[k]];
+      if (on1[k]) w1[k] = w[e1[k]];
+    }
 #pragma unroll
-  for (int k = 0; k < 2; ++k) {
-    if (bias && on0[k]) x0[k] += bias[col0 + e0[k]];
-    if (bias && on1[k]) x1[k] += bias[col0 + e1[k]];
-    ss = fmaf(x0[k], x0[k], fmaf(x1[k], x1[k], ss));
+    for (int r = 0; r < NR; ++r) {
+      const TI* row = rows + (size_t)min(t0 + r, a.T - 1) * a.row_w;
+      x0[r][k] = x1[r][k] = 0.f;
+      if constexpr (VEC) {
+        if (on0[k]) load_pair<TI>(row, col0 + e0[k], x0[r][k], x1[r][k]);
+      } else {
+        if (on0[k]) x0[r][k] = load_f32(row, col0 + e0[k]);
+        if (on1[k]) x1[r][k] = load_f32(row, col0 + e1[k]);
+      }
+      cs[r][k] = turned ? a.cos_t[(size_t)pos[r] * half + i] : 1.f;
+      sn[r][k] = turned ? a.sin_t[(size_t)pos[r] * half + i] : 0.f;
+    }
   }
-  ss = wave_sum(ss);
-  if (!is_q && page < 0) return;
-  const float inv = 1.f / sqrtf(ss / (float)d + eps);
-  TO* dst = is_q ? q_out + ((size_t)t * nH + h) * d : k_pool + (((size_t)page * nKV + (h - nH)) * page_size + tp) * d;
+  float ss[NR];
 #pragma unroll
-  for (int k = 0; k < 2; ++k) {
-    float y0, y1;
-    rotate_pair(x0[k] * inv * w0[k], x1[k] * inv * w1[k], cs[k], sn[k], y0, y1);
-    if (on0[k]) store_f32(dst, e0[k], y0);
-    if (on1[k]) store_f32(dst, e1[k], y1);
+  for (int r = 0; r < NR; ++r) {
+    ss[r] = 0.f;
+#pragma unroll
+    for (int k = 0; k < NP; ++k) {
+      if (a.bias && on0[k]) x0[r][k] += a.bias[col0 + e0[k]];
+      if (a.bias && on1[k]) x1[r][k] += a.bias[col0 + e1[k]];
+      ss[r] = fmaf(x0[r][k], x0[r][k], fmaf(x1[r][k], x1[r][k], ss[r]));
+    }
   }
+#pragma unroll
+  for (int r = 0; r < NR; ++r) ss[r] = wave_sum(ss[r]);
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const int t = t0 + r;
+    if (is_q ? t >= a.T : page[r] < 0) continue;
+    const float inv = 1.f / sqrtf(ss[r] / (float)d + a.eps);
+    TO* dst = is_q ? q_out + ((size_t)t * a.nH + h) * d : k_pool + ((size_t)page[r] * a.nKV + (h - a.nH)) * a.page_size * d;
+    const int tp = pos[r] % a.page_size;
+    auto at = [&](int e) -> size_t { return is_q ? (size_t)e : k_offset(a.layout, tp, e, d); };
+#pragma unroll
+    for (int k = 0; k < NP; ++k) {
+      float y0, y1;
+      rotate_pair(x0[r][k] * inv * w0[k], x1[r][k] * inv * w1[k], cs[r][k], sn[r][k], y0, y1);
+      if constexpr (VEC) {
+        if (on0[k]) store_pair(dst, at(e0[k]), y0, y1);         // (an even element and the next one are neighbours in both layouts)
+      } else {
+        if (on0[k]) store_f32(dst, at(e0[k]), y0);
+        if (on1[k]) store_f32(dst, at(e1[k]), y1);
+      }
+    }
+  }
+}
+
+template <typename TI, typename TO>
+void launch_heads(const void* rows, void* q_out, void* k_pool, void* v_pool, const HeadsArgs& a, hipStream_t stream) {
+  const bool vec = a.interleaved && a.d % 2 == 0 && a.row_w % 2 == 0 &&
+                   (((uintptr_t)rows | (uintptr_t)q_out | (uintptr_t)k_pool | (uintptr_t)a.norm_w) & 7) == 0;
+  const int nr = a.T >= 1024 ? 4 : 1;                           // many tokens: more loads of a wave in flight
+  const dim3 g(ceil_div(a.T, nr), ceil_div(a.n_heads, 4));
+#define GO(NP, NR, VEC) qkv_prepare_heads_kernel<TI, TO, NP, NR, VEC><<<g, 256, 0, stream>>>((const TI*)rows, (TO*)q_out, (TO*)k_pool, (TO*)v_pool, a)
+#define BY_VEC(NP, NR)          \
+  do {                          \
+    if (vec) GO(NP, NR, true);  \
+    else GO(NP, NR, false);     \
+  } while (0)
+  if (a.d <= 128) { if (nr == 4) BY_VEC(1, 4); else BY_VEC(1, 1); }
+  else { if (nr == 4) BY_VEC(2, 4); else BY_VEC(2, 1); }
+#undef BY_VEC
+#undef GO
 }
 
 // x[t, c] += (a ? a[t, c] : 0) + (v ? v[c] : 0)
@@ -199,10 +300,13 @@ extern "C" int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width
                                  int interleaved, const float* vcos, const float* vsin, const int* positions,
                                  const int* seq_of_token, const int* block_table, int bt_stride, int T, int nH, int nKV,
                                  int d, int dv, int page_size, int n_pages, const float* norm_w, int norm_heads, float norm_eps,
-                                 float* inv_rms, hipStream_t stream) {
+                                 float* inv_rms, int kv_layout, hipStream_t stream) {
   ALICE_CHECK(dtype_ok(rows_dtype) && dtype_ok(out_dtype), "qkv_prepare: unknown dtype");
   ALICE_CHECK(norm_w == nullptr || (norm_eps > 0.f && (norm_heads || inv_rms != nullptr)), "qkv_prepare: the norm needs a positive eps, and over the whole projection its workspace");
   ALICE_CHECK(norm_w == nullptr || !norm_heads || (d <= 256 && vcos == nullptr), "qkv_prepare: the norm a head takes heads of up to 256 and values as they are");
+  ALICE_CHECK(kv_layout == 0 || (kv_layout == 1 && norm_w && norm_heads && out_dtype == DT_BF16 && d % 32 == 0 && dv % 32 == 0 && (k_pool == nullptr || page_size == 64) &&
+                                 (((uintptr_t)k_pool | (uintptr_t)v_pool) & 15) == 0),
+              "qkv_prepare: pages in fragment order come with the norm a head, bfloat16, pages of 64 and head sizes that are multiples of 32");
   ALICE_CHECK(rows_dtype == DT_F32 || rows_dtype == out_dtype, "qkv_prepare: rows are float32 or in the outputs' dtype");
   ALICE_CHECK(T >= 0 && nH >= 1 && nKV >= 0 && d >= 1 && dv >= 1, "qkv_prepare: bad sizes T=%d nH=%d nKV=%d d=%d dv=%d", T, nH, nKV, d, dv);
   ALICE_CHECK(rotary_dim >= 0 && rotary_dim <= d && rotary_dim % 2 == 0, "qkv_prepare: rotated width %d must be even and at most %d", rotary_dim, d);
@@ -216,15 +320,11 @@ extern "C" int alice_qkv_prepare(const void* rows, int rows_dtype, int row_width
   if (T == 0) return 0;
   dim3 grid(T, nH + (k_pool ? 2 * nKV : 0));
   if (norm_w && norm_heads) {
-    const int n_heads = nH + (k_pool ? 2 * nKV : 0);
-    const dim3 g(T, ceil_div(n_heads, 4));
-#define GO(TI, TO)                                                                                                          \
-  qkv_prepare_heads_kernel<TI, TO><<<g, 256, 0, stream>>>((const TI*)rows, row_width, bias, norm_w, norm_eps, (TO*)q_out, (TO*)k_pool, (TO*)v_pool, \
-      cos_t, sin_t, rotary_dim, interleaved, positions, seq_of_token, block_table, bt_stride, nH, nKV, d, dv, page_size > 0 ? page_size : 1, n_pages, n_heads)
-    if (rows_dtype == DT_F32 && out_dtype == DT_F32) GO(float, float);
-    else if (rows_dtype == DT_F32) GO(float, bf16_t);
-    else GO(bf16_t, bf16_t);
-#undef GO
+    const HeadsArgs ha{row_width, rotary_dim, interleaved, bt_stride, T, nH, k_pool ? nKV : 0, d, dv, page_size > 0 ? page_size : 1, n_pages,
+                       nH + (k_pool ? 2 * nKV : 0), kv_layout, norm_eps, bias, norm_w, cos_t, sin_t, positions, seq_of_token, block_table};
+    if (rows_dtype == DT_F32 && out_dtype == DT_F32) launch_heads<float, float>(rows, q_out, k_pool, v_pool, ha, stream);
+    else if (rows_dtype == DT_F32) launch_heads<float, bf16_t>(rows, q_out, k_pool, v_pool, ha, stream);
+    else launch_heads<bf16_t, bf16_t>(rows, q_out, k_pool, v_pool, ha, stream);
     ALICE_LAUNCH_CHECK();
     return 0;
   }

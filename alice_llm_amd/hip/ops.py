@@ -17,8 +17,9 @@ from ..csrc import build as _build
 
 EPI_NONE, EPI_GEGLU, EPI_SOFTCAP = 0, 1, 2
 LAYOUT_ROW, LAYOUT_FRAG16 = 0, 1
+KV_ROW, KV_FRAGMENT = 0, 1
 LINEAR_AUTO, LINEAR_GENERIC, LINEAR_SKINNY, LINEAR_MFMA, LINEAR_TILED_W16, LINEAR_TILED_W32 = 0, 1, 2, 3, 4, 5
-ABI_VERSION = 14
+ABI_VERSION = 15
 GATED_SILU = -1.0        # epi_param of EPI_GEGLU that picks silu(gate) * up
 UNARY_RELU2 = -1.0       # epi_param of EPI_SOFTCAP that picks the square of max(y, 0) instead of the capped form
 UNARY_SILU = -2.0        # likewise y * sigmoid(y)
@@ -56,8 +57,8 @@ def _declare(lib) -> None:
         "alice_gelu_mul_rows": [P, I, P, I, I, I, P, P, I, I, I, I, I, P],
         "alice_linear_rope_cache": [P, I, P, I, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
         "alice_attention_mfma_supported": [I],
-        "alice_attention_prefill": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, I, I, I, P],
-        "alice_attention_decode": [P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, I, I, P, I, P],
+        "alice_attention_prefill": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, F, I, I, I, P, P],
+        "alice_attention_decode": [P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, I, I, P, I, P, P],
         "alice_attention_generic": [P, I, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, P, I, I, P, I, P],
         "alice_head_gate": [P, I, P, I, I, I, I, P],
         "alice_attention_masked": [P, I, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, P, I, I, P, I, I, F, I, I, P, P, P, P, P],
@@ -67,7 +68,7 @@ def _declare(lib) -> None:
         "alice_attention_split_supported": [I, I, I, I, I],
         "alice_attention_split_runs": [I],
         "alice_mix_heads": [P, P, P, I, F, P, I, I, I, I, I, I, P],
-        "alice_qkv_prepare": [P, I, I, P, P, P, P, I, P, P, I, I, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, F, P, P],
+        "alice_qkv_prepare": [P, I, I, P, P, P, P, I, P, P, I, I, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, F, P, I, P],
         "alice_short_conv": [P, I, I, I, I, P, P, P, P, I, P, P, P, I, I, P],
         "alice_ssm_prepare": [P, I, I, P, P, P, P, I, I, P],
         "alice_delta_prepare": [P, I, I, I, I, F, F, P, P, P, P, I, I, P, I, I, P],
@@ -766,7 +767,8 @@ def qkv_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], q_out: torch.T
                 value_head_dim: int, max_position: int, cos: Optional[torch.Tensor] = None,
                 sin: Optional[torch.Tensor] = None, rotary_dim: int = 0, interleaved: bool = True,
                 value_cos: Optional[torch.Tensor] = None, value_sin: Optional[torch.Tensor] = None,
-                norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0, norm_heads: bool = False) -> None:
+                norm_weight: Optional[torch.Tensor] = None, norm_eps: float = 0.0, norm_heads: bool = False,
+                kv_layout: int = KV_ROW) -> None:
     """From the rows [q | k | v | ...] of a fused projection (float32, or q_out's dtype): bias [>= q, k, v columns]
     added, q and k heads rotated over their first rotary_dim dimensions in pairs ((2i, 2i + 1) if interleaved, else
     (i, i + rotary_dim / 2)) from tables [positions, rotary_dim / 2], values turned over all their dimensions where
@@ -774,7 +776,8 @@ def qkv_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], q_out: torch.T
     norm_weight: float32 [q columns + k columns (where a cache is written)]: after the bias and before the rotation, the q
     columns (all heads together) and the k columns are each divided by their root mean square over the whole projection
     (norm_eps inside the root) and multiplied by this weight.  norm_heads: float32 [2, head_dim] instead: every q head and
-    every k head by its own root mean square, times the first row (q) or the second (k)."""
+    every k head by its own root mean square, times the first row (q) or the second (k); the pools may then be in fragment
+    order (kv_layout)."""
     T = rows.shape[0]
     dt = q_out.dtype
     d, dv = head_dim, value_head_dim
@@ -823,7 +826,7 @@ def qkv_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], q_out: torch.T
           int(rotary_dim if cos is not None else 0), int(interleaved), _opt(value_cos, "value_cos"), _opt(value_sin, "value_sin"),
           positions.data_ptr(), _opt(seq_of_token, "seq_of_token"), _opt(block_table, "block_table"), bt_stride, T,
           num_heads, num_kv_heads if k_pool is not None else 0, d, dv, page_size, n_pages,
-          _opt(norm_weight, "norm_weight"), int(norm_heads), float(norm_eps), _opt(inv_rms, "inv_rms"), _stream())
+          _opt(norm_weight, "norm_weight"), int(norm_heads), float(norm_eps), _opt(inv_rms, "inv_rms"), int(kv_layout), _stream())
 
 
 def add_rows(x: torch.Tensor, rows: Optional[torch.Tensor], vector: Optional[torch.Tensor]) -> None:
@@ -1370,7 +1373,6 @@ def fragment_layout_supported(rows: int, k_in: int, epilogue: int) -> bool:
     return bool(library().alice_frag16_supported(int(rows), int(k_in), int(epilogue)))
 
 
-KV_ROW, KV_FRAGMENT = 0, 1
 ATTN_PARTS_HEAD = 4             # floats before a split's output in the parts of attention_decode (ALICE_ATTN_PARTS_HEAD)
 KV_FRAGMENT_PAGE = 64            # positions per page that the fragment layout of keys and values is written for
 ATTENTION_MAX_HEAD_DIM = 256     # the largest head size any attention kernel here takes
@@ -1401,11 +1403,12 @@ PREFILL_AUTO, PREFILL_TILES, PREFILL_SPLIT, PREFILL_SHARED4, PREFILL_SHARED8, PR
 
 def attention_prefill(q, k_pool, v_pool, out, cu_seqlens, context_lens, block_table, *, num_heads: int, n_seqs: int,
                       max_new: int, max_context: int, scale: float, softcap: Optional[float], window: Optional[int],
-                      variant: int = PREFILL_AUTO, out_layout: int = LAYOUT_ROW) -> None:
+                      variant: int = PREFILL_AUTO, out_layout: int = LAYOUT_ROW, sink: Optional[torch.Tensor] = None) -> None:
     """Prompt attention on the matrix cores.  variant: whole query tiles per wave; one tile's keys split over a
     block's four waves (what fills the chip when there are few tiles); or the four or eight waves of a block
     sharing each block of keys and values through LDS.  AUTO picks by the grid's size.
-    out_layout FRAG16: `out` is a flat buffer of ceil16(T) * num_heads * d elements in fragment order."""
+    out_layout FRAG16: `out` is a flat buffer of ceil16(T) * num_heads * d elements in fragment order.
+    sink: float32 [num_heads], exp(sink) joins the softmax's denominator."""
     n_pages, nKV, page_size, d = k_pool.shape
     T = q.shape[0]
     _dev(q, "q", torch.bfloat16, (T, num_heads * d))
@@ -1423,13 +1426,14 @@ def attention_prefill(q, k_pool, v_pool, out, cu_seqlens, context_lens, block_ta
     _call("alice_attention_prefill", q.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr(), out.data_ptr(),
           cu_seqlens.data_ptr(), context_lens.data_ptr(), block_table.data_ptr(), block_table.shape[1], n_seqs,
           max_new, num_heads, nKV, d, page_size, float(scale), float(softcap or 0.0), int(window or 0), int(variant),
-          int(out_layout), _stream())
+          int(out_layout), _opt(sink, "sink", torch.float32, (num_heads,)), _stream())
 
 
 def attention_decode(q, k_pool, v_pool, out, context_lens, block_table, *, num_heads: int, max_context: int,
                      scale: float, softcap: Optional[float], window: Optional[int], splits: Optional[int] = None,
-                     out_layout: int = LAYOUT_ROW, gate: Optional[torch.Tensor] = None):
-    """gate: bfloat16 [B, >= heads] with unit column stride; applied where the key splits are combined (so only with
+                     out_layout: int = LAYOUT_ROW, gate: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None):
+    """sink: float32 [num_heads], exp(sink) joins the softmax's denominator (in the first of the key splits).
+    gate: bfloat16 [B, >= heads] with unit column stride; applied where the key splits are combined (so only with
     splits > 1 and an output; returns False in the third place otherwise and the caller gates the output itself).
     out_layout FRAG16: `out` is a flat buffer of ceil16(B) * num_heads * d elements in fragment order.
     Returns (parts, splits).  With out=None the keys' splits are left uncombined in `parts`
@@ -1465,7 +1469,7 @@ def attention_decode(q, k_pool, v_pool, out, context_lens, block_table, *, num_h
     _call("alice_attention_decode", q.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr(), None if out is None else out.data_ptr(),
           _opt(parts, "parts"), context_lens.data_ptr(), block_table.data_ptr(), block_table.shape[1], B, num_heads,
           nKV, d, page_size, float(scale), float(softcap or 0.0), int(window or 0), splits, int(out_layout),
-          gate_ptr, int(gate_stride), _stream())
+          gate_ptr, int(gate_stride), _opt(sink, "sink", torch.float32, (num_heads,)), _stream())
     if gate is not None:
         return parts, splits, gate_ptr is not None
     return parts, splits
@@ -1504,9 +1508,9 @@ def attention(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, out: 
               block_table: torch.Tensor, *, num_heads: int, scale: float, softcap: Optional[float],
               window: Optional[int], full_precision: bool, kv_layout: int = KV_ROW,
               out_layout: int = LAYOUT_ROW, bias_slopes: Optional[torch.Tensor] = None,
-              gate: Optional[torch.Tensor] = None) -> None:
+              gate: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None) -> None:
     """Attention of the step's query tokens over the cache; picks the kernel for the step's shape and
-    the cache's layout.  `ctx` carries positions, seq_of_token, cu_seqlens, context_lens and the
+    the cache's layout.  A sink (see attention_decode) is taken over a cache in fragment order.  `ctx` carries positions, seq_of_token, cu_seqlens, context_lens and the
     host-side sizes of the step.  out_layout FRAG16 is taken by the matrix-core kernels only; a score bias
     (bias_slopes, see attention_generic) by the generic kernel only, over a row-major cache."""
     if kv_layout == KV_FRAGMENT:
@@ -1516,19 +1520,19 @@ def attention(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, out: 
         if ctx.is_decode and num_heads // nKV <= 16:
             res = attention_decode(q, k_pool, v_pool, out, ctx.context_lens, block_table, num_heads=num_heads,
                                    max_context=ctx.max_context, scale=scale, softcap=softcap, window=window,
-                                   out_layout=out_layout, gate=gate)
+                                   out_layout=out_layout, gate=gate, sink=sink)
             if gate is not None and res[2]:
                 return                                         # gated where the key splits were combined
         else:
             attention_prefill(q, k_pool, v_pool, out, ctx.cu_seqlens, ctx.context_lens, block_table,
                               num_heads=num_heads, n_seqs=ctx.n_seqs, max_new=ctx.max_new,
                               max_context=ctx.max_context, scale=scale, softcap=softcap, window=window,
-                              out_layout=out_layout)
+                              out_layout=out_layout, sink=sink)
         if gate is not None:
             head_gate(out, out_layout, gate, q.shape[0], num_heads, k_pool.shape[3])
         return
-    if out_layout != LAYOUT_ROW:
-        raise HipLibraryError("only the matrix-core attention kernels write fragment order")
+    if out_layout != LAYOUT_ROW or sink is not None:
+        raise HipLibraryError("only the matrix-core attention kernels write fragment order, and here only they take a sink")
     attention_generic(q, k_pool, v_pool, out, ctx.positions, ctx.seq_of_token, block_table,
                       num_heads=num_heads, scale=scale, softcap=softcap, window=window,
                       max_position=ctx.max_position, full_precision=full_precision, bias_slopes=bias_slopes, gate=gate)

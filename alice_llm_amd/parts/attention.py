@@ -14,8 +14,9 @@ multiplied by sigmoid(gate_h) before the output projection.  tensor_names gives 
 matrices (q, k, v, o, g) where a file names them otherwise.
 
 Further constructor arguments, each off by default, make other attention mixers from the same part (they run
-on the 32-bit attention kernel over a row-major cache in both dtypes, from a projection whose sums stay 32-bit
-until the bias is added and the rotation done):
+on kernels of their own over a row-major cache, from a projection whose sums stay 32-bit until the bias is added and
+the rotation done; a mixer with a norm a head, with or without a sink, and no other of these terms keeps the matrix-core
+kernels and their cache in bfloat16):
   bias            q, k and v have biases (the matrix's name + ".b"), added in the projection
   chunk           a query sees the keys of its own chunk of that many positions only, chunks counted from the
                   sequence's position 0 (the cache gives the pages of finished chunks back like a window's)
@@ -129,9 +130,13 @@ class Attention(Part):
         # How this mixer lays keys and values out inside a page: the matrix-core kernels read a fragment
         # layout; every other case is row-major.  It depends on the arithmetic and the head size alone, so
         # that a run that reads another run's cache finds the layout it expects.
+        # Of the further arguments a norm a head, a sink and a rotation in neighbouring pairs go with the fragment layout
+        # as well: the one is done where keys are written, the other is where the running softmax starts.
+        plain_mask = not (chunk or keep_first or talk or output_gate or output_scale != 1.0 or output_bias) and own_keys
         self.kv_layout = (ops.KV_FRAGMENT if precision.name == "bfloat16" and precision.act == torch.bfloat16
                           and ops.library_ready() and ops.attention_mfma_supported(head_dim)
-                          and score_bias_slopes is None and self.dv == head_dim and not self.extended else ops.KV_ROW)
+                          and score_bias_slopes is None and self.dv == head_dim
+                          and (not self.extended or (qk_norm == "head" and plain_mask)) else ops.KV_ROW)
         self._parts: Dict[str, torch.Tensor] = {}
 
     def param_specs(self) -> Dict[str, ParamSpec]:
@@ -220,14 +225,16 @@ class Attention(Part):
         """x: [T, H] in the activation dtype (a tensor, or FragmentActs in decode steps); returns the branch
         in float32 ([T, H] or partial sums)."""
         T = x.shape[0]
-        if self.extended:
+        if self.extended and self.kv_layout != ops.KV_FRAGMENT:
             return self._forward_extended(x, ctx, cache)
         q = torch.empty((T, self.q_dim), dtype=self.precision.act, device=x.device)
         geometry = dict(num_heads=self.nH, num_kv_heads=self.nKV, head_dim=self.d, kv_layout=self.kv_layout)
         if self.dv != self.d:
             geometry["value_head_dim"] = self.dv
         gate = None
-        fused = self.pair_order and self.position.project_rotate_store(self.qkv, x, q, ctx, cache, **geometry)
+        if self.extended:
+            self._prepare(self.qkv(x, torch.float32), q, ctx, cache)
+        fused = self.extended or self.pair_order and self.position.project_rotate_store(self.qkv, x, q, ctx, cache, **geometry)
         if not fused:
             qkv = self.qkv(x, self.precision.act)
             if self.n_gate:
@@ -246,7 +253,7 @@ class Attention(Part):
             if slices > 0:
                 parts, _ = ops.attention_decode(q, cache.k, cache.v, None, ctx.context_lens, cache.block_table,
                                                 num_heads=self.nH, max_context=ctx.max_context, scale=self.scale,
-                                                softcap=self.softcap, window=self.window, splits=splits)
+                                                softcap=self.softcap, window=self.window, splits=splits, sink=self.sink)
                 y = torch.empty((slices, T, self.o.n), dtype=torch.float32, device=q.device)
                 ops.linear_parts(parts, splits, self.o.weight, y, num_heads=self.nH, head_dim=self.d)
                 return y if slices > 1 else y[0]
@@ -258,14 +265,11 @@ class Attention(Part):
         ops.attention(q, cache.k, cache.v, out.data if frag else out, ctx, cache.block_table, num_heads=self.nH,
                       scale=self.scale, softcap=self.softcap, window=self.window, full_precision=self.precision.full,
                       kv_layout=self.kv_layout, out_layout=ops.LAYOUT_FRAG16 if frag else ops.LAYOUT_ROW,
-                      bias_slopes=self._slopes, gate=gate)
+                      bias_slopes=self._slopes, gate=gate, sink=self.sink)
         return self.o(out, torch.float32, allow_partials=True)
 
-    def _forward_extended(self, x, ctx, cache) -> torch.Tensor:
-        """The mixers made by the further constructor arguments (see the top of the file)."""
-        T, act, dev = x.shape[0], self.precision.act, x.device
-        rows = self.qkv(x, torch.float32)                     # [q | k | v | g], the sums as they are
-        q = torch.empty((T, self.q_dim), dtype=act, device=dev)
+    def _prepare(self, rows, q, ctx, cache) -> None:
+        """From the projection's sums to q and the cached k and v: bias, norm, rotation."""
         pos = self.position
         write = cache is not None and cache.writable
         if write and not self.own_keys:
@@ -279,7 +283,15 @@ class Attention(Part):
                         max_position=ctx.max_position, cos=getattr(pos, "cos", None), sin=getattr(pos, "sin", None),
                         rotary_dim=getattr(pos, "rotary_dim", 0), interleaved=getattr(pos, "interleaved", True),
                         value_cos=getattr(pos, "value_cos", None), value_sin=getattr(pos, "value_sin", None),
-                        norm_weight=norm_w, norm_eps=self.qk_norm_eps, norm_heads=self.qk_norm == "head")
+                        norm_weight=norm_w, norm_eps=self.qk_norm_eps, norm_heads=self.qk_norm == "head", kv_layout=self.kv_layout)
+
+    def _forward_extended(self, x, ctx, cache) -> torch.Tensor:
+        """The mixers made by the further constructor arguments (see the top of the file)."""
+        T, act, dev = x.shape[0], self.precision.act, x.device
+        rows = self.qkv(x, torch.float32)                     # [q | k | v | g], the sums as they are
+        q = torch.empty((T, self.q_dim), dtype=act, device=dev)
+        pos = self.position
+        self._prepare(rows, q, ctx, cache)
         gate = None
         if self.n_gate:
             g0 = self.q_dim + self.kv_dim + self.v_dim

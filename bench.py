@@ -19,6 +19,8 @@ of 6,000 tokens, past the window, at the 27B shape.
         instead of the above: the Vifirax design beside Telulorn and Gemma 2 at equal layer sizes, in a line of its own
     python bench.py --kabapel w2048,w4096
         instead of the above: the Kabapel design beside Vifirax and Pefitar at equal layer sizes, in a line of its own
+    python bench.py --vazilorn w2048,w4096
+        instead of the above: the Vazilorn design beside Kabapel and Gemma 2 at equal layer sizes, in a line of its own
     python bench.py --novotar w2048,w4096
         instead of the above: prefill and decode throughput of the Novotar design at layer sizes of real models
         (random weights, a few layers), beside Gemma 2 at equal sizes; prints a line of its own
@@ -398,7 +400,22 @@ def kabapel_configs(size, vocab=32768):
                        layer("lightning", lin, moe), layer("latent_attention", dict(lat, kv_from=1), moe), layer("lightning", lin, dense)]}
 
 
-def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar=False, with_vifirax=False, with_kabapel=False):
+def vazilorn_configs(size, vocab=32768, window=1024):
+    """A Vazilorn configuration of six layers at the sizes of novotar_pair_configs: the same width, attention heads and window;
+    the first and the last feed-forward dense (the same size), the others routed (16 experts of a quarter of that size in two
+    groups, 2 a token from one of them, and a shared expert of a quarter), as in kabapel_configs."""
+    z = NOVOTAR_SIZES[size]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"] // 4}, "shared": {"ff": z["ff"] // 4},
+           "router": {"experts": 16, "top": 2, "scale": 2.5, "groups": {"count": 2, "keep": 1}}}
+    att = {"heads": z["heads"], "kv_heads": z["kv"], "dim": z["dim"], "vdim": z["dim"], "scale": z["dim"] ** -0.5, "mask": {"size": window},
+           "rot": {"base": 500000.0, "dims": z["dim"], "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    return {"architecture": "Vazilorn", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-6},
+            "layers": [{"type": "attention", "mixer": att, "mlp": dense if i in (0, 5) else moe} for i in range(6)]}
+
+
+def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar=False, with_vifirax=False, with_kabapel=False,
+                  with_vazilorn=False):
     out = {}
     for size in sizes:
         if size not in NOVOTAR_SIZES:
@@ -413,6 +430,8 @@ def novotar_bench(sizes, dtype, steps, warmup, with_telulorn=False, with_pefitar
             models = [("vifirax", vifirax_configs(size)), ("telulorn", telulorn_configs(size)), models[-1]]
         if with_kabapel:
             models = [("kabapel", kabapel_configs(size)), ("vifirax", vifirax_configs(size)), ("pefitar", pefitar_configs(size))]
+        if with_vazilorn:
+            models = [("vazilorn", vazilorn_configs(size)), ("kabapel", kabapel_configs(size)), models[-1]]
         for name, raw in models:
             run = Run(None, None, dtype, raw=raw)
             r = {"weights_gb": round(run.weight_bytes / 1e9, 3), "layer_runs": len(run.model.lm.plan.schedule)}
@@ -494,6 +513,8 @@ def main() -> int:
                     "equal layer sizes, in a line of its own")
     ap.add_argument("--kabapel", default="", help="sizes (w2048,w4096): measure the Kabapel design beside Vifirax and Pefitar at "
                     "equal layer sizes, in a line of its own")
+    ap.add_argument("--vazilorn", default="", help="sizes (w2048,w4096): measure the Vazilorn design beside Kabapel and Gemma 2 at "
+                    "equal layer sizes, in a line of its own")
     ap.add_argument("--no-peaks", action="store_true", help="skip the measurement of this GPU's own copy and matrix-product rates")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -502,6 +523,13 @@ def main() -> int:
 
     import torch
     torch.cuda.set_device(0)
+    if args.vazilorn:
+        steps = min(args.steps, 64)
+        res = novotar_bench([x for x in args.vazilorn.split(",") if x], args.dtype, steps, min(args.warmup, 5), with_vazilorn=True)
+        print(json.dumps({"metric": "Vazilorn beside Kabapel and Gemma 2 at equal layer sizes: prefill and decode, random weights",
+                          "unit": "tokens/s", "n_gpus": 1, "steps": steps, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                          "data": "synthetic (uniform random token ids, random weights)", "sizes": res}), flush=True)
+        return 0
     if args.kabapel:
         steps = min(args.steps, 64)
         res = novotar_bench([x for x in args.kabapel.split(",") if x], args.dtype, steps, min(args.warmup, 5), with_kabapel=True)
