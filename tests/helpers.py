@@ -801,3 +801,137 @@ def kabapel_folder(name: str, seed: int = 0) -> str:
         save_file({k: v.contiguous() for k, v in tensors.items()}, os.path.join(folder, "model.safetensors"))
         _FOLDERS[key] = folder
     return _FOLDERS[key]
+
+
+# ------------------------------------------------------------------ Vazilorn: small configurations that differ in every size and option
+
+def _vz_rot(dims, base=1000.0, scaling=None):
+    rot = {"base": base, "dims": dims}
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "low", "high", "original"), scaling))
+    return rot
+
+
+def _vz_att(heads, kv, dim, scale, window, rot, vdim=None):
+    return {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim if vdim is None else vdim, "scale": scale,
+            "mask": {"size": window}, "rot": rot}
+
+
+def _vz_moe(experts, top, ff, scale=1.0, groups=None, shared=None):
+    router = {"experts": experts, "top": top, "scale": scale}
+    if groups is not None:
+        router["groups"] = {"count": groups[0], "keep": groups[1]}
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": router}
+    if shared is not None:
+        mlp["shared"] = {"ff": shared}
+    return mlp
+
+
+def _vz_model(vocab, width, layers, eps=1e-6):
+    return {"architecture": "Vazilorn", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "layers": [{"type": "attention", "mixer": m, "mlp": f} for m, f in layers]}
+
+
+def _vz_a():
+    att = _vz_att(4, 2, 16, 0.5, 9, _vz_rot(8, 100.0, (4.0, 1.0, 4.0, 16)), vdim=24)
+    return _vz_model(97, 64, [(att, {"kind": "dense", "ff": 96}), (att, _vz_moe(6, 2, 24, 1.7, (2, 1), 40)), (att, None),
+                              (dict(att, mask={"size": 30}), _vz_moe(5, 1, 16))])
+
+
+def _vz_b():
+    """No size suits a tile; every expert serves; the whole head turned at frequencies as they are; one kv head a query head."""
+    return _vz_model(130, 72, [(_vz_att(3, 3, 20, 0.4, 33, _vz_rot(20, 10000.0)), _vz_moe(5, 5, 18, 0.8)),
+                               (_vz_att(3, 1, 12, 0.6, 1, _vz_rot(4, 50.0), vdim=28), {"kind": "dense", "ff": 100})], eps=1e-4)
+
+
+def _vz_c():
+    """Head sizes of the matrix-core attention kernels."""
+    rot = _vz_rot(32, 500.0, (16.0, 0.5, 8.0, 64))
+    return _vz_model(300, 160, [(_vz_att(6, 2, 64, 0.25, 70, rot), {"kind": "dense", "ff": 256}),
+                                (_vz_att(2, 1, 128, 0.15, 64, _vz_rot(128, 2e4, (8.0, 1.0, 4.0, 256))), _vz_moe(8, 3, 64, 2.0, (4, 2), 96)),
+                                (_vz_att(4, 4, 64, 0.2, 33, rot), _vz_moe(16, 2, 32, 1.3, (8, 3))),
+                                (_vz_att(1, 1, 256, 0.1, 100, _vz_rot(64, 1e4)), None)], eps=1e-5)
+
+
+def _vz_d():
+    """More query heads on a kv head than the single-token kernels of either kind take in one block."""
+    return _vz_model(61, 96, [(_vz_att(18, 1, 64, 0.2, 66, _vz_rot(64, 300.0, (2.0, 1.0, 2.0, 32))), _vz_moe(4, 3, 40, 3.0, (2, 2), 24)),
+                              (_vz_att(18, 1, 16, 0.4, 12, _vz_rot(16, 300.0)), {"kind": "dense", "ff": 80})])
+
+
+def _vz_e():
+    """Values wider and narrower than keys at sizes that fit tiles; a window as long as a page, one longer than the prompts."""
+    return _vz_model(200, 128, [(_vz_att(4, 2, 64, 0.25, 64, _vz_rot(48, 700.0, (4.0, 2.0, 3.0, 128)), vdim=128), _vz_moe(12, 4, 32, 2.5, (6, 4), 64)),
+                                (_vz_att(2, 2, 128, 0.12, 1000, _vz_rot(96, 1e5), vdim=64), _vz_moe(3, 2, 96, 1.0, None, 32))], eps=3e-6)
+
+
+def _vz_f():
+    """Odd sizes, groups of a single expert, a group that outscores another by its second best."""
+    return _vz_model(83, 50, [(_vz_att(5, 5, 7, 0.7, 20, _vz_rot(6, 80.0, (3.0, 1.0, 4.0, 24)), vdim=5), _vz_moe(4, 2, 9, 1.1, (4, 3), 15)),
+                              (_vz_att(2, 1, 10, 0.5, 25, _vz_rot(2, 80.0)), _vz_moe(9, 3, 16, 0.6, (3, 1)))])
+
+
+VAZILORN = {"vz-a": _vz_a, "vz-b": _vz_b, "vz-c": _vz_c, "vz-d": _vz_d, "vz-e": _vz_e, "vz-f": _vz_f}
+
+
+def vazilorn_tensors(raw: dict, seed: int):
+    """Random tensors for a Vazilorn configuration, by name, in bfloat16 on the CPU: matrices N(0, gain^2 / inputs) with gains
+    that make softmaxes sharp and routers decide; factors of the tanh norms from almost linear to well bent, weights around 1
+    and biases that matter; sinks that take a good part of the weight; corrections below zero, so that choices are of either
+    sign and a choice among masked experts' zeros would show."""
+    import alice_llm_amd as alice
+    from alice_llm_amd.engine.model import CausalLM
+    from alice_llm_amd.parts import Precision
+    cfg = alice.config_from_dict(raw)
+    specs = CausalLM(cfg.plan(), Precision.of("float32"), "cpu").param_specs()
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, spec in specs.items():
+        shape = tuple(spec.shape)
+        r = torch.randn(shape, generator=g)
+        last = name.rsplit(".", 1)[-1]
+        if last == "correction":
+            t = -0.6 + 0.15 * r
+        elif last == "alpha":
+            t = 0.3 + 0.5 * torch.rand(shape, generator=g)
+        elif last == "sink":
+            t = 1.0 + 1.5 * r
+        elif last == "b":
+            t = 0.2 * r
+        elif len(shape) == 1:
+            t = 1.0 + 0.2 * r
+        elif name == "embed":
+            t = r
+        else:
+            gain = 2.5 if last == "router" else 1.5 if last in ("up", "gate") else 1.0
+            t = r * gain / shape[1] ** 0.5
+        out[name] = t.to(torch.bfloat16)
+    return cfg, out
+
+
+def vazilorn_pair(name: str, dtype: str, seed: int = 0, device="cuda"):
+    """(the package's model, the plain model) on the same tensors."""
+    from plain.vazilorn_plain import PlainVazilorn
+    raw = VAZILORN[name]()
+    cfg, tensors = vazilorn_tensors(raw, seed)
+    plain = PlainVazilorn(raw, {k: v.double() for k, v in tensors.items()})
+    return model_from_tensors(cfg, {k: v.to(device) for k, v in tensors.items()}, dtype), plain
+
+
+def vazilorn_folder(name: str, seed: int = 0) -> str:
+    """A model folder (config.json, model.safetensors in bfloat16) of a Vazilorn test configuration."""
+    global _TMP
+    key = ("vazilorn", name, seed)
+    if key not in _FOLDERS:
+        from safetensors.torch import save_file
+        if _TMP is None:
+            _TMP = tempfile.TemporaryDirectory(prefix="alice_tests_")
+        folder = os.path.join(_TMP.name, f"{name}-{seed}")
+        os.makedirs(folder, exist_ok=True)
+        raw = VAZILORN[name]()
+        _, tensors = vazilorn_tensors(raw, seed)
+        with open(os.path.join(folder, "config.json"), "w") as f:
+            json.dump(raw, f)
+        save_file({k: v.contiguous() for k, v in tensors.items()}, os.path.join(folder, "model.safetensors"))
+        _FOLDERS[key] = folder
+    return _FOLDERS[key]
