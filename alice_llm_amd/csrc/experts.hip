@@ -434,30 +434,35 @@ __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
   f32x4 ag[RS], au[RS];
 #pragma unroll
   for (int s = 0; s < RS; ++s) ag[s] = au[s] = f32x4{0.f, 0.f, 0.f, 0.f};
-  auto step = [&](int kt, u32x4 vg, u32x4 vu) {
-    const int k = min(kt * 32 + g * 8, a.W - 8);          // a row's last, partial k-tile: the weights are zero there
+  // A burst of N k-tiles: the tokens' rows (from the L2) and the weight tiles are all on their way before the first product.
+  auto burst = [&](auto count, int kt0) {
+    constexpr int N = decltype(count)::value;
+    u32x4 vg[N], vu[N], b[N][RS];
 #pragma unroll
-    for (int s = 0; s < RS; ++s) {
-      if (!on[s]) continue;
-      const u32x4 b = *reinterpret_cast<const u32x4*>(xr[s] + k);
-      ag[s] = mfma16(vg, b, ag[s]);
-      au[s] = mfma16(vu, b, au[s]);
+    for (int u = 0; u < N; ++u) {
+      const int k = min((kt0 + 4 * u) * 32 + g * 8, a.W - 8);        // a row's last, partial k-tile: the weights are zero there
+#pragma unroll
+      for (int s = 0; s < RS; ++s) b[u][s] = *reinterpret_cast<const u32x4*>(xr[s] + k);
     }
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      vg[u] = *reinterpret_cast<const u32x4*>(wg + (size_t)(kt0 + 4 * u) * 512);
+      vu[u] = *reinterpret_cast<const u32x4*>(wu + (size_t)(kt0 + 4 * u) * 512);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int u = 0; u < N; ++u)
+#pragma unroll
+      for (int s = 0; s < RS; ++s) {
+        if (RS > 1 && !on[s]) continue;
+        ag[s] = mfma16(vg[u], b[u][s], ag[s]);
+        au[s] = mfma16(vu[u], b[u][s], au[s]);
+      }
   };
-  constexpr int U = 8;                                    // weight tiles in flight: 2 U loads of 1 KB a wave
+  constexpr int U = RS == 1 ? 8 : 4;                      // weight tiles in flight: 2 U loads of 1 KB a wave
   int kt = wave;
-  for (; kt + 4 * (U - 1) < KT; kt += 4 * U) {
-    u32x4 vg[U], vu[U];
-#pragma unroll
-    for (int u = 0; u < U; ++u) {
-      vg[u] = *reinterpret_cast<const u32x4*>(wg + (size_t)(kt + 4 * u) * 512);
-      vu[u] = *reinterpret_cast<const u32x4*>(wu + (size_t)(kt + 4 * u) * 512);
-    }
-#pragma unroll
-    for (int u = 0; u < U; ++u) step(kt + 4 * u, vg[u], vu[u]);
-  }
-  for (; kt < KT; kt += 4)
-    step(kt, *reinterpret_cast<const u32x4*>(wg + (size_t)kt * 512), *reinterpret_cast<const u32x4*>(wu + (size_t)kt * 512));
+  for (; kt + 4 * (U - 1) < KT; kt += 4 * U) burst(std::integral_constant<int, U>{}, kt);
+  for (; kt < KT; kt += 4) burst(std::integral_constant<int, 1>{}, kt);
 #pragma unroll
   for (int s = 0; s < RS; ++s) {
     part[wave][s][0][lane] = ag[s];
@@ -491,9 +496,17 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
     int n = 0;
     for (int e0 = 0; e0 < n_exp; e0 += 64) {
       const int e = e0 + lane;
+      const float* col = e < a.E ? a.w + e : a.side + 1;
+      const int stride = e < a.E ? a.E : 2;
       bool any = false;
       if (e < n_exp)
-        for (int t = 0; t < a.T; ++t) any = any || few_weight(a, t, e) != 0.f;
+        for (int t0 = 0; t0 < a.T; t0 += 8) {             // eight loads on their way at a time
+          float v[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) v[j] = col[(size_t)min(t0 + j, a.T - 1) * stride];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) any = any | (v[j] != 0.f);
+        }
       const unsigned long long m = __ballot(any);
       if (any) list[n + __popcll(m & ((1ull << lane) - 1ull))] = (unsigned short)e;
       n += __popcll(m);
@@ -519,25 +532,29 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
       on[s] = __ballot(use[s]) != 0ull;
       mr[s] = a.mid + (size_t)min(t, a.T - 1) * row + e * a.F + g * 8;
     }
-    auto step = [&](int kt, u32x4 v) {
+    auto burst = [&](auto count, int kt0) {               // as above; rows of tokens that do not use the expert count as zero
+      constexpr int N = decltype(count)::value;
+      u32x4 v[N], b[N][RS];
 #pragma unroll
-      for (int s = 0; s < RS; ++s) {
-        if (!on[s]) continue;
-        u32x4 b = {0u, 0u, 0u, 0u};
-        if (use[s]) b = *reinterpret_cast<const u32x4*>(mr[s] + kt * 32);
-        acc[s] = mfma16(v, b, acc[s]);
-      }
+      for (int u = 0; u < N; ++u)
+#pragma unroll
+        for (int s = 0; s < RS; ++s) b[u][s] = *reinterpret_cast<const u32x4*>(mr[s] + (kt0 + 4 * u) * 32);
+#pragma unroll
+      for (int u = 0; u < N; ++u) v[u] = *reinterpret_cast<const u32x4*>(wd + (size_t)(kt0 + 4 * u) * 512);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int u = 0; u < N; ++u)
+#pragma unroll
+        for (int s = 0; s < RS; ++s) {
+          if (RS > 1 && !on[s]) continue;
+          const u32x4 bz = use[s] ? b[u][s] : u32x4{0u, 0u, 0u, 0u};
+          acc[s] = mfma16(v[u], bz, acc[s]);
+        }
     };
-    constexpr int U = 8;
+    constexpr int U = RS == 4 ? 4 : 8;
     int kt = wave;
-    for (; kt + 4 * (U - 1) < kts; kt += 4 * U) {
-      u32x4 v[U];
-#pragma unroll
-      for (int u = 0; u < U; ++u) v[u] = *reinterpret_cast<const u32x4*>(wd + (size_t)(kt + 4 * u) * 512);
-#pragma unroll
-      for (int u = 0; u < U; ++u) step(kt + 4 * u, v[u]);
-    }
-    for (; kt < kts; kt += 4) step(kt, *reinterpret_cast<const u32x4*>(wd + (size_t)kt * 512));
+    for (; kt + 4 * (U - 1) < kts; kt += 4 * U) burst(std::integral_constant<int, U>{}, kt);
+    for (; kt < kts; kt += 4) burst(std::integral_constant<int, 1>{}, kt);
   }
 #pragma unroll
   for (int s = 0; s < RS; ++s) part[wave][s][lane] = acc[s];
