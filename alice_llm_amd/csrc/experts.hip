@@ -409,9 +409,11 @@ __device__ __forceinline__ float few_weight(const FewArgs& a, int t, int e) {
   return e < a.E ? a.w[(size_t)t * a.E + e] : a.side[2 * (size_t)t + 1];
 }
 
+// RS: tokens a step in sets of 16.  The tokens that use the expert stand side by side as the products' columns, whichever
+// they are, so most blocks need one set.
 template <int RS>
 __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
-  __shared__ f32x4 part[4][RS][2][64];
+  __shared__ f32x4 part[4][2][64];
   const int e = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
   const bool shared = e == a.E;
   const int F = shared ? a.Fs : a.F, f0 = blockIdx.x * 16;
@@ -419,31 +421,33 @@ __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
   const float wt = few_weight(a, lane, e);                // lane = token (at most 64)
   const unsigned long long used = __ballot(wt != 0.f);
   if (used == 0ull) return;
+  const int n_used = __popcll(used), sets = RS == 1 ? 1 : (n_used + 15) >> 4;
+  const unsigned long long below = (1ull << lane) - 1ull;
+  // lane i: the i-th token that uses the expert, then the others
+  const int token_at = __builtin_amdgcn_ds_permute((wt != 0.f ? __popcll(used & below) : n_used + __popcll(~used & below)) * 4, lane);
   const int KT = (a.W + 31) / 32;
   const bf16_t* base = shared ? a.shared_gate_up : a.gate_up;
   const int first = shared ? f0 : e * F + f0, half = shared ? F : a.E * F;
   const bf16_t* wg = base + (size_t)(first / 16) * KT * 512 + lane * 8;
   const bf16_t* wu = base + (size_t)((half + first) / 16) * KT * 512 + lane * 8;
-  const bf16_t* xr[RS];
-  bool on[RS];
-#pragma unroll
-  for (int s = 0; s < RS; ++s) {
-    on[s] = ((used >> (16 * s)) & 0xffffull) != 0ull;
-    xr[s] = a.x + (size_t)min(s * 16 + c, a.T - 1) * a.W;
-  }
+  int token[RS];
   f32x4 ag[RS], au[RS];
 #pragma unroll
-  for (int s = 0; s < RS; ++s) ag[s] = au[s] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // A burst of N k-tiles: the tokens' rows (from the L2) and the weight tiles are all on their way before the first product.
+  for (int s = 0; s < RS; ++s) {
+    token[s] = __shfl(token_at, s * 16 + c, 64);
+    ag[s] = au[s] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  // A burst of N k-tiles: the first set's rows (from the L2) and the weight tiles are all on their way before the first product.
   auto burst = [&](auto count, int kt0) {
     constexpr int N = decltype(count)::value;
-    u32x4 vg[N], vu[N], b[N][RS];
+    u32x4 vg[N], vu[N], b[N];
+    auto rows = [&](int s) {
+      const bf16_t* xr = a.x + (size_t)min(token[s], a.T - 1) * a.W;
 #pragma unroll
-    for (int u = 0; u < N; ++u) {
-      const int k = min((kt0 + 4 * u) * 32 + g * 8, a.W - 8);        // a row's last, partial k-tile: the weights are zero there
-#pragma unroll
-      for (int s = 0; s < RS; ++s) b[u][s] = *reinterpret_cast<const u32x4*>(xr[s] + k);
-    }
+      for (int u = 0; u < N; ++u)                          // a row's last, partial k-tile: the weights are zero there
+        b[u] = *reinterpret_cast<const u32x4*>(xr + min((kt0 + 4 * u) * 32 + g * 8, a.W - 8));
+    };
+    rows(0);
 #pragma unroll
     for (int u = 0; u < N; ++u) {
       vg[u] = *reinterpret_cast<const u32x4*>(wg + (size_t)(kt0 + 4 * u) * 512);
@@ -451,43 +455,48 @@ __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
     }
     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int u = 0; u < N; ++u)
+    for (int s = 0; s < RS; ++s) {
+      if (s >= sets) break;                                // (the same for the whole block)
+      if (s > 0) rows(s);
 #pragma unroll
-      for (int s = 0; s < RS; ++s) {
-        if (RS > 1 && !on[s]) continue;
-        ag[s] = mfma16(vg[u], b[u][s], ag[s]);
-        au[s] = mfma16(vu[u], b[u][s], au[s]);
+      for (int u = 0; u < N; ++u) {
+        ag[s] = mfma16(vg[u], b[u], ag[s]);
+        au[s] = mfma16(vu[u], b[u], au[s]);
       }
+    }
   };
-  constexpr int U = RS == 1 ? 8 : 4;                      // weight tiles in flight: 2 U loads of 1 KB a wave
+  constexpr int U = 8;                                    // weight tiles in flight: 2 U loads of 1 KB a wave
   int kt = wave;
   for (; kt + 4 * (U - 1) < KT; kt += 4 * U) burst(std::integral_constant<int, U>{}, kt);
-  for (; kt < KT; kt += 4) burst(std::integral_constant<int, 1>{}, kt);
+  if (kt + 4 * 3 < KT) { burst(std::integral_constant<int, 4>{}, kt); kt += 16; }
+  if (kt + 4 < KT) { burst(std::integral_constant<int, 2>{}, kt); kt += 8; }
+  if (kt < KT) burst(std::integral_constant<int, 1>{}, kt);
 #pragma unroll
   for (int s = 0; s < RS; ++s) {
-    part[wave][s][0][lane] = ag[s];
-    part[wave][s][1][lane] = au[s];
-  }
-  __syncthreads();
-  for (int s = wave; s < RS; s += 4) {
-    const int t = s * 16 + c;
-    const float wr = __shfl(wt, t, 64);
-    f32x4 gs = part[0][s][0][lane], us = part[0][s][1][lane];
+    if (s >= sets) break;
+    if (s > 0) __syncthreads();                           // the last set's parts have been read
+    part[wave][0][lane] = ag[s];
+    part[wave][1][lane] = au[s];
+    __syncthreads();
+    if (wave != s % 4) continue;
+    const float wr = __shfl(wt, token[s], 64);
+    f32x4 gs = part[0][0][lane], us = part[0][1][lane];
 #pragma unroll
     for (int n = 1; n < 4; ++n) {
-      gs += part[n][s][0][lane];
-      us += part[n][s][1][lane];
+      gs += part[n][0][lane];
+      us += part[n][1][lane];
     }
     f32x4 o;
 #pragma unroll
     for (int i = 0; i < 4; ++i) o[i] = gated_act(gs[i], us[i], shared ? a.shared_epi : a.epi, false) * wr;
-    if (t < a.T && wr != 0.f) store4(a.mid, (size_t)t * (a.E * a.F + a.Fs), e * a.F + f0 + g * 4, e * a.F + F, o);
+    if (wr != 0.f) store4(a.mid, (size_t)token[s] * (a.E * a.F + a.Fs), e * a.F + f0 + g * 4, e * a.F + F, o);
   }
 }
 
 template <int RS>
 __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
   __shared__ unsigned short list[MAX_EXPERTS + 1];
+  __shared__ unsigned long long users[MAX_EXPERTS + 1];
   __shared__ int n_list;
   __shared__ f32x4 part[4][RS][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, c = lane & 15;
@@ -498,17 +507,22 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
       const int e = e0 + lane;
       const float* col = e < a.E ? a.w + e : a.side + 1;
       const int stride = e < a.E ? a.E : 2;
-      bool any = false;
+      unsigned long long who = 0ull;                      // bit t: token t uses the expert
       if (e < n_exp)
         for (int t0 = 0; t0 < a.T; t0 += 8) {             // eight loads on their way at a time
           float v[8];
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[j] = col[(size_t)min(t0 + j, a.T - 1) * stride];
 #pragma unroll
-          for (int j = 0; j < 8; ++j) any = any | (v[j] != 0.f);
+          for (int j = 0; j < 8; ++j)
+            if (t0 + j < a.T && v[j] != 0.f) who |= 1ull << (t0 + j);
         }
-      const unsigned long long m = __ballot(any);
-      if (any) list[n + __popcll(m & ((1ull << lane) - 1ull))] = (unsigned short)e;
+      const unsigned long long m = __ballot(who != 0ull);
+      if (who) {
+        const int at = n + __popcll(m & ((1ull << lane) - 1ull));
+        list[at] = (unsigned short)e;
+        users[at] = who;
+      }
       n += __popcll(m);
     }
     if (lane == 0) n_list = n;
@@ -520,6 +534,7 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
   for (int s = 0; s < RS; ++s) acc[s] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int i = z; i < n_list; i += a.splits) {
     const int e = list[i];
+    const unsigned long long who = users[i];
     const bool shared = e == a.E;
     const int kts = (shared ? a.Fs : a.F) / 32;           // F and Fs are multiples of 32: an expert's k-tiles are its own
     const bf16_t* wd = (shared ? a.shared_down + (size_t)(n0 / 16) * KTS * 512 : a.down + ((size_t)(n0 / 16) * KT + e * a.F / 32) * 512) + lane * 8;
@@ -528,17 +543,22 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
 #pragma unroll
     for (int s = 0; s < RS; ++s) {
       const int t = s * 16 + c;
-      use[s] = few_weight(a, t, e) != 0.f;
+      use[s] = (who >> t) & 1ull;
       on[s] = __ballot(use[s]) != 0ull;
       mr[s] = a.mid + (size_t)min(t, a.T - 1) * row + e * a.F + g * 8;
     }
-    auto burst = [&](auto count, int kt0) {               // as above; rows of tokens that do not use the expert count as zero
+    auto burst = [&](auto count, int kt0) {               // as above; tokens that do not use the expert count as zero
       constexpr int N = decltype(count)::value;
       u32x4 v[N], b[N][RS];
 #pragma unroll
-      for (int u = 0; u < N; ++u)
+      for (int s = 0; s < RS; ++s) {
 #pragma unroll
-        for (int s = 0; s < RS; ++s) b[u][s] = *reinterpret_cast<const u32x4*>(mr[s] + (kt0 + 4 * u) * 32);
+        for (int u = 0; u < N; ++u) b[u][s] = u32x4{0u, 0u, 0u, 0u};
+        if (use[s]) {
+#pragma unroll
+          for (int u = 0; u < N; ++u) b[u][s] = *reinterpret_cast<const u32x4*>(mr[s] + (kt0 + 4 * u) * 32);
+        }
+      }
 #pragma unroll
       for (int u = 0; u < N; ++u) v[u] = *reinterpret_cast<const u32x4*>(wd + (size_t)(kt0 + 4 * u) * 512);
       __builtin_amdgcn_sched_barrier(0);
@@ -547,14 +567,15 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
 #pragma unroll
         for (int s = 0; s < RS; ++s) {
           if (RS > 1 && !on[s]) continue;
-          const u32x4 bz = use[s] ? b[u][s] : u32x4{0u, 0u, 0u, 0u};
-          acc[s] = mfma16(v[u], bz, acc[s]);
+          acc[s] = mfma16(v[u], b[u][s], acc[s]);
         }
     };
     constexpr int U = RS == 4 ? 4 : 8;
     int kt = wave;
     for (; kt + 4 * (U - 1) < kts; kt += 4 * U) burst(std::integral_constant<int, U>{}, kt);
-    for (; kt < kts; kt += 4) burst(std::integral_constant<int, 1>{}, kt);
+    if (kt + 4 * 3 < kts) { burst(std::integral_constant<int, 4>{}, kt); kt += 16; }
+    if (kt + 4 < kts) { burst(std::integral_constant<int, 2>{}, kt); kt += 8; }
+    if (kt < kts) burst(std::integral_constant<int, 1>{}, kt);
   }
 #pragma unroll
   for (int s = 0; s < RS; ++s) part[wave][s][lane] = acc[s];

@@ -41,10 +41,14 @@ from .feedforward import GatedMLP
 from .linear import Linear
 
 _GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
-GROUPED_FROM_TOKENS = 64       # steps of this many tokens and more take the grouped products (bfloat16, sizes that suit the tiles): as
-                               # fast as one pass over all experts' matrices with 16 experts, faster with 64 (2 a token)
-FEW_CHOICES = 1.9              # steps of at most 64 tokens whose tokens x top is at most this many times the router's outputs read
-                               # the chosen experts only (beyond, one pass over all of them is as fast: measured at 16 and 64 experts)
+# Which of the ways (bfloat16, sizes that suit the tiles), measured with choices spread evenly over 8 to 128 experts.  Steps of at
+# most 32 tokens read the chosen experts only.  Steps of 33 to 64 tokens do so too if there are at most FEW_CHOICES (token,
+# expert) pairs to a router output (beyond, most tokens meet most experts) and an expert's matrices have at most
+# FEW_MATRIX_ELEMENTS numbers each.  Else steps of GROUPED_FROM_TOKENS and more take the grouped products, and smaller ones one
+# pass over all experts' matrices.  (At most 32 tokens have at most 32 pairs to an output, twice FEW_CHOICES.)
+GROUPED_FROM_TOKENS = 64
+FEW_CHOICES = 16.0
+FEW_MATRIX_ELEMENTS = 1 << 23
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
 
 
@@ -187,9 +191,14 @@ class ExpertMLP(Part):
         it (single tokens: the batch's bucket; short prompts: a multiple of 16), so that both kinds of step add alike."""
         n = (getattr(ctx, "rounded_seqs", 0) if getattr(ctx, "is_decode", False) else 0) or -(-T // 16) * 16
         tiles = [self.gate_up, self.down] + ([] if self.shared is None else [self.shared.gate_up, self.shared.down])
-        return (T <= n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs and n < GROUPED_FROM_TOKENS
+        return (T <= n and self._few_pays(n)
                 and all(p.layout == ops.LAYOUT_FRAG16 for p in tiles) and (self.shared is None or self.shared.I % 32 == 0)
                 and ops.expert_products_supported(x.dtype, self.H, self.F))
+
+    def _few_pays(self, n: int) -> bool:
+        if n <= 32:
+            return n * self.top <= 2 * FEW_CHOICES * self.outputs
+        return n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs and self.H * self.F <= FEW_MATRIX_ELEMENTS
 
     def unread_bytes(self, tokens: int) -> int:
         """Bytes of expert matrices that a step of so many single tokens is expected to leave unread, for tokens that choose
@@ -197,7 +206,7 @@ class ExpertMLP(Part):
         b = 1
         while b < tokens:
             b *= 2
-        if not (b < GROUPED_FROM_TOKENS and b * self.top <= FEW_CHOICES * self.outputs and self.gate_up.layout == ops.LAYOUT_FRAG16):
+        if not (self._few_pays(b) and self.gate_up.layout == ops.LAYOUT_FRAG16):
             return 0
         none = (1.0 - self.top / self.outputs) ** tokens
         return int(none * (self.gate_up.nbytes() + self.down.nbytes()))
