@@ -139,14 +139,26 @@ __device__ __forceinline__ float value_of(const TI* rows, const HeadsArgs& a, in
   return a.bias ? x + a.bias[col] : x;
 }
 
-// One token's value head by one wave.
-template <typename TI, typename TO>
-__device__ __forceinline__ void put_values(const TI* rows, TO* v_pool, const HeadsArgs& a, int t, int hv, int pos, int page, int lane) {
-  const size_t col0 = (size_t)(a.nH + a.nKV) * a.d + (size_t)hv * a.dv;
-  TO* dst = v_pool + ((size_t)page * a.nKV + hv) * a.page_size * a.dv;
-  const int tp = pos % a.page_size;
+template <typename T> __device__ __forceinline__ void load4(const T* p, size_t i, float (&x)[4]);
+template <> __device__ __forceinline__ void load4<float>(const float* p, size_t i, float (&x)[4]) {
+  const float4 v = *reinterpret_cast<const float4*>(p + i);
+  x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
+}
+template <> __device__ __forceinline__ void load4<bf16_t>(const bf16_t* p, size_t i, float (&x)[4]) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p + i);
+  x[0] = bf16_bits_to_f32(v.x & 0xffffu); x[1] = bf16_bits_to_f32(v.x >> 16);
+  x[2] = bf16_bits_to_f32(v.y & 0xffffu); x[3] = bf16_bits_to_f32(v.y >> 16);
+}
+
+// One token's value heads [h0, h1) by one wave.  V4: four neighbouring columns a lane (rows, bias and head size allow it).
+template <typename TI, typename TO, bool V4>
+__device__ __forceinline__ void put_values(const TI* rows, TO* v_pool, const HeadsArgs& a, int t, int h0, int h1, int pos, int page, int lane) {
+  const size_t c0 = (size_t)(a.nH + a.nKV) * a.d;              // the first value column
+  TO* dst = v_pool + (size_t)page * a.nKV * a.page_size * a.dv;
+  const int tp = pos % a.page_size, begin = h0 * a.dv, end = h1 * a.dv;
   if (a.layout == 0) {
-    for (int e = lane; e < a.dv; e += 64) store_f32(dst, (size_t)tp * a.dv + e, value_of(rows, a, t, col0 + e));
+    for (int c = begin + lane; c < end; c += 64)
+      store_f32(dst, ((size_t)(c / a.dv) * a.page_size + tp) * a.dv + c % a.dv, value_of(rows, a, t, c0 + c));
     return;
   }
   if constexpr (sizeof(TO) == 2) {
@@ -156,17 +168,31 @@ __device__ __forceinline__ void put_values(const TI* rows, TO* v_pool, const Hea
       const int s = a.seq_of_token[t];
       whole = a.seq_of_token[lead] == s && a.seq_of_token[last] == s && a.positions[lead] == pos - back && a.positions[last] == pos - back + 19;
     }
+    const size_t head = (size_t)a.page_size * a.dv;
     if (!whole) {
-      for (int e = lane; e < a.dv; e += 64) store_f32(dst, v_offset(1, tp, e, a.dv), value_of(rows, a, t, col0 + e));
+      for (int c = begin + lane; c < end; c += 64)
+        store_f32(dst, (c / a.dv) * head + v_offset(1, tp, c % a.dv, a.dv), value_of(rows, a, t, c0 + c));
       return;
     }
     if (back) return;
-    for (int e = lane; e < a.dv; e += 64) {
-      float x[8];
+    constexpr int N = V4 ? 4 : 1;
+    for (int c = begin + lane * N; c < end; c += 64 * N) {
+      float x[8][N];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) x[j] = value_of(rows, a, t + (j & 3) + 16 * (j >> 2), col0 + e);
-      *reinterpret_cast<uint4*>(dst + v_offset(1, tp, e, a.dv)) =
-          uint4{pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]), pack_bf16x2(x[4], x[5]), pack_bf16x2(x[6], x[7])};
+      for (int j = 0; j < 8; ++j) {
+        const int tj = t + (j & 3) + 16 * (j >> 2);
+        if constexpr (V4) load4<TI>(rows + (size_t)tj * a.row_w, c0 + c, x[j]);
+        else x[j][0] = load_f32(rows, (size_t)tj * a.row_w + c0 + c);
+      }
+#pragma unroll
+      for (int i = 0; i < N; ++i) {
+        const float bias = a.bias ? a.bias[c0 + c + i] : 0.f;
+        float y[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[j] = x[j][i] + bias;
+        *reinterpret_cast<uint4*>(dst + (c / a.dv) * head + v_offset(1, tp, (c + i) % a.dv, a.dv)) =
+            uint4{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]), pack_bf16x2(y[4], y[5]), pack_bf16x2(y[6], y[7])};
+      }
     }
   }
 }
@@ -191,7 +217,7 @@ __global__ __launch_bounds__(256) void qkv_prepare_heads_kernel(const TI* __rest
   if (h >= a.nH + a.nKV) {
 #pragma unroll
     for (int r = 0; r < NR; ++r)
-      if (page[r] >= 0) put_values<TI, TO>(rows, v_pool, a, t0 + r, h - a.nH - a.nKV, pos[r], page[r], lane);
+      if (page[r] >= 0) put_values<TI, TO, false>(rows, v_pool, a, t0 + r, h - a.nH - a.nKV, h - a.nH - a.nKV + 1, pos[r], page[r], lane);
     return;
   }
   const bool is_q = h < a.nH;
@@ -265,10 +291,95 @@ __global__ __launch_bounds__(256) void qkv_prepare_heads_kernel(const TI* __rest
   }
 }
 
+template <typename T> __device__ __forceinline__ void load8(const T* p, float (&x)[8]);
+template <> __device__ __forceinline__ void load8<float>(const float* p, float (&x)[8]) {
+  const float4 u = *reinterpret_cast<const float4*>(p), v = *reinterpret_cast<const float4*>(p + 4);
+  x[0] = u.x; x[1] = u.y; x[2] = u.z; x[3] = u.w; x[4] = v.x; x[5] = v.y; x[6] = v.z; x[7] = v.w;
+}
+template <> __device__ __forceinline__ void load8<bf16_t>(const bf16_t* p, float (&x)[8]) {
+  const uint4 u = *reinterpret_cast<const uint4*>(p);
+  const uint32_t w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    x[2 * i] = bf16_bits_to_f32(w[i] & 0xffffu);
+    x[2 * i + 1] = bf16_bits_to_f32(w[i] >> 16);
+  }
+}
+__device__ __forceinline__ void store8(float* p, const float (&y)[8]) {
+  *reinterpret_cast<float4*>(p) = float4{y[0], y[1], y[2], y[3]};
+  *reinterpret_cast<float4*>(p + 4) = float4{y[4], y[5], y[6], y[7]};
+}
+__device__ __forceinline__ void store8(bf16_t* p, const float (&y)[8]) {
+  *reinterpret_cast<uint4*>(p) = uint4{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]), pack_bf16x2(y[4], y[5]), pack_bf16x2(y[6], y[7])};
+}
+
+// The same for heads of d = 8 LPH numbers turned in neighbouring pairs (the turned part a multiple of 8): eight numbers a
+// lane, LPH lanes a head, so that a wave takes neighbouring heads of a token and the work around a head (its place, the sum
+// over its lanes, the root) is one instruction for all of them.  The blocks beyond the first qk_blocks take the values.
+template <typename TI, typename TO, int LPH>
+__global__ __launch_bounds__(256) void qkv_prepare_wide_kernel(const TI* __restrict__ rows, TO* __restrict__ q_out, TO* __restrict__ k_pool,
+                                                               TO* __restrict__ v_pool, HeadsArgs a, int qk_blocks, int heads_a_wave) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  constexpr int d = 8 * LPH;
+  if ((int)blockIdx.x >= qk_blocks) {
+    const int per = a.nKV / heads_a_wave, item = (blockIdx.x - qk_blocks) * 4 + wave, t = item / per, hv = item % per * heads_a_wave;
+    if (t >= a.T) return;
+    const int pos = a.positions[t], page = a.block_table[(size_t)a.seq_of_token[t] * a.bt_stride + pos / a.page_size];
+    if (page >= 0 && page < a.n_pages) put_values<TI, TO, true>(rows, v_pool, a, t, hv, hv + heads_a_wave, pos, page, lane);
+    return;
+  }
+  const int n_qk = a.nH + a.nKV, item = blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  const bool on = item < a.T * n_qk;
+  const int t = on ? item / n_qk : a.T - 1, h = on ? item % n_qk : 0, e = (threadIdx.x % LPH) * 8;
+  const bool is_q = h < a.nH;
+  float x[8], w[8], c[4], sn[4];
+  load8<TI>(rows + (size_t)t * a.row_w + (size_t)h * d + e, x);
+  load8<float>(a.norm_w + (is_q ? 0 : d) + e, w);
+  const int pos = a.positions[t], half = a.R >> 1;
+  int page = 0;
+  if (!is_q) page = a.block_table[(size_t)a.seq_of_token[t] * a.bt_stride + pos / a.page_size];
+  const bool turned = e < a.R;
+  const float4 c4 = turned ? *reinterpret_cast<const float4*>(a.cos_t + (size_t)pos * half + (e >> 1)) : float4{1.f, 1.f, 1.f, 1.f};
+  const float4 s4 = turned ? *reinterpret_cast<const float4*>(a.sin_t + (size_t)pos * half + (e >> 1)) : float4{0.f, 0.f, 0.f, 0.f};
+  c[0] = c4.x; c[1] = c4.y; c[2] = c4.z; c[3] = c4.w;
+  sn[0] = s4.x; sn[1] = s4.y; sn[2] = s4.z; sn[3] = s4.w;
+  if (a.bias) {
+    float b[8];
+    load8<float>(a.bias + (size_t)h * d + e, b);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] += b[i];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) ss = fmaf(x[i], x[i], ss);
+#pragma unroll
+  for (int o = 1; o < LPH; o <<= 1) ss += __shfl_xor(ss, o, 64);
+  const float inv = 1.f / sqrtf(ss / (float)d + a.eps);
+  float y[8];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) rotate_pair(x[2 * i] * inv * w[2 * i], x[2 * i + 1] * inv * w[2 * i + 1], c[i], sn[i], y[2 * i], y[2 * i + 1]);
+  if (!on) return;
+  if (is_q) store8(q_out + ((size_t)t * a.nH + h) * d + e, y);
+  else if (page >= 0 && page < a.n_pages)
+    store8(k_pool + ((size_t)page * a.nKV + (h - a.nH)) * a.page_size * d + k_offset(a.layout, pos % a.page_size, e, d), y);
+}
+
 template <typename TI, typename TO>
 void launch_heads(const void* rows, void* q_out, void* k_pool, void* v_pool, const HeadsArgs& a, hipStream_t stream) {
   const bool vec = a.interleaved && a.d % 2 == 0 && a.row_w % 2 == 0 &&
                    (((uintptr_t)rows | (uintptr_t)q_out | (uintptr_t)k_pool | (uintptr_t)a.norm_w) & 7) == 0;
+  const uintptr_t all = (uintptr_t)rows | (uintptr_t)q_out | (uintptr_t)k_pool | (uintptr_t)a.norm_w | (uintptr_t)a.cos_t | (uintptr_t)a.sin_t | (uintptr_t)a.bias;
+  if (a.interleaved && (a.d == 64 || a.d == 128 || a.d == 256) && a.R % 8 == 0 && a.row_w % 8 == 0 && a.dv % 4 == 0 && (all & 15) == 0 &&
+      (long)a.T * (a.nH + a.nKV) < (1L << 30)) {
+    const int heads_a_wave = a.T >= 1024 && a.nKV > 0 ? a.nKV : 1;    // (few tokens: more waves)
+    const int qk_blocks = ceil_div(a.T * (a.nH + a.nKV), 256 * 8 / a.d), blocks = qk_blocks + ceil_div(a.T * (a.nKV / heads_a_wave), 4);
+#define GO(LPH) qkv_prepare_wide_kernel<TI, TO, LPH><<<blocks, 256, 0, stream>>>((const TI*)rows, (TO*)q_out, (TO*)k_pool, (TO*)v_pool, a, qk_blocks, heads_a_wave)
+    if (a.d == 64) GO(8);
+    else if (a.d == 128) GO(16);
+    else GO(32);
+#undef GO
+    return;
+  }
   const int nr = a.T >= 1024 ? 4 : 1;                           // many tokens: more loads of a wave in flight
   const dim3 g(ceil_div(a.T, nr), ceil_div(a.n_heads, 4));
 #define GO(NP, NR, VEC) qkv_prepare_heads_kernel<TI, TO, NP, NR, VEC><<<g, 256, 0, stream>>>((const TI*)rows, (TO*)q_out, (TO*)k_pool, (TO*)v_pool, a)

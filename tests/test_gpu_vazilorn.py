@@ -108,14 +108,16 @@ def _fragment_places(kp, vp, page, tp):
     ("float32", 0, 3, 3, 20, 12, 20, True, False), ("bfloat16", 0, 4, 2, 16, 24, 8, True, True), ("float32", 0, 2, 1, 7, 5, 4, True, False),
     ("bfloat16", 0, 5, 1, 136, 40, 64, False, False), ("float32", 0, 1, 1, 256, 256, 256, False, True), ("float32", 0, 6, 2, 64, 64, 0, True, False),
     ("bfloat16", 1, 6, 2, 64, 64, 64, True, False), ("bfloat16", 1, 4, 4, 128, 128, 32, True, False), ("bfloat16", 1, 2, 1, 256, 256, 96, True, True),
-    ("bfloat16", 1, 3, 1, 64, 64, 0, True, False), ("bfloat16", 1, 2, 2, 128, 128, 128, False, False)])
+    ("bfloat16", 1, 3, 1, 64, 64, 0, True, False), ("bfloat16", 1, 10, 5, 64, 64, 24, True, True), ("float32", 0, 4, 2, 128, 96, 64, True, True),
+    ("bfloat16", 0, 2, 1, 256, 44, 256, True, False), ("bfloat16", 1, 2, 2, 128, 128, 128, False, False)])
+@pytest.mark.parametrize("spare", [4, 8])                    # further columns of a row: the wide loads want rows of whole 32-byte units
 @pytest.mark.parametrize("starts,lens", [([60, 3], [10, 70]), ([0, 17, 5], [700, 380, 1]), ([0], [64]), ([31, 0, 100, 9], [1, 1, 1, 1])])
-def test_norm_a_head_rotation_and_cache_write(dtype, layout, H, G, d, dv, R, interleaved, bias, starts, lens):
+def test_norm_a_head_rotation_and_cache_write(dtype, layout, H, G, d, dv, R, interleaved, bias, starts, lens, spare):
     """Every head divided by its own root mean square and weighted, turned, and put with its value into scattered pages, for
     sequences of one step that start at other positions than 0; nothing beside their own places is touched."""
     act, page, eps, T = Precision.of(dtype).act, 64, 1e-3, sum(lens)
     width = H * d + G * (d + dv)
-    rows, bv, wn = rnd(T, width + 4, seed=1), rnd(width, seed=2, scale=0.5), 1.0 + rnd(2, d, seed=3, scale=0.3)
+    rows, bv, wn = rnd(T, width + spare, seed=1), rnd(width, seed=2, scale=0.5), 1.0 + rnd(2, d, seed=3, scale=0.3)
     pos = torch.cat([torch.arange(s, s + n) for s, n in zip(starts, lens)])
     seq = torch.cat([torch.full((n,), i) for i, n in enumerate(lens)])
     per = int(pos.max()) // page + 1
@@ -162,8 +164,8 @@ def test_norm_a_head_rotation_and_cache_write(dtype, layout, H, G, d, dv, R, int
     assert int((kp == 9.0).sum()) == (n_pages * page - T) * G * d
     # queries alone, from rows that hold no k and v
     q2 = torch.empty_like(q_out)
-    ops.qkv_prepare(rows[:, :H * d + 2].contiguous().to(DEV), b_dev, q2, None, None, i32(pos.tolist()), None, None, **common)
-    assert max_err(q2, q_out) == 0.0
+    ops.qkv_prepare(rows[:, :H * d + spare // 2].contiguous().to(DEV), b_dev, q2, None, None, i32(pos.tolist()), None, None, **common)
+    assert max_err(q2, q_out) < tol * big(q)
     if layout:
         with pytest.raises(ops.HipLibraryError):
             ops.qkv_prepare(rows.to(DEV), b_dev, q_out, kp, vp, i32(pos.tolist()), i32(seq.tolist()), bt.to(DEV), kv_layout=layout,
