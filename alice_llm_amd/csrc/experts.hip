@@ -444,8 +444,12 @@ __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
     auto rows = [&](int s) {
       const bf16_t* xr = a.x + (size_t)min(token[s], a.T - 1) * a.W;
 #pragma unroll
-      for (int u = 0; u < N; ++u)                          // a row's last, partial k-tile: the weights are zero there
-        b[u] = *reinterpret_cast<const u32x4*>(xr + min((kt0 + 4 * u) * 32 + g * 8, a.W - 8));
+      for (int u = 0; u < N; ++u) b[u] = u32x4{0u, 0u, 0u, 0u};
+      if (s * 16 + c < n_used) {                           // (no row is read for a column without a token)
+#pragma unroll
+        for (int u = 0; u < N; ++u)                        // a row's last, partial k-tile: the weights are zero there
+          b[u] = *reinterpret_cast<const u32x4*>(xr + min((kt0 + 4 * u) * 32 + g * 8, a.W - 8));
+      }
     };
     rows(0);
 #pragma unroll
@@ -493,12 +497,14 @@ __global__ __launch_bounds__(256) void expert_few_gate_up_kernel(FewArgs a) {
   }
 }
 
+// 16 outputs of every splits-th chosen expert: again the expert's tokens side by side; a wave adds each expert's products to
+// its own sums a token in LDS, and the four waves' sums meet at the end.
 template <int RS>
 __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
   __shared__ unsigned short list[MAX_EXPERTS + 1];
   __shared__ unsigned long long users[MAX_EXPERTS + 1];
   __shared__ int n_list;
-  __shared__ f32x4 part[4][RS][64];
+  __shared__ f32x4 sums[4][16 * RS][4];                   // [wave][token][four of the 16 outputs]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, c = lane & 15;
   const int n0 = blockIdx.x * 16, z = blockIdx.y, n_exp = a.E + (a.Fs > 0 ? 1 : 0), row = a.E * a.F + a.Fs;
   if (wave == 0) {                                        // the chosen experts in their order
@@ -527,63 +533,64 @@ __global__ __launch_bounds__(256) void expert_few_down_kernel(FewArgs a) {
     }
     if (lane == 0) n_list = n;
   }
+#pragma unroll
+  for (int s = 0; s < RS; ++s) sums[wave][s * 16 + (lane >> 2)][lane & 3] = f32x4{0.f, 0.f, 0.f, 0.f};
   __syncthreads();
   const int KT = (a.E * a.F + 31) / 32, KTS = (a.Fs + 31) / 32;
-  f32x4 acc[RS];
-#pragma unroll
-  for (int s = 0; s < RS; ++s) acc[s] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const unsigned long long below = (1ull << lane) - 1ull;
   for (int i = z; i < n_list; i += a.splits) {
     const int e = list[i];
     const unsigned long long who = users[i];
-    const bool shared = e == a.E;
+    const bool shared = e == a.E, mine = (who >> lane) & 1ull;
+    const int n_used = __popcll(who), sets = RS == 1 ? 1 : (n_used + 15) >> 4;
     const int kts = (shared ? a.Fs : a.F) / 32;           // F and Fs are multiples of 32: an expert's k-tiles are its own
     const bf16_t* wd = (shared ? a.shared_down + (size_t)(n0 / 16) * KTS * 512 : a.down + ((size_t)(n0 / 16) * KT + e * a.F / 32) * 512) + lane * 8;
-    bool use[RS], on[RS];
-    const bf16_t* mr[RS];
+    const int token_at = __builtin_amdgcn_ds_permute((mine ? __popcll(who & below) : n_used + __popcll(~who & below)) * 4, lane);
+    int token[RS];
+    f32x4 acc[RS];
 #pragma unroll
     for (int s = 0; s < RS; ++s) {
-      const int t = s * 16 + c;
-      use[s] = (who >> t) & 1ull;
-      on[s] = __ballot(use[s]) != 0ull;
-      mr[s] = a.mid + (size_t)min(t, a.T - 1) * row + e * a.F + g * 8;
+      token[s] = __shfl(token_at, s * 16 + c, 64);
+      acc[s] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    auto burst = [&](auto count, int kt0) {               // as above; tokens that do not use the expert count as zero
+    auto burst = [&](auto count, int kt0) {               // as above
       constexpr int N = decltype(count)::value;
-      u32x4 v[N], b[N][RS];
+      u32x4 v[N], b[N];
+      auto rows = [&](int s) {
+        const bf16_t* mr = a.mid + (size_t)min(token[s], a.T - 1) * row + e * a.F + g * 8;
 #pragma unroll
-      for (int s = 0; s < RS; ++s) {
+        for (int u = 0; u < N; ++u) b[u] = u32x4{0u, 0u, 0u, 0u};
+        if (s * 16 + c < n_used) {
 #pragma unroll
-        for (int u = 0; u < N; ++u) b[u][s] = u32x4{0u, 0u, 0u, 0u};
-        if (use[s]) {
-#pragma unroll
-          for (int u = 0; u < N; ++u) b[u][s] = *reinterpret_cast<const u32x4*>(mr[s] + (kt0 + 4 * u) * 32);
+          for (int u = 0; u < N; ++u) b[u] = *reinterpret_cast<const u32x4*>(mr + (kt0 + 4 * u) * 32);
         }
-      }
+      };
+      rows(0);
 #pragma unroll
       for (int u = 0; u < N; ++u) v[u] = *reinterpret_cast<const u32x4*>(wd + (size_t)(kt0 + 4 * u) * 512);
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int u = 0; u < N; ++u)
+      for (int s = 0; s < RS; ++s) {
+        if (s >= sets) break;                              // (the same for the whole block)
+        if (s > 0) rows(s);
 #pragma unroll
-        for (int s = 0; s < RS; ++s) {
-          if (RS > 1 && !on[s]) continue;
-          acc[s] = mfma16(v[u], b[u][s], acc[s]);
-        }
+        for (int u = 0; u < N; ++u) acc[s] = mfma16(v[u], b[u], acc[s]);
+      }
     };
-    constexpr int U = RS == 4 ? 4 : 8;
+    constexpr int U = 8;
     int kt = wave;
     for (; kt + 4 * (U - 1) < kts; kt += 4 * U) burst(std::integral_constant<int, U>{}, kt);
     if (kt + 4 * 3 < kts) { burst(std::integral_constant<int, 4>{}, kt); kt += 16; }
     if (kt + 4 < kts) { burst(std::integral_constant<int, 2>{}, kt); kt += 8; }
     if (kt < kts) burst(std::integral_constant<int, 1>{}, kt);
-  }
 #pragma unroll
-  for (int s = 0; s < RS; ++s) part[wave][s][lane] = acc[s];
+    for (int s = 0; s < RS; ++s)
+      if (s * 16 + c < n_used) sums[wave][token[s]][g] += acc[s];      // (n_used <= T <= 16 RS: no set is left out)
+  }
   __syncthreads();
-  for (int s = wave; s < RS; s += 4) {
-    const int t = s * 16 + c, n = n0 + g * 4;
-    if (t >= a.T) continue;
-    f32x4 o = (part[0][s][lane] + part[1][s][lane]) + (part[2][s][lane] + part[3][s][lane]);
+  for (int j = tid; j < a.T * 4; j += 256) {
+    const int t = j >> 2, q = j & 3, n = n0 + q * 4;
+    f32x4 o = (sums[0][t][q] + sums[1][t][q]) + (sums[2][t][q] + sums[3][t][q]);
     if (z == 0 && a.side) {
       const float id = a.side[2 * (size_t)t];
 #pragma unroll
