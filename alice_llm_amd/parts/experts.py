@@ -42,13 +42,11 @@ from .linear import Linear
 
 _GATED = {"gelu_tanh": 0.0, "silu": ops.GATED_SILU, "swish_limited": None}
 # Which of the ways (bfloat16, sizes that suit the tiles), measured with choices spread evenly over 8 to 128 experts.  Steps of at
-# most 32 tokens read the chosen experts only.  Steps of 33 to 64 tokens do so too if there are at most FEW_CHOICES (token,
-# expert) pairs to a router output (beyond, most tokens meet most experts) and an expert's matrices have at most
-# FEW_MATRIX_ELEMENTS numbers each.  Else steps of GROUPED_FROM_TOKENS and more take the grouped products, and smaller ones one
-# pass over all experts' matrices.  (At most 32 tokens have at most 32 pairs to an output, twice FEW_CHOICES.)
+# most 64 tokens read the chosen experts only where there are at most FEW_CHOICES (token, expert) pairs to a router output
+# (beyond, most tokens meet most experts).  Else steps of GROUPED_FROM_TOKENS and more take the grouped products, and smaller
+# ones one pass over all experts' matrices.
 GROUPED_FROM_TOKENS = 64
-FEW_CHOICES = 16.0
-FEW_MATRIX_ELEMENTS = 1 << 23
+FEW_CHOICES = 24.0
 MIDDLE_ELEMENTS = 1 << 28      # the most middle activations (tokens x experts x their width) that a step holds at a time
 
 
@@ -196,9 +194,7 @@ class ExpertMLP(Part):
                 and ops.expert_products_supported(x.dtype, self.H, self.F))
 
     def _few_pays(self, n: int) -> bool:
-        if n <= 32:
-            return n * self.top <= 2 * FEW_CHOICES * self.outputs
-        return n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs and self.H * self.F <= FEW_MATRIX_ELEMENTS
+        return n <= ops.EXPERT_FEW_MAX_TOKENS and n * self.top <= FEW_CHOICES * self.outputs
 
     def unread_bytes(self, tokens: int) -> int:
         """Bytes of expert matrices that a step of so many single tokens is expected to leave unread, for tokens that choose
