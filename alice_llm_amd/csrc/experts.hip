@@ -26,8 +26,8 @@
 // Steps of few tokens read every chosen expert's matrices once and do little else (expert_few_*): a block of the first
 // kernel takes one expert and 16 of its middle columns, and ends at once if no token of the step chose it; its four waves
 // share the inner dimension and meet in LDS.  A block of the second takes 16 outputs and every splits-th of the chosen
-// experts, with the tokens as the columns of all its products (zeros where a token did not choose the expert), and leaves
-// partial sums for the residual add.  The shared expert is one more expert with sizes of its own, chosen by every token,
+// experts, adds each one's products to its sums a token, and leaves partial sums for the residual add.  In both the tokens that
+// chose the expert stand side by side as the products' columns, 16 to a set.  The shared expert is one more expert with sizes of its own, chosen by every token,
 // and the identity experts' share is added by the first split.  Which experts are chosen is read on the device.
 #include "linear_mfma.h"
 

@@ -174,5 +174,5 @@ def write_safetensors(path: str, specs: Sequence[Tuple[str, torch.dtype, Sequenc
                 raise WeightFileError(f"producer gave {tuple(t.shape)} {t.dtype} for '{name}', "
                                       f"declared {tuple(shape)} {dt}")
             t = t.detach().contiguous().cpu()
-            f.write(t.view(torch.uint8).numpy().tobytes() if t.numel() else b"")
+            f.write(t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")
     os.replace(tmp, path)

@@ -126,6 +126,19 @@ def test_tensor_names_shapes_and_cache_needs():
         assert set(tensors) == set(CausalLM(cfg.plan(), Precision.of("bfloat16"), "cpu").param_specs()), name
 
 
+def test_random_folder_holds_every_tensor_and_runs(tmp_path):
+    """The random-weights mode: names, shapes (a number without dimensions too), norm weights around one, logits of order one."""
+    raw = VAZILORN["vz-a"]()
+    alice.write_random_model(str(tmp_path), dict(raw), seed=3)
+    plain = P.PlainVazilorn.from_folder(str(tmp_path))
+    specs = CausalLM(alice.config_from_dict(raw).plan(), Precision.of("float32"), "cpu").param_specs()
+    assert {k: tuple(v.shape) for k, v in plain.tensors.items()} == {k: tuple(v.shape) for k, v in specs.items()}
+    assert abs(float(plain.tensors["l0.norm1"].mean()) - 1.0) < 0.1 and 0.2 < float(plain.tensors["l0.norm1.alpha"]) < 0.8
+    assert abs(float(plain.tensors["l0.mix.q.norm"].mean()) - 1.0) < 0.2 and float(plain.tensors["embed"].std()) > 0.8
+    logits = plain.forward(random_tokens(97, 12, 1))
+    assert bool(torch.isfinite(logits).all()) and float(logits.std()) > 0.01
+
+
 # ------------------------------------------------------------------ the plain implementation's own invariants
 
 def test_dynamic_tanh_acts_on_every_element_by_itself():
